@@ -195,6 +195,7 @@ void moe_align(Tensor ids, Tensor w, int64_t T, int64_t k, int64_t e0, int64_t E
 
 // mode 0: out [M, F] = act(A[sorted_tok] @ W_e[:F]^T) * (A[sorted_tok] @ W_e[F:]^T)
 // mode 1: out [M, N] = (A @ W_e^T) * sorted_w
+// mode 2 (act 3): out [M, N] = gelu(A[sorted_tok] @ W_e^T), erf gelu, N % 4 == 0
 // act 2: clamped GLU (limit, alpha); in_weight: the routing weight scales the gate | up accumulators (the
 // expert's input) and the down GEMM is left unscaled
 void moe_gemm(Tensor A, Tensor W, Tensor sorted_tok, Tensor sorted_w, Tensor tiles, int64_t mt,
@@ -204,7 +205,7 @@ void moe_gemm(Tensor A, Tensor W, Tensor sorted_tok, Tensor sorted_w, Tensor til
   CHECK_DEV(sorted_tok); CHECK_DT(sorted_tok, at::kInt);
   CHECK_DEV(sorted_w); CHECK_DT(sorted_w, at::kFloat);
   CHECK_DEV(tiles); CHECK_DT(tiles, at::kInt);
-  TORCH_CHECK(mode == 0 || mode == 1);
+  TORCH_CHECK(mode >= 0 && mode <= 2 && (mode == 2) == (act == 3), "moe_gemm: mode 2 is act 3");
   TORCH_CHECK(bm == 64 || bm == 128);
   TORCH_CHECK(W.dim() == 3 && A.dim() == 2 && out.dim() == 2 && A.stride(1) == 1);
   const int64_t K = W.size(2);
@@ -222,6 +223,9 @@ void moe_gemm(Tensor A, Tensor W, Tensor sorted_tok, Tensor sorted_w, Tensor til
     p.F = (int)(W.size(1) / 2);
     TORCH_CHECK(out.size(1) == p.F, "moe_gemm: out must be [M, F]");
     p.nt = p.F / 128;
+  } else if (mode == 2) {
+    TORCH_CHECK(W.size(1) % 4 == 0 && out.size(1) == W.size(1), "moe_gemm: out must be [M, N], N % 4 == 0");
+    p.nt = (int)((W.size(1) + 255) / 256);
   } else {
     TORCH_CHECK(W.size(1) % 256 == 0 && out.size(1) == W.size(1), "moe_gemm: out must be [M, N], N % 256 == 0");
     p.F = 0;
@@ -235,7 +239,7 @@ void moe_gemm(Tensor A, Tensor W, Tensor sorted_tok, Tensor sorted_w, Tensor til
   p.tiles = tiles.data_ptr<int32_t>();
   p.out = bfp(out);
   p.ldo = out.stride(0);
-  TORCH_CHECK(act >= 0 && act <= 2);
+  TORCH_CHECK(act >= 0 && act <= 3);
   p.act = (int)act;
   p.limit = (float)limit;
   p.alpha = (float)alpha;
@@ -258,6 +262,7 @@ void moe_route_scores(Tensor logits, int64_t k, int64_t score, bool renorm, Tens
 // the grouped GEMMs of moe_gemm on fp32-accumulating VALU tiles (bf16 or fp32, any sizes; 64-row M tiles).
 // mode 0: out [M, F] = clamped_glu(s (A[sorted_tok] W_e[:F]^T), s (A[sorted_tok] W_e[F:]^T)), s = sorted_w or 1
 // mode 1: out [M, N] = (A W_e^T) * (sorted_w or 1)
+// mode 2: out [M, N] = gelu(A[sorted_tok] W_e^T), erf gelu
 void moe_gemm_rows(Tensor A, Tensor W, Tensor sorted_tok, Tensor sorted_w, Tensor tiles, int64_t mt, Tensor out,
                    int64_t mode, double limit, double alpha, bool use_weight, double shift) {
   const bool f32 = act_f32(A);
@@ -266,7 +271,7 @@ void moe_gemm_rows(Tensor A, Tensor W, Tensor sorted_tok, Tensor sorted_w, Tenso
   CHECK_DEV(sorted_tok); CHECK_DT(sorted_tok, at::kInt);
   CHECK_DEV(sorted_w); CHECK_DT(sorted_w, at::kFloat);
   CHECK_DEV(tiles); CHECK_DT(tiles, at::kInt);
-  TORCH_CHECK(mode == 0 || mode == 1);
+  TORCH_CHECK(mode >= 0 && mode <= 2);
   TORCH_CHECK(W.dim() == 3 && A.dim() == 2 && out.dim() == 2 && A.stride(1) == 1 && A.size(1) == W.size(2));
   TORCH_CHECK(tiles.numel() >= 3 * mt && sorted_tok.numel() >= out.size(0) && sorted_w.numel() >= out.size(0));
   nga::MoeRowsParams p{};
@@ -280,7 +285,7 @@ void moe_gemm_rows(Tensor A, Tensor W, Tensor sorted_tok, Tensor sorted_w, Tenso
     TORCH_CHECK(W.size(1) % 2 == 0 && out.size(1) == W.size(1) / 2, "moe_gemm_rows: out must be [M, F]");
     p.F = (int)(W.size(1) / 2);
   } else {
-    TORCH_CHECK(out.size(1) == W.size(1) && A.size(0) >= out.size(0), "moe_gemm_rows: out must be [M, N]");
+    TORCH_CHECK(out.size(1) == W.size(1) && (mode == 2 || A.size(0) >= out.size(0)), "moe_gemm_rows: out must be [M, N]");
     p.N = (int)W.size(1);
   }
   p.sorted_tok = sorted_tok.data_ptr<int32_t>();
@@ -295,19 +300,20 @@ void moe_gemm_rows(Tensor A, Tensor W, Tensor sorted_tok, Tensor sorted_w, Tenso
   nga::launch_moe_gemm_rows(p, (int)mode, f32, cur_stream(out));
 }
 
-void moe_route_grouped(Tensor logits, Tensor correction, int64_t k, int64_t groups, int64_t keep, double scale,
+const float* opt_f32(const c10::optional<Tensor>& t, int64_t n, const char* what);
+
+void moe_route_grouped(Tensor logits, c10::optional<Tensor> correction, int64_t k, int64_t groups, int64_t keep, double scale,
                        Tensor ids, Tensor w) {
   CHECK_DEV(logits); CHECK_DT(logits, at::kFloat);
-  CHECK_DEV(correction); CHECK_DT(correction, at::kFloat); CHECK_CONTIG(correction);
   TORCH_CHECK(logits.dim() == 2 && logits.stride(1) == 1, "moe_route_grouped: logits must be [T, E]");
   const int64_t T = logits.size(0), E = logits.size(1);
-  TORCH_CHECK(correction.numel() == E && E >= 1 && E <= 512, "moe_route_grouped: one correction per expert, E <= 512");
+  TORCH_CHECK(E >= 1 && E <= 512, "moe_route_grouped: E <= 512");
   TORCH_CHECK(groups >= 1 && groups <= 64 && E % groups == 0 && keep >= 1 && keep <= groups && k >= 1 &&
               k <= keep * (E / groups), "moe_route_grouped: groups / keep / k do not fit the experts");
   CHECK_DEV(ids); CHECK_DT(ids, at::kInt); CHECK_DEV(w); CHECK_DT(w, at::kFloat);
   TORCH_CHECK(ids.is_contiguous() && w.is_contiguous() && ids.numel() >= T * k && w.numel() >= T * k);
-  nga::launch_moe_route_grouped(logits.data_ptr<float>(), logits.stride(0), correction.data_ptr<float>(), (int)T, (int)E,
-                                (int)k, (int)groups, (int)keep, (float)scale, ids.data_ptr<int32_t>(),
+  nga::launch_moe_route_grouped(logits.data_ptr<float>(), logits.stride(0), opt_f32(correction, E, "correction"), (int)T,
+                                (int)E, (int)k, (int)groups, (int)keep, (float)scale, ids.data_ptr<int32_t>(),
                                 w.data_ptr<float>(), cur_stream(logits));
 }
 
@@ -1288,7 +1294,7 @@ void residual_add_rmsnorm(Tensor x, Tensor y, c10::optional<Tensor> w, double ep
   const bool f32 = act_f32(y);
   const int64_t H = x.size(1);
   TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && y.size(0) == x.size(0) && y.size(1) == H && y.stride(1) == 1);
-  TORCH_CHECK(w.has_value() == out.has_value(), "residual_add_rmsnorm: a norm weight and its output come together");
+  TORCH_CHECK(!w.has_value() || out.has_value(), "residual_add_rmsnorm: a norm weight needs an output");
   void* op = nullptr;
   if (out.has_value()) {
     CHECK_CONTIG(*out);
@@ -1367,8 +1373,10 @@ void latent_rope_cache(Tensor proj, Tensor pos, Tensor slots, c10::optional<Tens
   nga::launch_latent_rope_cache(p, T, f32, cur_stream(proj));
 }
 
-void group_rmsnorm(Tensor out, Tensor x, Tensor w, int64_t groups, double eps, c10::optional<Tensor> gate) {
-  CHECK_F32(x); CHECK_F32(w); CHECK_CONTIG(out);
+void group_rmsnorm(Tensor out, Tensor x, Tensor w, int64_t groups, double eps, c10::optional<Tensor> gate,
+                   bool gate_silu) {
+  CHECK_F32(x); CHECK_F32(w); CHECK_CONTIG(x);
+  TORCH_CHECK(out.dim() == 2 && out.stride(1) == 1);
   const bool f32 = act_f32(out);
   TORCH_CHECK(x.dim() == 2 && out.sizes() == x.sizes() && groups > 0 && x.size(1) % groups == 0 &&
               (w.numel() == x.size(1) / groups || w.numel() == x.size(1)));
@@ -1381,8 +1389,8 @@ void group_rmsnorm(Tensor out, Tensor x, Tensor w, int64_t groups, double eps, c
     gp = gate->data_ptr();
     gs = gate->stride(0);
   }
-  nga::launch_group_rmsnorm(out.data_ptr(), x.data_ptr<float>(), w.data_ptr<float>(),
-                            groups > 1 && w.numel() == x.size(1), gp, gs, x.size(0), (int)groups,
+  nga::launch_group_rmsnorm(out.data_ptr(), out.stride(0), x.data_ptr<float>(), w.data_ptr<float>(),
+                            groups > 1 && w.numel() == x.size(1), gp, gs, gate_silu, x.size(0), (int)groups,
                             (int)(x.size(1) / groups), (float)eps, f32, cur_stream(x));
 }
 
@@ -1568,8 +1576,7 @@ struct SoftmaxArgs {
 SoftmaxArgs check_softmax_args(const Tensor& out, const Tensor& q, const c10::optional<Tensor>& gate, const Tensor& kc,
                                const Tensor& vc, int64_t H, int64_t G, int64_t dk, int64_t dv, int64_t window,
                                int64_t maps, bool v_in_k = false) {
-  CHECK_CONTIG(out);
-  TORCH_CHECK(out.is_cuda() && out.scalar_type() == q.scalar_type());
+  TORCH_CHECK(out.is_cuda() && out.scalar_type() == q.scalar_type() && out.stride(1) == 1);
   const int64_t T = q.size(0);
   TORCH_CHECK(maps == 1 || maps == 2, "softmax_attention: one or two maps per head");
   TORCH_CHECK(q.dim() == 2 && q.stride(1) == 1 && q.size(1) == H * maps * dk, "q must be [T, H * maps * dk] rows");
@@ -1597,17 +1604,18 @@ SoftmaxArgs check_softmax_args(const Tensor& out, const Tensor& q, const c10::op
 void softmax_attention(Tensor out, Tensor q, c10::optional<Tensor> gate, Tensor kc, Tensor vc, Tensor block_tables,
                        Tensor tok_seq, Tensor pos, int64_t H, int64_t G, int64_t dk, int64_t dv, double scale,
                        int64_t window, int64_t maps, double lam, double unit_eps, double out_scale, bool v_in_k,
-                       double softcap) {
+                       double softcap, int64_t chunk, double sink) {
+  TORCH_CHECK(chunk >= 0);
   const bool f32 = act_f32(q);
   CHECK_I32(block_tables); CHECK_I32(tok_seq); CHECK_I32(pos);
   const SoftmaxArgs a = check_softmax_args(out, q, gate, kc, vc, H, G, dk, dv, window, maps, v_in_k);
   const int64_t T = q.size(0);
   TORCH_CHECK(tok_seq.numel() == T && pos.numel() == T && block_tables.dim() == 2);
-  nga::launch_softmax_attention(out.data_ptr(), q.data_ptr(), q.stride(0), a.gp, a.gs, kc.data_ptr(), vc.data_ptr(),
+  nga::launch_softmax_attention(out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), a.gp, a.gs, kc.data_ptr(), vc.data_ptr(),
                                 block_tables.data_ptr<int32_t>(), (int)block_tables.size(1),
                                 tok_seq.data_ptr<int32_t>(), pos.data_ptr<int32_t>(), T, (int)H, (int)G, (int)dk,
                                 (int)dv, (float)scale, (int)window, (int)maps, (float)lam, (float)unit_eps,
-                                (float)out_scale, v_in_k, (float)softcap, f32, cur_stream(q));
+                                (float)out_scale, v_in_k, (float)softcap, (int)chunk, (float)sink, f32, cur_stream(q));
 }
 
 // prompt portions on the MFMA kernel (bf16): sequence b owns rows [cu_q[b], cu_q[b + 1]) of q / gate / out,
@@ -1615,27 +1623,33 @@ void softmax_attention(Tensor out, Tensor q, c10::optional<Tensor> gate, Tensor 
 void softmax_attention_prefill(Tensor out, Tensor q, c10::optional<Tensor> gate, Tensor kc, Tensor vc,
                                Tensor block_tables, Tensor cu_q, Tensor ctx_lens, int64_t max_q_len, int64_t H,
                                int64_t G, int64_t dk, int64_t dv, double scale, int64_t window, int64_t maps, double lam,
-                               double unit_eps, double out_scale, bool v_in_k, double softcap) {
-  CHECK_BF16(q); CHECK_BF16(out); CHECK_I32(block_tables); CHECK_I32(cu_q); CHECK_I32(ctx_lens);
+                               double unit_eps, double out_scale, bool v_in_k, double softcap, int64_t chunk, double sink) {
+  TORCH_CHECK(chunk >= 0);
+  CHECK_BF16(q); CHECK_BF16(out);
+  TORCH_CHECK(out.stride(0) % 4 == 0 && (uintptr_t)out.data_ptr() % 8 == 0, "output rows must be 8-B aligned");
+  CHECK_I32(block_tables); CHECK_I32(cu_q); CHECK_I32(ctx_lens);
   const SoftmaxArgs a = check_softmax_args(out, q, gate, kc, vc, H, G, dk, dv, window, maps, v_in_k);
   TORCH_CHECK(nga::softmax_attention_mfma_supported((int)dk, (int)dv, (int)(H / G), (int)maps),
               "softmax_attention_prefill: head sizes the MFMA kernel does not take");
   TORCH_CHECK(q.stride(0) % 8 == 0 && (uintptr_t)q.data_ptr() % 16 == 0, "q rows must be 16-B aligned");
   const int64_t B = ctx_lens.numel();
   TORCH_CHECK(cu_q.numel() == B + 1 && block_tables.dim() == 2 && block_tables.size(0) >= B && max_q_len >= 0);
-  nga::launch_softmax_attention_mfma(bfp(out), bfp(q), q.stride(0), (const uint16_t*)a.gp, a.gs, bfp(kc), bfp(vc),
+  nga::launch_softmax_attention_mfma(bfp(out), out.stride(0), bfp(q), q.stride(0), (const uint16_t*)a.gp, a.gs, bfp(kc), bfp(vc),
                                      block_tables.data_ptr<int32_t>(), (int)block_tables.size(1),
                                      cu_q.data_ptr<int32_t>(), ctx_lens.data_ptr<int32_t>(), (int)B, (int)max_q_len,
                                      (int)H, (int)G, (int)dk, (int)dv, (float)scale, (int)window, (int)maps, (float)lam,
-                                     (float)unit_eps, (float)out_scale, v_in_k, (float)softcap, cur_stream(q));
+                                     (float)unit_eps, (float)out_scale, v_in_k, (float)softcap, (int)chunk, (float)sink, cur_stream(q));
 }
 
 // single-token rows on the MFMA kernel (bf16): ws is the fp32 partial workspace [T, H, maps, parts, dv + 4]
 void softmax_attention_decode(Tensor out, Tensor ws, int64_t parts, Tensor q, c10::optional<Tensor> gate, Tensor kc,
                               Tensor vc, Tensor block_tables, Tensor tok_seq, Tensor pos, int64_t H, int64_t G,
                               int64_t dk, int64_t dv, double scale, int64_t window, int64_t maps, double lam,
-                              double unit_eps, double out_scale, bool v_in_k, double softcap) {
-  CHECK_BF16(q); CHECK_BF16(out); CHECK_F32(ws); CHECK_I32(block_tables); CHECK_I32(tok_seq); CHECK_I32(pos);
+                              double unit_eps, double out_scale, bool v_in_k, double softcap, int64_t chunk, double sink) {
+  TORCH_CHECK(chunk >= 0);
+  CHECK_BF16(q); CHECK_BF16(out);
+  TORCH_CHECK(out.stride(0) % 4 == 0 && (uintptr_t)out.data_ptr() % 8 == 0, "output rows must be 8-B aligned");
+  CHECK_F32(ws); CHECK_I32(block_tables); CHECK_I32(tok_seq); CHECK_I32(pos);
   const SoftmaxArgs a = check_softmax_args(out, q, gate, kc, vc, H, G, dk, dv, window, maps, v_in_k);
   TORCH_CHECK(nga::softmax_attention_mfma_supported((int)dk, (int)dv, (int)(H / G), (int)maps),
               "softmax_attention_decode: head sizes the MFMA kernel does not take");
@@ -1644,11 +1658,143 @@ void softmax_attention_decode(Tensor out, Tensor ws, int64_t parts, Tensor q, c1
   TORCH_CHECK(parts >= 1 && parts <= 64 && ws.numel() >= T * H * maps * parts * (dv + 4) &&
               (uintptr_t)ws.data_ptr() % 16 == 0);
   TORCH_CHECK(tok_seq.numel() == T && pos.numel() == T && block_tables.dim() == 2);
-  nga::launch_softmax_decode_mfma(bfp(out), ws.data_ptr<float>(), (int)parts, bfp(q), q.stride(0),
+  nga::launch_softmax_decode_mfma(bfp(out), out.stride(0), ws.data_ptr<float>(), (int)parts, bfp(q), q.stride(0),
                                   (const uint16_t*)a.gp, a.gs, bfp(kc), bfp(vc), block_tables.data_ptr<int32_t>(),
                                   (int)block_tables.size(1), tok_seq.data_ptr<int32_t>(), pos.data_ptr<int32_t>(), T,
                                   (int)H, (int)G, (int)dk, (int)dv, (float)scale, (int)window, (int)maps, (float)lam,
-                                  (float)unit_eps, (float)out_scale, v_in_k, (float)softcap, cur_stream(q));
+                                  (float)unit_eps, (float)out_scale, v_in_k, (float)softcap, (int)chunk, (float)sink, cur_stream(q));
+}
+
+// ------------------------------------------------------------------ bigram embedding, token gate, short convolution, delta rules
+void bigram_embed(Tensor x, Tensor ids, Tensor embed, Tensor table, Tensor src, Tensor prev, int64_t mul_prev,
+                  int64_t mul_cur, c10::optional<Tensor> save) {
+  CHECK_F32(x); CHECK_CONTIG(x); CHECK_I32(ids); CHECK_I32(src); CHECK_I32(prev);
+  const bool f32 = act_f32(embed);
+  CHECK_CONTIG(embed); CHECK_CONTIG(table);
+  const int64_t T = x.size(0), H = x.size(1);
+  TORCH_CHECK(x.dim() == 2 && embed.dim() == 2 && table.dim() == 2 && embed.size(1) == H && table.size(1) == H &&
+              table.size(0) >= 2 && table.is_cuda() && table.scalar_type() == embed.scalar_type());
+  TORCH_CHECK(ids.numel() == T && src.numel() == T && mul_prev >= 0 && mul_cur >= 0);
+  const int32_t* sp = nullptr;
+  if (save.has_value()) {
+    CHECK_I32(*save);
+    TORCH_CHECK(save->numel() == T, "bigram_embed: save takes one slot per row");
+    sp = save->data_ptr<int32_t>();
+  }
+  nga::launch_bigram_embed(x.data_ptr<float>(), ids.data_ptr<int32_t>(), embed.data_ptr(), table.data_ptr(),
+                           src.data_ptr<int32_t>(), prev.data_ptr<int32_t>(), mul_prev, mul_cur, sp, T, (int)H,
+                           (int)embed.size(0), (int)(table.size(0) - 1), f32, cur_stream(x));
+}
+
+void token_save(Tensor prev, Tensor ids, Tensor last_row, Tensor slot) {
+  CHECK_I32(prev); CHECK_I32(ids); CHECK_I32(last_row); CHECK_I32(slot);
+  TORCH_CHECK(last_row.numel() == slot.numel());
+  nga::launch_token_save(prev.data_ptr<int32_t>(), ids.data_ptr<int32_t>(), last_row.data_ptr<int32_t>(),
+                         slot.data_ptr<int32_t>(), (int)slot.numel(), cur_stream(prev));
+}
+
+void gelu_gate_rows(Tensor out, Tensor z, Tensor ids, Tensor table, int64_t off) {
+  const bool f32 = act_f32(z);
+  CHECK_CONTIG(out); CHECK_I32(ids); CHECK_CONTIG(table);
+  TORCH_CHECK(z.dim() == 2 && z.stride(1) == 1 && out.is_cuda() && out.scalar_type() == z.scalar_type() &&
+              out.sizes() == z.sizes() && ids.numel() == z.size(0));
+  TORCH_CHECK(table.is_cuda() && table.scalar_type() == z.scalar_type() && table.dim() == 2 && off >= 0 &&
+              off + z.size(1) <= table.size(1), "gelu_gate_rows: columns outside the table");
+  nga::launch_gelu_gate_rows(out.data_ptr(), z.data_ptr(), z.stride(0), ids.data_ptr<int32_t>(),
+                             (const char*)table.data_ptr() + off * table.element_size(), table.stride(0), z.size(0),
+                             (int)z.size(1), (int)table.size(0), f32, cur_stream(z));
+}
+
+void tanh_rows(Tensor out, Tensor x) {
+  const bool f32 = act_f32(x);
+  CHECK_CONTIG(out);
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && out.is_cuda() && out.scalar_type() == x.scalar_type() &&
+              out.sizes() == x.sizes());
+  nga::launch_tanh_rows(out.data_ptr(), x.data_ptr(), x.stride(0), x.size(0), (int)x.size(1), f32, cur_stream(x));
+}
+
+void short_conv(Tensor out, Tensor x, Tensor taps, Tensor state, c10::optional<Tensor> cu, Tensor slots, Tensor seq,
+                Tensor pos) {
+  const bool f32 = act_f32(x);
+  CHECK_CONTIG(out); CHECK_F32(taps); CHECK_CONTIG(taps); CHECK_CONTIG(state); CHECK_I32(slots); CHECK_I32(seq); CHECK_I32(pos);
+  const int64_t T = x.size(0), C = x.size(1), n = taps.size(0);
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && out.is_cuda() && out.scalar_type() == x.scalar_type() &&
+              out.sizes() == x.sizes());
+  TORCH_CHECK(taps.dim() == 2 && taps.size(1) == C && n >= 1 && n <= 16, "short_conv: taps [n, C], n <= 16");
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == x.scalar_type() && state.dim() == 3 && state.size(1) == n - 1 &&
+              state.size(2) == C, "short_conv: state [slots, n - 1, C] of the rows' type");
+  TORCH_CHECK(pos.numel() == T);
+  const int64_t ns = slots.numel();
+  const int32_t* cp = nullptr;
+  if (cu.has_value()) {
+    CHECK_I32(*cu);
+    TORCH_CHECK(cu->numel() == ns + 1 && seq.numel() == T);
+    cp = cu->data_ptr<int32_t>();
+  } else {
+    TORCH_CHECK(ns == T, "short_conv: without cu every row is a segment");
+  }
+  nga::launch_short_conv(out.data_ptr(), x.data_ptr(), x.stride(0), taps.data_ptr<float>(), state.data_ptr(), (int)C, (int)n,
+                         cp, slots.data_ptr<int32_t>(), seq.data_ptr<int32_t>(), pos.data_ptr<int32_t>(), T, (int)ns, f32,
+                         cur_stream(x));
+}
+
+nga::DeltaParams delta_params(const Tensor& out, const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& w,
+                              const Tensor& b, const Tensor& w_vec, const Tensor& b_vec, const Tensor& state, int64_t mode,
+                              int64_t H, int64_t G, int64_t d, int64_t dv, double decay, const Tensor& slots,
+                              const Tensor& pos) {
+  CHECK_F32(out); CHECK_CONTIG(out); CHECK_F32(w_vec); CHECK_F32(b_vec); CHECK_F32(state); CHECK_CONTIG(state);
+  CHECK_I32(slots); CHECK_I32(pos);
+  const int64_t T = q.size(0);
+  TORCH_CHECK(mode == 0 || mode == 1);
+  TORCH_CHECK(H >= 1 && G >= 1 && H % G == 0 && (mode == 0 || G == H) && d >= 1 && d <= 256 && dv >= 1,
+              "delta: heads, key size (at most 256) or value size");
+  const int64_t gates = mode == 0 ? H : H * d;
+  auto rows = [&](const Tensor& t, int64_t cols, const char* what) {
+    TORCH_CHECK(t.is_cuda() && t.scalar_type() == q.scalar_type() && t.dim() == 2 && t.size(0) == T && t.size(1) == cols &&
+                t.stride(1) == 1, "delta: ", what, " rows");
+  };
+  rows(q, G * d, "q"); rows(k, G * d, "k"); rows(v, H * dv, "v"); rows(w, gates, "decay"); rows(b, gates, "gate");
+  TORCH_CHECK(w_vec.numel() == gates && b_vec.numel() == gates);
+  TORCH_CHECK(out.dim() == 2 && out.size(0) == T && out.size(1) == H * dv && pos.numel() == T);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == d && state.size(3) == dv,
+              "delta: state [slots, H, d, dv]");
+  TORCH_CHECK(decay >= 0 && decay <= 4);
+  nga::DeltaParams p{};
+  p.out = out.data_ptr<float>();
+  p.q = q.data_ptr(); p.k = k.data_ptr(); p.v = v.data_ptr(); p.w = w.data_ptr(); p.b = b.data_ptr();
+  p.qs = q.stride(0); p.ks = k.stride(0); p.vs = v.stride(0); p.ws = w.stride(0); p.bs = b.stride(0);
+  p.w_vec = w_vec.data_ptr<float>();
+  p.b_vec = b_vec.data_ptr<float>();
+  p.state = state.data_ptr<float>();
+  p.mode = (int)mode; p.H = (int)H; p.G = (int)G; p.d = (int)d; p.dv = (int)dv;
+  p.decay = (float)decay;
+  p.slots = slots.data_ptr<int32_t>();
+  p.pos = pos.data_ptr<int32_t>();
+  return p;
+}
+
+// single rows: row i is segment i
+void delta_rows(Tensor out, Tensor q, Tensor k, Tensor v, Tensor w, Tensor b, Tensor w_vec, Tensor b_vec, Tensor state,
+                int64_t mode, int64_t H, int64_t G, int64_t d, int64_t dv, double decay, Tensor slots, Tensor pos) {
+  const bool f32 = act_f32(q);
+  TORCH_CHECK(slots.numel() == q.size(0), "delta_rows: every row is a segment");
+  nga::launch_delta_rows(delta_params(out, q, k, v, w, b, w_vec, b_vec, state, mode, H, G, d, dv, decay, slots, pos),
+                         (int)q.size(0), f32, cur_stream(q));
+}
+
+// portions: segment i is rows cu[i] .. cu[i + 1] of the launch's rows, at most max_q of them; ws: block operands
+void delta_blocks(Tensor out, Tensor ws, Tensor q, Tensor k, Tensor v, Tensor w, Tensor b, Tensor w_vec, Tensor b_vec,
+                  Tensor state, int64_t mode, int64_t H, int64_t G, int64_t d, int64_t dv, double decay, Tensor cu,
+                  Tensor slots, Tensor pos, int64_t max_q) {
+  const bool f32 = act_f32(q);
+  CHECK_F32(ws); CHECK_CONTIG(ws); CHECK_I32(cu);
+  nga::DeltaParams p = delta_params(out, q, k, v, w, b, w_vec, b_vec, state, mode, H, G, d, dv, decay, slots, pos);
+  const int64_t n = slots.numel(), T = q.size(0), dt = nga::delta_key_tiles((int)d);
+  TORCH_CHECK(cu.numel() == n + 1 && max_q >= 1 && max_q <= T);
+  TORCH_CHECK(ws.numel() >= (T / 16 + n) * H * (65 * 16 * dt + 256) && (uintptr_t)ws.data_ptr() % 16 == 0,
+              "delta_blocks: workspace too small");
+  p.cu = cu.data_ptr<int32_t>();
+  nga::launch_delta_blocks(p, ws.data_ptr<float>(), (int)n, (int)max_q, f32, cur_stream(q));
 }
 
 void hgrn2_scan(Tensor out, Tensor proj, Tensor f_bias, Tensor lower, Tensor state, int64_t H, int64_t d, int64_t dv,
@@ -1741,6 +1887,14 @@ PYBIND11_MODULE(_C, m) {
   m.def("headnorm_cache", checked("headnorm_cache", &headnorm_cache));
   m.def("softmax_attention", checked("softmax_attention", &softmax_attention));
   m.def("hgrn2_scan", checked("hgrn2_scan", &hgrn2_scan));
+  m.def("bigram_embed", checked("bigram_embed", &bigram_embed));
+  m.def("token_save", checked("token_save", &token_save));
+  m.def("gelu_gate_rows", checked("gelu_gate_rows", &gelu_gate_rows));
+  m.def("tanh_rows", checked("tanh_rows", &tanh_rows));
+  m.def("short_conv", checked("short_conv", &short_conv));
+  m.def("delta_rows", checked("delta_rows", &delta_rows));
+  m.def("delta_blocks", checked("delta_blocks", &delta_blocks));
+  m.def("delta_key_tiles", [](int64_t d) { return (int64_t)nga::delta_key_tiles((int)d); });
   m.def("mlstm_scan", checked("mlstm_scan", &mlstm_scan));
   m.def("dyt_norm", checked("dyt_norm", &dyt_norm));
   m.def("residual_dyt", checked("residual_dyt", &residual_dyt));

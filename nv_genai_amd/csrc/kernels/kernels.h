@@ -154,30 +154,30 @@ void launch_quant_fp8_rows(const uint16_t* x, int64_t ldx, int64_t rows, int H, 
 
 // moe.hip (sparse MoE MLP)
 struct MoeGemmParams {
-  const uint16_t* A;         // MODE 0: token rows x [T, K] (gathered); MODE 1: [M, K] sorted rows
+  const uint16_t* A;         // MODE 0, 2: token rows x [T, K] (gathered); MODE 1: [M, K] sorted rows
   int64_t lda;
   const uint16_t* W;         // [E, w_rows, K] expert weights
   int64_t w_rows;            // rows per expert (2F for gate|up, N for down)
   int K;
   int F;                     // MODE 0: features (up rows start at F)
   int mt;                    // M tiles (table entries)
-  int nt;                    // N blocks: F / 128 (MODE 0) or N / 256 (MODE 1)
+  int nt;                    // N blocks: F / 128 (MODE 0), N / 256 (MODE 1), ceil(F / 256) (MODE 2)
   const int32_t* sorted_tok;
   const float* sorted_w;
   const int32_t* tiles;      // [mt, 3]: expert, first row, end row (expert -1: unused)
   uint16_t* out;
   int64_t ldo;
-  int act;                   // MODE 0: 0 silu, 1 gelu_tanh, 2 clamped GLU (limit, alpha)
+  int act;                   // MODE 0: 0 silu, 1 gelu_tanh, 2 clamped GLU (limit, alpha); MODE 2: 3 gelu (erf)
   float limit, alpha;
   int in_weight;             // the routing weight scales the expert's input (MODE 0) and not its output (MODE 1)
 };
 // grouped GEMMs on fp32-accumulating VALU tiles: any sizes, bf16 or fp32 operands
 struct MoeRowsParams {
-  const void* A;             // MODE 0: token rows [T, K] (gathered); MODE 1: [M, K] sorted rows
+  const void* A;             // MODE 0, 2: token rows [T, K] (gathered); MODE 1: [M, K] sorted rows
   int64_t lda;
   const void* W;             // [E, w_rows, K]
   int64_t w_rows;
-  int K, F, N, mt;           // MODE 0: F features (up rows start at F); MODE 1: N outputs
+  int K, F, N, mt;           // MODE 0: F features (up rows start at F); MODE 1: N outputs; MODE 2: N features, gelu (erf)
   const int32_t* sorted_tok;
   const float* sorted_w;
   const int32_t* tiles;
@@ -345,33 +345,47 @@ struct RopeHeadnormParams {
 };
 void launch_rope_headnorm_cache(const RopeHeadnormParams& p, int64_t T, bool f32, hipStream_t stream);
 // w: gs weights shared by the groups, or groups * gs (w_full); gate [T, groups * gs] rows of the output type or nullptr
-void launch_group_rmsnorm(void* out, const float* x, const float* w, bool w_full, const void* gate, int64_t g_stride,
-                          int64_t T, int groups, int gs, float eps, bool f32, hipStream_t stream);
+// gate_silu: times silu(gate) instead of sigmoid(gate); o_stride: elements between output rows
+void launch_group_rmsnorm(void* out, int64_t o_stride, const float* x, const float* w, bool w_full, const void* gate,
+                          int64_t g_stride, bool gate_silu, int64_t T, int groups, int gs, float eps, bool f32,
+                          hipStream_t stream);
+
+// bigram embedding, token gate, tanh of strided rows (postnorm.hip)
+void launch_bigram_embed(float* x, const int32_t* ids, const void* embed, const void* table, const int32_t* src,
+                         int32_t* prev, int64_t mul_prev, int64_t mul_cur, const int32_t* save, int64_t T, int H,
+                         int vocab, int buckets, bool f32, hipStream_t stream);
+void launch_token_save(int32_t* prev, const int32_t* ids, const int32_t* last_row, const int32_t* slot, int n,
+                       hipStream_t stream);
+void launch_gelu_gate_rows(void* out, const void* z, int64_t z_stride, const int32_t* ids, const void* table,
+                           int64_t t_stride, int64_t T, int C, int vocab, bool f32, hipStream_t stream);
+void launch_tanh_rows(void* out, const void* x, int64_t x_stride, int64_t T, int C, bool f32, hipStream_t stream);
 
 // softmax_attention.hip: K [blocks, G * maps, 64, dk], V [blocks, G, 64, dv] pages, bf16 or fp32
 void launch_headnorm_cache(void* proj, int64_t stride, const int32_t* slots, void* kc, void* vc, int64_t T, int nq,
                            int nk, int dk, int nv, int dv, float eps, const float* qw, const float* kw,
                            const float* bias, const int32_t* pos, float coef, int every, bool f32, hipStream_t stream);
-void launch_softmax_attention(void* out, const void* q, int64_t q_stride, const void* gate, int64_t g_stride,
+// chunk > 0: keys of the query's own chunk only; sink: score of a key without a value (-inf: none); o_stride: elements
+// between output rows
+void launch_softmax_attention(void* out, int64_t o_stride, const void* q, int64_t q_stride, const void* gate, int64_t g_stride,
                               const void* kc, const void* vc, const int32_t* block_tables, int max_blocks,
                               const int32_t* tok_seq, const int32_t* pos, int64_t T, int H, int G, int dk, int dv,
                               float scale, int window, int maps, float lam, float unit_eps, float out_scale, bool v_in_k,
-                              float softcap, bool f32, hipStream_t stream);
+                              float softcap, int chunk, float sink, bool f32, hipStream_t stream);
 
 bool softmax_attention_mfma_supported(int dk, int dv, int group, int maps);
-void launch_softmax_attention_mfma(uint16_t* out, const uint16_t* q, int64_t q_stride, const uint16_t* gate,
+void launch_softmax_attention_mfma(uint16_t* out, int64_t o_stride, const uint16_t* q, int64_t q_stride, const uint16_t* gate,
                                    int64_t g_stride, const uint16_t* kc, const uint16_t* vc,
                                    const int32_t* block_tables, int max_blocks, const int32_t* cu_q,
                                    const int32_t* ctx_lens, int B, int max_q_len, int H, int G, int dk, int dv,
                                    float scale, int window, int maps, float lam, float unit_eps, float out_scale,
-                                   bool v_in_k, float softcap, hipStream_t stream);
+                                   bool v_in_k, float softcap, int chunk, float sink, hipStream_t stream);
 int softmax_decode_parts(int rows, int G, int max_ctx, int window);
-void launch_softmax_decode_mfma(uint16_t* out, float* ws, int parts, const uint16_t* q, int64_t q_stride,
+void launch_softmax_decode_mfma(uint16_t* out, int64_t o_stride, float* ws, int parts, const uint16_t* q, int64_t q_stride,
                                 const uint16_t* gate, int64_t g_stride, const uint16_t* kc, const uint16_t* vc,
                                 const int32_t* block_tables, int max_blocks, const int32_t* tok_seq,
                                 const int32_t* pos, int64_t T, int H, int G, int dk, int dv, float scale, int window,
                                 int maps, float lam, float unit_eps, float out_scale, bool v_in_k, float softcap,
-                                hipStream_t stream);
+                                int chunk, float sink, hipStream_t stream);
 
 // recurrent.hip
 int mlstm_max_dim();
@@ -383,5 +397,27 @@ int hgrn2_max_dim(int dv);
 bool launch_hgrn2_scan(float* out, const void* proj, int64_t stride, const float* f_bias, const float* lower,
                        float* state, int H, int d, int dv, const int32_t* cu, const int32_t* slots, const int32_t* pos,
                        int n_seg, bool f32, hipStream_t stream);
+// causal convolution per channel + silu (recurrent.hip); cu == nullptr: every row is a segment
+void launch_short_conv(void* out, const void* x, int64_t x_stride, const float* taps, void* state, int C, int n_taps,
+                       const int32_t* cu, const int32_t* slots, const int32_t* seq, const int32_t* pos, int64_t T,
+                       int n_seg, bool f32, hipStream_t stream);
+
+// delta.hip: rows q / r, k [G * d], v [H * dv], mode 0: w = decay, b = step size pre-activations [H], w_vec = log rates,
+// b_vec = decay bias [H]; mode 1: w = decay, b = removal rate pre-activations [H * d], w_vec / b_vec their biases
+struct DeltaParams {
+  float* out;                // [T, H * dv]
+  const void *q, *k, *v, *w, *b;
+  int64_t qs, ks, vs, ws, bs;      // row strides
+  const float *w_vec, *b_vec;
+  float* state;              // [slots, H, d, dv]
+  int mode, H, G, d, dv;     // head h reads q / k head h / (H / G) (mode 1: G = H)
+  float decay;               // mode 1: w = exp(-decay sigmoid(.))
+  const int32_t* cu;         // portions: [n_seg + 1] row offsets
+  const int32_t* slots;      // [n_seg]
+  const int32_t* pos;        // [T]
+};
+int delta_key_tiles(int d);
+void launch_delta_rows(const DeltaParams& p, int n, bool f32, hipStream_t stream);
+void launch_delta_blocks(const DeltaParams& p, float* ws, int n_seg, int max_q, bool f32, hipStream_t stream);
 
 }  // namespace nga

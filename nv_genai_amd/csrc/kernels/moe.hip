@@ -17,6 +17,8 @@
 //   moe_gemm act 2    clamped GLU epilogue g sigmoid(alpha g) (u + 1), g = min(gate, limit),
 //                u = clamp(up, +-limit), with the routing weight on the expert's input
 //                (the accumulators are scaled: W (s x) = s (W x)) and none on the down GEMM
+//   moe_gemm MODE 2   gathered token rows x the expert's rows as they are (no gate), gelu (erf) in the
+//                epilogue
 //   moe_gemm_rows     the grouped GEMMs on 64 x 64 fp32-accumulating VALU tiles: bf16 or fp32
 //                operands, any K / F / N (experts too small or too odd for the MFMA tiles,
 //                and the true-fp32 path)
@@ -51,6 +53,7 @@ __device__ __forceinline__ float gelu_tanh(float x) {
   const float u = 0.7978845608028654f * (x + 0.044715f * x * x * x);
   return x - x / (1.f + __expf(2.f * u));
 }
+__device__ __forceinline__ float gelu_erf(float x) { return 0.5f * x * (1.f + erff(x * 0.7071067811865475f)); }
 // g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit)
 __device__ __forceinline__ float clamped_glu(float gate, float up, float limit, float alpha, float shift = 1.f) {
   const float g = fminf(gate, limit);
@@ -215,6 +218,7 @@ __global__ void __launch_bounds__(256) moe_gemm_kernel(MoeGemmParams P) {
       wrow = (r & 16) ? P.F + f : f;
     } else {
       wrow = nb * BN + r;
+      if (MODE == 2 && wrow >= P.w_rows) wrow = 0;   // a partial last block: any valid row (not stored)
     }
     wsrc[i] = We + (int64_t)wrow * P.K + ch * 8;
   }
@@ -225,7 +229,7 @@ __global__ void __launch_bounds__(256) moe_gemm_kernel(MoeGemmParams P) {
     const int ch = (lane & 7) ^ ((r >> 1) & 7);
     int pos = row0 + r;
     if (pos >= row1) pos = row0;   // padding rows of a partial tile: any valid row (not stored)
-    const int64_t arow = MODE == 0 ? (int64_t)P.sorted_tok[pos] : (int64_t)pos;
+    const int64_t arow = MODE != 1 ? (int64_t)P.sorted_tok[pos] : (int64_t)pos;
     xsrc[i] = P.A + arow * P.lda + ch * 8;
   }
   auto issue = [&](int kt, int buf) {
@@ -315,6 +319,16 @@ __global__ void __launch_bounds__(256) moe_gemm_kernel(MoeGemmParams P) {
                                  : (P.act == 0 ? silu(gt) : gelu_tanh(gt)) * up);
         }
         *reinterpret_cast<u16x4*>(op + f) = v;
+      }
+    } else if (MODE == 2) {
+#pragma unroll
+      for (int nt = 0; nt < NTW; ++nt) {
+        const int n = nb * BN + wn * 128 + nt * 16 + 4 * h;
+        if (n >= P.w_rows) continue;
+        u16x4 v;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = f2bf(gelu_erf(acc[nt][mt][r]));
+        *reinterpret_cast<u16x4*>(op + n) = v;
       }
     } else {
       const float sc = P.in_weight ? 1.f : P.sorted_w[pos];
@@ -445,7 +459,7 @@ __global__ void __launch_bounds__(RG_THREADS) moe_route_grouped_kernel(
   for (int e = 0; e < E; ++e) {
     const float v = s[e * RG_THREADS] / den;
     s[e * RG_THREADS] = v;
-    c[e * RG_THREADS] = v + correction[e];
+    c[e * RG_THREADS] = correction ? v + correction[e] : v;
   }
   if (groups > 1) {
     const int per = E / groups;
@@ -498,7 +512,8 @@ __global__ void __launch_bounds__(RG_THREADS) moe_route_grouped_kernel(
 // output columns; K in steps of 16 through LDS; a thread owns 4 rows x 4 columns (fp32). MODE 0:
 // gathered token rows x the expert's gate and up rows of the same 64 features (two accumulator
 // sets), epilogue = routing weight on the input (optional) and the clamped GLU; MODE 1: sorted
-// activation rows x the expert's down rows, optionally times the routing weight. No alignment
+// activation rows x the expert's down rows, optionally times the routing weight; MODE 2: gathered
+// token rows x the expert's rows, gelu (erf). No alignment
 // or divisibility is assumed.
 namespace {
 template <typename T> __device__ __forceinline__ float ldv(const T* p);
@@ -535,7 +550,7 @@ __global__ void __launch_bounds__(256) moe_gemm_rows_kernel(MoeRowsParams P) {
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int pos = row0 + lr + 16 * i;
-    arow[i] = pos < row1 ? (MODE == 0 ? (int64_t)P.sorted_tok[pos] : (int64_t)pos) : -1;
+    arow[i] = pos < row1 ? (MODE != 1 ? (int64_t)P.sorted_tok[pos] : (int64_t)pos) : -1;
   }
   for (int k0 = 0; k0 < P.K; k0 += RK) {
     const int kk = k0 + lk;
@@ -579,7 +594,9 @@ __global__ void __launch_bounds__(256) moe_gemm_rows_kernel(MoeRowsParams P) {
     for (int j = 0; j < 4; ++j) {
       const int n = nb * RT + 4 * tc + j;
       if (n >= N) continue;
-      const float v = MODE == 0 ? clamped_glu(accA[i][j] * sw, accB[i][j] * sw, P.limit, P.alpha, P.shift) : accA[i][j] * sw;
+      const float v = MODE == 0   ? clamped_glu(accA[i][j] * sw, accB[i][j] * sw, P.limit, P.alpha, P.shift)
+                      : MODE == 2 ? gelu_erf(accA[i][j] * sw)
+                                  : accA[i][j] * sw;
       stv(out + (int64_t)pos * P.ldo + n, v);
     }
   }
@@ -641,7 +658,10 @@ void launch_moe_gemm(const MoeGemmParams& p, int bm, int mode, hipStream_t strea
     return;
   }
 #endif
-  if (mode == 0) {
+  if (mode == 2) {
+    if (bm == 64) moe_gemm_kernel<64, 2><<<grid, 256, 0, stream>>>(p);
+    else moe_gemm_kernel<128, 2><<<grid, 256, 0, stream>>>(p);
+  } else if (mode == 0) {
     if (bm == 64) moe_gemm_kernel<64, 0><<<grid, 256, 0, stream>>>(p);
     else moe_gemm_kernel<128, 0><<<grid, 256, 0, stream>>>(p);
   } else {
@@ -677,9 +697,11 @@ void launch_moe_gemm_rows(const MoeRowsParams& p, int mode, bool f32, hipStream_
   dim3 grid((N + RT - 1) / RT, p.mt);
   if (f32) {
     if (mode == 0) moe_gemm_rows_kernel<float, 0><<<grid, 256, 0, stream>>>(p);
+    else if (mode == 2) moe_gemm_rows_kernel<float, 2><<<grid, 256, 0, stream>>>(p);
     else moe_gemm_rows_kernel<float, 1><<<grid, 256, 0, stream>>>(p);
   } else {
     if (mode == 0) moe_gemm_rows_kernel<uint16_t, 0><<<grid, 256, 0, stream>>>(p);
+    else if (mode == 2) moe_gemm_rows_kernel<uint16_t, 2><<<grid, 256, 0, stream>>>(p);
     else moe_gemm_rows_kernel<uint16_t, 1><<<grid, 256, 0, stream>>>(p);
   }
 }

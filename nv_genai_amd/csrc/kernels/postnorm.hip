@@ -23,6 +23,11 @@
 //                     the step between two parallel layers in one pass
 //   pack_pair         [a | b] rows of two fp32 streams in the activation type
 //   bias_gelu_tanh    gelu_tanh(x + bias) in place, fp32 bias, any width
+//   bigram_embed      x[t] = embed[id] + table[(previous id * a + id * b) mod buckets], the previous id
+//                     from this step's rows or from a state slot; the table's last row at the start
+//   token_save        the slot takes the last id of every sequence of the step
+//   gelu_gate_rows    gelu_tanh(z) * (columns of the token's own row of a table)
+//   tanh_rows         tanh of a column slice
 //
 // The residual, the norms and the shift interpolation are fp32 whatever the activation type T
 // (bf16 storage as uint16_t, or float). Memory-bound: one workgroup per row, columns strided
@@ -195,7 +200,8 @@ __global__ void __launch_bounds__(256) relu_sq_bf16x8_kernel(uint16_t* __restric
 }
 
 // Two passes over the row: residual sum with the statistic of the new x, then the norm's output
-// (each thread re-reads only the columns it wrote itself). out == nullptr: the sum only.
+// (each thread re-reads only the columns it wrote itself). out == nullptr: the sum only; w == nullptr:
+// out is a copy of the sum.
 template <typename T>
 __global__ void __launch_bounds__(256) residual_add_rmsnorm_kernel(float* __restrict__ x, const T* __restrict__ y,
                                                                    int64_t y_stride, const float* __restrict__ w,
@@ -211,6 +217,10 @@ __global__ void __launch_bounds__(256) residual_add_rmsnorm_kernel(float* __rest
     ss += v * v;
   }
   if (!out) return;
+  if (!w) {     // a copy of the sum
+    for (int c = threadIdx.x; c < H; c += blockDim.x) stf(out + row * H + c, xr[c]);
+    return;
+  }
   ss = block_sum(ss, red);
   const float r = 1.0f / sqrtf(ss / (float)H + eps);
   for (int c = threadIdx.x; c < H; c += blockDim.x) stf(out + row * H + c, xr[c] * r * w[c]);
@@ -267,7 +277,8 @@ template <typename T>
 __global__ void __launch_bounds__(256) group_rmsnorm_kernel(T* __restrict__ out, const float* __restrict__ x,
                                                             const float* __restrict__ w, int64_t n_groups, int gs,
                                                             float eps, int groups, int w_full,
-                                                            const T* __restrict__ gate, int64_t g_stride, int pair) {
+                                                            const T* __restrict__ gate, int64_t g_stride, int pair,
+                                                            int silu, int64_t o_stride) {
   const int64_t g = blockIdx.x * (int64_t)(blockDim.x >> 6) + (threadIdx.x >> 6);
   if (g >= n_groups) return;
   const int lane = threadIdx.x & 63;
@@ -276,6 +287,11 @@ __global__ void __launch_bounds__(256) group_rmsnorm_kernel(T* __restrict__ out,
   const int hg = (int)(g - row * groups);
   const float* wr = w_full ? w + (int64_t)hg * gs : w;
   const T* gr = gate ? gate + row * g_stride + (int64_t)hg * gs : nullptr;
+  T* orow = out + row * o_stride + (int64_t)hg * gs;
+  auto gated = [&](int c) {
+    const float z = ldf(gr + c);
+    return (silu ? z : 1.0f) / (1.0f + expf(-z));
+  };
   float ss = 0.f;
   if (pair) {   // gs even, 8-byte aligned fp32 rows: two neighbouring elements per lane
     for (int c = 2 * lane; c < gs; c += 128) {
@@ -288,11 +304,11 @@ __global__ void __launch_bounds__(256) group_rmsnorm_kernel(T* __restrict__ out,
       const float2 v = *reinterpret_cast<const float2*>(xr + c);
       float a = v.x * r * wr[c], b = v.y * r * wr[c + 1];
       if (gr) {
-        a *= 1.0f / (1.0f + expf(-ldf(gr + c)));
-        b *= 1.0f / (1.0f + expf(-ldf(gr + c + 1)));
+        a *= gated(c);
+        b *= gated(c + 1);
       }
-      stf(out + g * gs + c, a);
-      stf(out + g * gs + c + 1, b);
+      stf(orow + c, a);
+      stf(orow + c + 1, b);
     }
     return;
   }
@@ -301,8 +317,8 @@ __global__ void __launch_bounds__(256) group_rmsnorm_kernel(T* __restrict__ out,
   const float r = 1.0f / sqrtf(ss / (float)gs + eps);
   for (int c = lane; c < gs; c += 64) {
     float v = xr[c] * r * wr[c];
-    if (gr) v *= 1.0f / (1.0f + expf(-ldf(gr + c)));
-    stf(out + g * gs + c, v);
+    if (gr) v *= gated(c);
+    stf(orow + c, v);
   }
 }
 
@@ -312,7 +328,8 @@ __global__ void __launch_bounds__(256) group_rmsnorm_kernel(T* __restrict__ out,
 __global__ void __launch_bounds__(256) group_rmsnorm_bf16x4_kernel(uint16_t* __restrict__ out, const float* __restrict__ x,
                                                                    const float* __restrict__ w, int64_t n_groups, int gs,
                                                                    float eps, int groups, int w_full,
-                                                                   const uint16_t* __restrict__ gate, int64_t g_stride) {
+                                                                   const uint16_t* __restrict__ gate, int64_t g_stride,
+                                                                   int silu, int64_t o_stride) {
   const int64_t g = blockIdx.x * (int64_t)(blockDim.x >> 5) + (threadIdx.x >> 5);
   const bool live = g < n_groups;
   const int sub = threadIdx.x & 31;
@@ -337,12 +354,15 @@ __global__ void __launch_bounds__(256) group_rmsnorm_bf16x4_kernel(uint16_t* __r
     if (gr) {
       const u16x4 g4 = *reinterpret_cast<const u16x4*>(gr + c);
 #pragma unroll
-      for (int q = 0; q < 4; ++q) y[q] *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * bf2f(g4[q])));
+      for (int q = 0; q < 4; ++q) {
+        const float z = bf2f(g4[q]);
+        y[q] *= (silu ? z : 1.0f) * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+      }
     }
     u16x4 o4;
 #pragma unroll
     for (int q = 0; q < 4; ++q) o4[q] = f2bf(y[q]);
-    *reinterpret_cast<u16x4*>(out + gg * gs + c) = o4;
+    *reinterpret_cast<u16x4*>(out + row * o_stride + (int64_t)hg * gs + c) = o4;
   }
 }
 
@@ -474,6 +494,66 @@ __global__ void __launch_bounds__(256) bias_gelu_tanh_bf16x8_kernel(uint16_t* __
       o[j] = f2bf(z - z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.8853900817779268f * u)));
     }
     store8(xb + (int64_t)i * 8, o);
+  }
+}
+
+// Bigram embedding. src as in token_shift; save (steps of single rows): slot that takes the row's id
+// afterwards - read and written by the same workgroup, the read in front of the barrier.
+template <typename T>
+__global__ void __launch_bounds__(256) bigram_embed_kernel(float* __restrict__ x, const int32_t* __restrict__ ids,
+                                                           const T* __restrict__ embed, const T* __restrict__ table,
+                                                           const int32_t* __restrict__ src, int32_t* __restrict__ prev,
+                                                           int64_t mul_prev, int64_t mul_cur,
+                                                           const int32_t* __restrict__ save, int H, int vocab,
+                                                           int buckets) {
+  __shared__ int64_t brow;
+  const int64_t row = blockIdx.x;
+  int id = ids[row];
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);   // padding rows of a captured step
+  if (threadIdx.x == 0) {
+    const int s = src[row];
+    int64_t r = buckets;
+    if (s != -1) {
+      const int p = s >= 0 ? ids[s] : prev[-(s + 2)];
+      r = ((int64_t)(p < 0 ? 0 : p) * mul_prev + (int64_t)id * mul_cur) % buckets;
+    }
+    if (save && save[row] >= 0) prev[save[row]] = id;
+    brow = r;
+  }
+  __syncthreads();
+  const T* er = embed + (int64_t)id * H;
+  const T* br = table + brow * H;
+  for (int c = threadIdx.x; c < H; c += blockDim.x) x[row * H + c] = ldf(er + c) + ldf(br + c);
+}
+
+__global__ void __launch_bounds__(256) token_save_kernel(int32_t* __restrict__ prev, const int32_t* __restrict__ ids,
+                                                         const int32_t* __restrict__ last_row,
+                                                         const int32_t* __restrict__ slot, int n) {
+  const int i = blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n && slot[i] >= 0 && last_row[i] >= 0) prev[slot[i]] = ids[last_row[i]];
+}
+
+// table: first column of the slice
+template <typename T>
+__global__ void __launch_bounds__(256) gelu_gate_rows_kernel(T* __restrict__ out, const T* __restrict__ z, int64_t z_stride,
+                                                             const int32_t* __restrict__ ids,
+                                                             const T* __restrict__ table, int64_t t_stride,
+                                                             int64_t total, int C, int vocab) {
+  for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
+    const int64_t t = i / C;
+    const int c = (int)(i - t * C);
+    int id = ids[t];
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    stf(out + i, gelu_tanh_exact(ldf(z + t * z_stride + c)) * ldf(table + (int64_t)id * t_stride + c));
+  }
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256) tanh_rows_kernel(T* __restrict__ out, const T* __restrict__ x, int64_t x_stride,
+                                                        int64_t total, int C) {
+  for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
+    const int64_t t = i / C;
+    stf(out + i, tanhf(ldf(x + t * x_stride + (i - t * C))));
   }
 }
 
@@ -610,24 +690,27 @@ void launch_clamped_glu(void* out, const void* in, int64_t in_stride, int64_t T,
                                                                        T, F, limit, alpha, gate_col, shift);
 }
 
-void launch_group_rmsnorm(void* out, const float* x, const float* w, bool w_full, const void* gate, int64_t g_stride,
-                          int64_t T, int groups, int gs, float eps, bool f32, hipStream_t stream) {
+void launch_group_rmsnorm(void* out, int64_t o_stride, const float* x, const float* w, bool w_full, const void* gate,
+                          int64_t g_stride, bool gate_silu, int64_t T, int groups, int gs, float eps, bool f32,
+                          hipStream_t stream) {
   const int64_t ng = T * groups;
   if (ng == 0) return;
   if (!f32 && gs % 4 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0 && ((uintptr_t)out % 8) == 0 &&
-      (gate == nullptr || (g_stride % 4 == 0 && ((uintptr_t)gate % 8) == 0))) {
+      o_stride % 4 == 0 && (gate == nullptr || (g_stride % 4 == 0 && ((uintptr_t)gate % 8) == 0))) {
     group_rmsnorm_bf16x4_kernel<<<dim3((unsigned)((ng + 7) / 8)), 256, 0, stream>>>(
-        (uint16_t*)out, x, w, ng, gs, eps, groups, w_full ? 1 : 0, (const uint16_t*)gate, g_stride);
+        (uint16_t*)out, x, w, ng, gs, eps, groups, w_full ? 1 : 0, (const uint16_t*)gate, g_stride, gate_silu ? 1 : 0,
+        o_stride);
     return;
   }
   const unsigned g = (unsigned)((ng + 3) / 4);
   const int pair = (gs % 2 == 0 && ((uintptr_t)x % 8) == 0) ? 1 : 0;
   if (f32)
     group_rmsnorm_kernel<float><<<dim3(g), 256, 0, stream>>>((float*)out, x, w, ng, gs, eps, groups, w_full ? 1 : 0,
-                                                             (const float*)gate, g_stride, pair);
+                                                             (const float*)gate, g_stride, pair, gate_silu ? 1 : 0, o_stride);
   else
     group_rmsnorm_kernel<uint16_t><<<dim3(g), 256, 0, stream>>>((uint16_t*)out, x, w, ng, gs, eps, groups, w_full ? 1 : 0,
-                                                                (const uint16_t*)gate, g_stride, pair);
+                                                                (const uint16_t*)gate, g_stride, pair, gate_silu ? 1 : 0,
+                                                                o_stride);
 }
 
 void launch_dyt_norm(void* out, const float* x, float alpha, const float* w, const float* b, const int64_t* rows,
@@ -685,6 +768,52 @@ void launch_bias_gelu_tanh(void* x, const float* bias, int64_t T, int F, bool f3
     bias_gelu_tanh_kernel<float><<<dim3((unsigned)g), 256, 0, stream>>>((float*)x, bias, T, F);
   else
     bias_gelu_tanh_kernel<uint16_t><<<dim3((unsigned)g), 256, 0, stream>>>((uint16_t*)x, bias, T, F);
+}
+
+void launch_bigram_embed(float* x, const int32_t* ids, const void* embed, const void* table, const int32_t* src,
+                         int32_t* prev, int64_t mul_prev, int64_t mul_cur, const int32_t* save, int64_t T, int H,
+                         int vocab, int buckets, bool f32, hipStream_t stream) {
+  if (T == 0) return;
+  if (f32)
+    bigram_embed_kernel<float><<<dim3((unsigned)T), 256, 0, stream>>>(x, ids, (const float*)embed, (const float*)table, src,
+                                                                     prev, mul_prev, mul_cur, save, H, vocab, buckets);
+  else
+    bigram_embed_kernel<uint16_t><<<dim3((unsigned)T), 256, 0, stream>>>(x, ids, (const uint16_t*)embed,
+                                                                        (const uint16_t*)table, src, prev, mul_prev,
+                                                                        mul_cur, save, H, vocab, buckets);
+}
+
+void launch_token_save(int32_t* prev, const int32_t* ids, const int32_t* last_row, const int32_t* slot, int n,
+                       hipStream_t stream) {
+  if (n == 0) return;
+  token_save_kernel<<<dim3((unsigned)((n + 255) / 256)), 256, 0, stream>>>(prev, ids, last_row, slot, n);
+}
+
+void launch_gelu_gate_rows(void* out, const void* z, int64_t z_stride, const int32_t* ids, const void* table,
+                           int64_t t_stride, int64_t T, int C, int vocab, bool f32, hipStream_t stream) {
+  const int64_t total = T * C;
+  if (total == 0) return;
+  int64_t g = (total + 255) / 256;
+  if (g > 8192) g = 8192;
+  if (f32)
+    gelu_gate_rows_kernel<float><<<dim3((unsigned)g), 256, 0, stream>>>((float*)out, (const float*)z, z_stride, ids,
+                                                                       (const float*)table, t_stride, total, C, vocab);
+  else
+    gelu_gate_rows_kernel<uint16_t><<<dim3((unsigned)g), 256, 0, stream>>>((uint16_t*)out, (const uint16_t*)z, z_stride,
+                                                                          ids, (const uint16_t*)table, t_stride, total, C,
+                                                                          vocab);
+}
+
+void launch_tanh_rows(void* out, const void* x, int64_t x_stride, int64_t T, int C, bool f32, hipStream_t stream) {
+  const int64_t total = T * C;
+  if (total == 0) return;
+  int64_t g = (total + 255) / 256;
+  if (g > 8192) g = 8192;
+  if (f32)
+    tanh_rows_kernel<float><<<dim3((unsigned)g), 256, 0, stream>>>((float*)out, (const float*)x, x_stride, total, C);
+  else
+    tanh_rows_kernel<uint16_t><<<dim3((unsigned)g), 256, 0, stream>>>((uint16_t*)out, (const uint16_t*)x, x_stride, total,
+                                                                     C);
 }
 
 }  // namespace nga

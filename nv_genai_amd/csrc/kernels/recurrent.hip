@@ -15,7 +15,10 @@
 //                reads what another tile of the launch writes. The gate chain of a pass (m, both
 //                decays, e^(-m)) is a prefix scan over the lanes of the first wave, shared through LDS.
 //
-// A workgroup owns (segment, head, tile of VT value columns): thread (rg, j) keeps the state
+//   short_conv   causal convolution over time per channel with silu (in front of a recurrence); the
+//                last inputs of a sequence stay in its state slot
+//
+// The scans: a workgroup owns (segment, head, tile of VT value columns): thread (rg, j) keeps the state
 // elements S[rg * NR + k][j] in registers for the whole segment, so the state is read from its
 // slot once and written back once. Rows are staged through LDS TC at a time: the raw values of the
 // next TC rows are loaded into registers before the current ones are processed, and the
@@ -460,7 +463,159 @@ bool launch_mlstm_t(float* out, const T* proj, int64_t stride, const float* gate
 #undef NGA_MLSTM_ARGS
 }
 
+// ---------------------------------------------------------------------------------------------
+// Short convolution: out[t] = silu(sum_j taps[n - 1 - j][c] x[t - j]), V channels per thread. Inputs in
+// front of the segment come from the state slot [n - 1][C] (oldest first), zeros in front of
+// position 0. SINGLE = false: rows of portions (seq[t]: the row's segment), the slots are written by
+// short_conv_save_kernel behind this launch; SINGLE = true: every row is a segment, and the thread that reads
+// its channels of the slot also writes them.
+constexpr int MAX_TAPS = 16;
+
+template <typename T, int V>
+__device__ __forceinline__ void ldv_(const T* p, float* v) {
+  if constexpr (V == 8) {
+    const u16x8 x = load8((const uint16_t*)p);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = bf2f(x[e]);
+  } else {
+    v[0] = ldf(p);
+  }
+}
+template <typename T, int V>
+__device__ __forceinline__ void stv_(T* p, const float* v) {
+  if constexpr (V == 8) {
+    u16x8 x;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] = f2bf(v[e]);
+    store8((uint16_t*)p, x);
+  } else {
+    if constexpr (sizeof(T) == 4) *p = v[0];
+    else *p = f2bf(v[0]);
+  }
+}
+
+// NT > 0: the number of taps at compile time
+template <typename T, int V, bool SINGLE, int NT>
+__global__ void __launch_bounds__(256) short_conv_kernel(T* __restrict__ out, const T* __restrict__ x, int64_t x_stride,
+                                                         const float* __restrict__ taps, T* __restrict__ state, int C,
+                                                         int n_taps, const int32_t* __restrict__ cu,
+                                                         const int32_t* __restrict__ slots,
+                                                         const int32_t* __restrict__ seq,
+                                                         const int32_t* __restrict__ pos) {
+  const int n = NT > 0 ? NT : n_taps;
+  const int64_t row = blockIdx.x;
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+  if (c >= C) return;
+  const int b = SINGLE ? (int)row : seq[row];
+  const int slot = slots[b], p = pos[row];
+  const int in_seg = SINGLE ? 0 : (int)row - cu[b];      // rows of the segment in front of this one
+  float acc[V];
+#pragma unroll
+  for (int e = 0; e < V; ++e) acc[e] = 0.f;
+  T* st = slot >= 0 ? state + (int64_t)slot * (n - 1) * C + c : nullptr;
+  const float* tp = taps + c;      // [n][C]
+#pragma unroll
+  for (int j = 0; j < (NT > 0 ? NT : MAX_TAPS); ++j) {
+    if (NT == 0 && j >= n) break;
+    float v[V];
+    if (j <= in_seg) {
+      ldv_<T, V>(x + (row - j) * x_stride + c, v);
+    } else if (p - j >= 0 && st) {
+      ldv_<T, V>(st + (int64_t)(n - 1 - (j - in_seg)) * C, v);
+    } else {
+      continue;
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[e] += tp[(int64_t)(n - 1 - j) * C + e] * v[e];
+  }
+  float o[V];
+#pragma unroll
+  for (int e = 0; e < V; ++e) o[e] = sizeof(T) == 4 ? acc[e] / (1.0f + expf(-acc[e])) : acc[e] * sigmoid_fast(acc[e]);
+  stv_<T, V>(out + row * C + c, o);
+  if (SINGLE && st) {     // shift the slot by one input (zeros in front of position 0)
+    for (int e2 = 0; e2 + 1 < n; ++e2) {
+      float v[V];
+      if (e2 + 2 < n) {
+        if (p - (n - 2 - e2) >= 0) {
+          ldv_<T, V>(st + (int64_t)(e2 + 1) * C, v);
+        } else {
+#pragma unroll
+          for (int e = 0; e < V; ++e) v[e] = 0.f;
+        }
+      } else {
+        ldv_<T, V>(x + row * x_stride + c, v);
+      }
+      stv_<T, V>(st + (int64_t)e2 * C, v);
+    }
+  }
+}
+
+// the last n - 1 inputs of every segment into its slot; entry e takes row t1 - (n - 1) + e, which may
+// lie in front of the segment: then the old entry e + rows (read in front of its own rewrite: e ascends)
+template <typename T>
+__global__ void __launch_bounds__(256) short_conv_save_kernel(const T* __restrict__ x, int64_t x_stride,
+                                                              T* __restrict__ state, int C, int n,
+                                                              const int32_t* __restrict__ cu,
+                                                              const int32_t* __restrict__ slots,
+                                                              const int32_t* __restrict__ pos) {
+  const int b = blockIdx.y, c = blockIdx.x * blockDim.x + threadIdx.x;
+  const int t0 = cu[b], t1 = cu[b + 1], slot = slots[b];
+  if (c >= C || t1 <= t0 || slot < 0) return;
+  T* st = state + (int64_t)slot * (n - 1) * C + c;
+  const int p0 = pos[t0];
+  for (int e = 0; e < n - 1; ++e) {
+    const int t = t1 - (n - 1) + e;
+    T v = (T)0;
+    if (t >= t0) v = x[(int64_t)t * x_stride + c];
+    else if (p0 - (t0 - t) >= 0) v = st[(int64_t)(e + t1 - t0) * C];
+    st[(int64_t)e * C] = v;
+  }
+}
+
+template <typename T, int V, bool SINGLE>
+void launch_short_conv_v(T* out, const T* x, int64_t x_stride, const float* taps, T* state, int C, int n,
+                         const int32_t* cu, const int32_t* slots, const int32_t* seq, const int32_t* pos, int64_t rows,
+                         hipStream_t stream) {
+  const dim3 grid((unsigned)rows, (unsigned)((C / V + 255) / 256));
+  if (n == 4)
+    short_conv_kernel<T, V, SINGLE, 4><<<grid, 256, 0, stream>>>(out, x, x_stride, taps, state, C, n, cu, slots, seq, pos);
+  else
+    short_conv_kernel<T, V, SINGLE, 0><<<grid, 256, 0, stream>>>(out, x, x_stride, taps, state, C, n, cu, slots, seq, pos);
+}
+
+template <typename T>
+void launch_short_conv_t(T* out, const T* x, int64_t x_stride, const float* taps, T* state, int C, int n,
+                         const int32_t* cu, const int32_t* slots, const int32_t* seq, const int32_t* pos, int64_t rows,
+                         int n_seg, hipStream_t stream) {
+  const bool vec = sizeof(T) == 2 && C % 8 == 0 && x_stride % 8 == 0 && ((uintptr_t)x % 16) == 0 &&
+                   ((uintptr_t)out % 16) == 0 && ((uintptr_t)state % 16) == 0;
+#define NGA_CONV_ARGS out, x, x_stride, taps, state, C, n, cu, slots, seq, pos, rows, stream
+  if (cu == nullptr) {
+    if (vec) launch_short_conv_v<T, sizeof(T) == 2 ? 8 : 1, true>(NGA_CONV_ARGS);
+    else launch_short_conv_v<T, 1, true>(NGA_CONV_ARGS);
+    return;
+  }
+  if (vec) launch_short_conv_v<T, sizeof(T) == 2 ? 8 : 1, false>(NGA_CONV_ARGS);
+  else launch_short_conv_v<T, 1, false>(NGA_CONV_ARGS);
+#undef NGA_CONV_ARGS
+  if (n > 1)
+    short_conv_save_kernel<T><<<dim3((unsigned)((C + 255) / 256), (unsigned)n_seg), 256, 0, stream>>>(x, x_stride, state, C,
+                                                                                                     n, cu, slots, pos);
+}
+
 }  // namespace
+
+void launch_short_conv(void* out, const void* x, int64_t x_stride, const float* taps, void* state, int C, int n_taps,
+                       const int32_t* cu, const int32_t* slots, const int32_t* seq, const int32_t* pos, int64_t T,
+                       int n_seg, bool f32, hipStream_t stream) {
+  if (T == 0 || n_seg == 0) return;
+  if (f32)
+    launch_short_conv_t<float>((float*)out, (const float*)x, x_stride, taps, (float*)state, C, n_taps, cu, slots, seq, pos,
+                               T, n_seg, stream);
+  else
+    launch_short_conv_t<uint16_t>((uint16_t*)out, (const uint16_t*)x, x_stride, taps, (uint16_t*)state, C, n_taps, cu,
+                                  slots, seq, pos, T, n_seg, stream);
+}
 
 int mlstm_max_dim() { return 256; }   // padded rows of a head that fit the LDS staging
 

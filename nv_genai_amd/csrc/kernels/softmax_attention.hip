@@ -18,8 +18,9 @@
 // `maps` score maps (1 or 2) that share its values: q head (h, m) is column block h * maps + m,
 // its keys are k head (h / (H / G)) * maps + m. Two maps combine as a_0 - lam * a_1
 // (differential attention). Optional: unit RMS of the head output (eps inside the root) times
-// out_scale, and a per-head sigmoid gate. Visible keys of the query at position i: j <= i, and
-// i - j < window when window > 0. v_row: elements between two value rows of a page; v_row = dk with
+// out_scale, and a per-head sigmoid gate; a sink: one more key of a given score without a value. Visible
+// keys of the query at position i: j <= i, i - j < window when window > 0, and, when chunk > 0, keys of
+// the query's own chunk only (j >= floor(i / chunk) chunk). v_row: elements between two value rows of a page; v_row = dk with
 // vc = kc reads the values out of the first dv elements of the key rows (one map: a latent that is
 // key and value, followed by key-only columns).
 #include <cstdlib>
@@ -32,6 +33,13 @@ namespace nga {
 namespace {
 
 constexpr int BS = 64;   // tokens per page
+
+// first key the query at position i can see
+__device__ __forceinline__ int first_key(int i, int window, int chunk) {
+  const int lo = window > 0 && i - window + 1 > 0 ? i - window + 1 : 0;
+  const int ch = chunk > 0 ? i / chunk * chunk : 0;
+  return lo > ch ? lo : ch;
+}
 
 template <typename T> __device__ __forceinline__ float ldf(const T* p);
 template <> __device__ __forceinline__ float ldf<uint16_t>(const uint16_t* p) { return bf2f(*p); }
@@ -126,7 +134,8 @@ __global__ void __launch_bounds__(64) softmax_attention_kernel(
     T* __restrict__ out, const T* __restrict__ q, int64_t q_stride, const T* __restrict__ gate, int64_t g_stride,
     const T* __restrict__ kc, const T* __restrict__ vc, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ pos, int H, int G, int dk, int dv, float scale,
-    int window, int maps, float lam, float unit_eps, float out_scale, int v_row, float softcap) {
+    int window, int maps, float lam, float unit_eps, float out_scale, int v_row, float softcap, int chunk, float sink,
+    int64_t o_stride) {
   extern __shared__ float smem[];
   float* qs = smem;                 // [maps * dk]
   float* ws = smem + maps * dk;     // [64]
@@ -134,7 +143,7 @@ __global__ void __launch_bounds__(64) softmax_attention_kernel(
   const int h = blockIdx.y;
   const int lane = threadIdx.x;
   const int i = pos[row];
-  T* orow = out + row * (int64_t)H * dv + (int64_t)h * dv;
+  T* orow = out + row * o_stride + (int64_t)h * dv;
   if (i < 0) {   // padding row
     for (int d = lane; d < dv; d += 64) stf(orow + d, 0.f);
     return;
@@ -147,13 +156,13 @@ __global__ void __launch_bounds__(64) softmax_attention_kernel(
   float res[MAXV], acc[MAXV];
 #pragma unroll
   for (int u = 0; u < MAXV; ++u) res[u] = 0.f;
-  const int lo = window > 0 && i - window + 1 > 0 ? i - window + 1 : 0;
+  const int lo = first_key(i, window, chunk);
   const int p_lo = lo / BS, p_hi = i / BS;
   const bool vec = (dk % (16 / (int)sizeof(T))) == 0;
   __syncthreads();
   for (int m = 0; m < maps; ++m) {
     const int kh = g * maps + m;
-    float mx = -INFINITY, l = 0.f;
+    float mx = sink, l = sink == -INFINITY ? 0.f : 1.f;
 #pragma unroll
     for (int u = 0; u < MAXV; ++u) acc[u] = 0.f;
     for (int p = p_lo; p <= p_hi; ++p) {
@@ -166,7 +175,7 @@ __global__ void __launch_bounds__(64) softmax_attention_kernel(
         if (softcap > 0.f) s = softcap * tanhf(s / softcap);
       }
       const float nmx = fmaxf(mx, wave_max(s));   // every visited page holds a visible key
-      const float corr = expf(mx - nmx);          // 0 on the first page (mx = -inf)
+      const float corr = expf(mx - nmx);          // 0 on the first page without a sink (mx = -inf)
       const float w = vis ? expf(s - nmx) : 0.f;
       l = l * corr + wave_sum(w);
       mx = nmx;
@@ -190,7 +199,7 @@ __global__ void __launch_bounds__(64) softmax_attention_kernel(
 #pragma unroll
     for (int u = 0; u < MAXV; ++u) res[u] = m == 0 ? acc[u] * inv : res[u] - lam * (acc[u] * inv);
   }
-  float r = 1.0f;
+  float r = out_scale;
   if (unit_eps >= 0.f) {
     float ss = 0.f;
 #pragma unroll
@@ -229,7 +238,7 @@ __device__ __forceinline__ float capped_score(float dot, float k, float cap_log2
 __device__ __forceinline__ int sm_row_swz(int row) { return (row & 3) | (((row >> 3) & 3) << 2); }
 
 struct SmMfmaParams {
-  uint16_t* out;             // [T, H * DV]
+  uint16_t* out;             // [T, H * DV], row stride o_stride
   const uint16_t* q;         // row stride q_stride, head (h, m) at (h * MAPS + m) * DK
   const uint16_t* gate;      // row stride g_stride, one value per head (nullptr: none)
   const uint16_t* kc;
@@ -242,6 +251,9 @@ struct SmMfmaParams {
   float scale_log2, lam, unit_eps, out_scale;
   float cap_log2;            // soft cap of the scores times log2 e (0: none)
   int v_row;                 // elements between value rows of a page (DV, or DK when the values lie in the key rows)
+  int chunk;                 // > 0: keys of the query's own chunk only
+  float sink_log2;           // score of a key without a value times log2 e (-inf: none)
+  int64_t o_stride;
 };
 
 // WPE: waves per SIMD the register allocation aims at. Large tiles (maps x DK + DV >= 192) are
@@ -297,19 +309,19 @@ softmax_attention_mfma_kernel(const SmMfmaParams P) {
   }
   const int qpos_lo = ctx - qlen + tile * 64;
   const int qpos_hi = ctx - qlen + min(qlen - 1, tile * 64 + 63);
-  const int lo_min = W > 0 ? max(0, qpos_lo - W + 1) : 0;
-  const int t_first = lo_min / KT, t_last = qpos_hi / KT;
-  const float fW = W > 0 ? (float)W : 3.0e38f;
+  const int t_first = first_key(qpos_lo, W, P.chunk) / KT, t_last = qpos_hi / KT;
+  const float fW = (float)(qpos - first_key(qpos, W, P.chunk) + 1);     // keys the row sees, its own included
   // positions of this wave's first and last rows
   const int wq_lo = ctx - qlen + min(qlen - 1, tile * 64 + w * 16);
   const int wq_hi = ctx - qlen + min(qlen - 1, tile * 64 + w * 16 + 15);
+  const int wk_lo = first_key(wq_hi, W, P.chunk);     // keys below it are out of sight of some row of the wave
 
   f32x4 o[MAPS][DT];
   float mrun[MAPS], lrun[MAPS];
 #pragma unroll
   for (int m = 0; m < MAPS; ++m) {
-    mrun[m] = -INFINITY;
-    lrun[m] = 0.f;
+    mrun[m] = P.sink_log2;
+    lrun[m] = P.sink_log2 == -INFINITY ? 0.f : 1.f;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) o[m][dt] = (f32x4)(0.f);
   }
@@ -376,7 +388,7 @@ softmax_attention_mfma_kernel(const SmMfmaParams P) {
 
     const int kbase = t * KT;
     const float fd = (float)(qpos - kbase - 8 * h);
-    const bool need_mask = kbase + KT - 1 > wq_lo || (W > 0 && wq_hi - kbase >= W);
+    const bool need_mask = kbase + KT - 1 > wq_lo || kbase < wk_lo;
     const bool capped = P.cap_log2 > 0.f;
     const float cap_k = capped ? 2.8853900817779268f * P.scale_log2 / P.cap_log2 : 0.f, cap_m2 = -2.0f * P.cap_log2;
     bf16x8 pf[MAPS][2];
@@ -486,7 +498,7 @@ softmax_attention_mfma_kernel(const SmMfmaParams P) {
           o[m][dt][rr] = v;
           s2 += v * v;
         }
-      float rs = 1.0f;
+      float rs = P.out_scale;
       if (P.unit_eps >= 0.f) {
         s2 += __shfl_xor(s2, 16, 64);
         s2 += __shfl_xor(s2, 32, 64);
@@ -495,7 +507,7 @@ softmax_attention_mfma_kernel(const SmMfmaParams P) {
       if (row_ok) {
         const int head = 2 * hq + m;
         if (P.gate) rs *= sigmoidf_(bf2f(P.gate[(int64_t)(q0 + r) * P.g_stride + head]));
-        uint16_t* op = P.out + (int64_t)(q0 + r) * P.H * DV + (int64_t)head * DV;
+        uint16_t* op = P.out + (int64_t)(q0 + r) * P.o_stride + (int64_t)head * DV;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) {
           u16x4 ov;
@@ -517,7 +529,7 @@ softmax_attention_mfma_kernel(const SmMfmaParams P) {
       o[0][dt][rr] = v;
       ss += v * v;
     }
-  float rs = 1.0f;
+  float rs = P.out_scale;
   if (P.unit_eps >= 0.f) {
     ss += __shfl_xor(ss, 16, 64);
     ss += __shfl_xor(ss, 32, 64);
@@ -525,7 +537,7 @@ softmax_attention_mfma_kernel(const SmMfmaParams P) {
   }
   if (!row_ok) return;
   if (P.gate) rs *= sigmoidf_(bf2f(P.gate[(int64_t)(q0 + r) * P.g_stride + hq]));
-  uint16_t* op = P.out + (int64_t)(q0 + r) * P.H * DV + (int64_t)hq * DV;
+  uint16_t* op = P.out + (int64_t)(q0 + r) * P.o_stride + (int64_t)hq * DV;
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) {
     u16x4 ov;
@@ -622,7 +634,7 @@ __device__ __forceinline__ void softmax_decode_mfma_body(
     float* __restrict__ ws, const uint16_t* __restrict__ q, int64_t q_stride, const uint16_t* __restrict__ kc,
     const uint16_t* __restrict__ vc, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ pos, int H, int G, float scale_log2, float cap_log2, int window,
-    int v_row) {
+    int v_row, int chunk) {
   constexpr int KT = 64;
   constexpr int DS = DK / 32;
   constexpr int DT = DV / 16;
@@ -638,7 +650,7 @@ __device__ __forceinline__ void softmax_decode_mfma_body(
   const int col = lane & 15, h = lane >> 4;
   const int head = g * grp + (c0 + col < grp ? c0 + col : grp - 1);
   const int i = pos[row];
-  const int lo = window > 0 && i - window + 1 > 0 ? i - window + 1 : 0;
+  const int lo = i < 0 ? 0 : first_key(i, window, chunk);
   const int p_lo = lo / KT, p_hi = i / KT;           // i < 0: no pages
   const int n_pages = i < 0 ? 0 : p_hi - p_lo + 1;
   const int stride = 4 * parts;
@@ -837,9 +849,9 @@ __global__ void __launch_bounds__(256) softmax_decode_mfma_kernel(
     float* __restrict__ ws, const uint16_t* __restrict__ q, int64_t q_stride, const uint16_t* __restrict__ kc,
     const uint16_t* __restrict__ vc, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ pos, int H, int G, float scale_log2, float cap_log2, int window,
-    int v_row) {
+    int v_row, int chunk) {
   softmax_decode_mfma_body<DK, DV, MAPS>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2,
-                                         window, v_row);
+                                         window, v_row, chunk);
 }
 
 template <int DK, int DV, int MAPS>
@@ -847,25 +859,26 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     float* __restrict__ ws, const uint16_t* __restrict__ q, int64_t q_stride, const uint16_t* __restrict__ kc,
     const uint16_t* __restrict__ vc, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ pos, int H, int G, float scale_log2, float cap_log2, int window,
-    int v_row) {
+    int v_row, int chunk) {
   softmax_decode_mfma_body<DK, DV, MAPS>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2,
-                                         window, v_row);
+                                         window, v_row, chunk);
 }
 
 // one wave per (token row, head): merge the partials of each map, a_0 - lam * a_1, unit RMS, gate
 __global__ void __launch_bounds__(64) softmax_decode_reduce_kernel(
     uint16_t* __restrict__ out, const float* __restrict__ ws, int slots, const uint16_t* __restrict__ gate,
-    int64_t g_stride, int H, int dv, int maps, float lam, float unit_eps, float out_scale) {
+    int64_t g_stride, int H, int dv, int maps, float lam, float unit_eps, float out_scale, float sink_log2,
+    int64_t o_stride) {
   const int64_t row = blockIdx.x;
   const int head = blockIdx.y, lane = threadIdx.x;
   constexpr int MAXV = 4;   // dv <= 256
   float res[MAXV] = {0.f, 0.f, 0.f, 0.f};
   for (int m = 0; m < maps; ++m) {
     const float* wp = ws + (((int64_t)row * H + head) * maps + m) * slots * (int64_t)(dv + 4);
-    float M = -INFINITY;
+    float M = sink_log2;
 #pragma unroll 4
     for (int s = 0; s < slots; ++s) M = fmaxf(M, wp[(int64_t)s * (dv + 4) + dv]);
-    float L = 0.f, acc[MAXV] = {0.f, 0.f, 0.f, 0.f};
+    float L = sink_log2 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(sink_log2 - M), acc[MAXV] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
     for (int s = 0; s < slots; ++s) {
       const float* sp = wp + (int64_t)s * (dv + 4);
@@ -881,7 +894,7 @@ __global__ void __launch_bounds__(64) softmax_decode_reduce_kernel(
 #pragma unroll
     for (int u = 0; u < MAXV; ++u) res[u] = m == 0 ? acc[u] * inv : res[u] - lam * (acc[u] * inv);
   }
-  float r = 1.0f;
+  float r = out_scale;
   if (unit_eps >= 0.f) {
     float ss = 0.f;
 #pragma unroll
@@ -893,13 +906,13 @@ __global__ void __launch_bounds__(64) softmax_decode_reduce_kernel(
   if (gate) r *= sigmoidf_(bf2f(gate[row * g_stride + head]));
 #pragma unroll
   for (int u = 0; u < MAXV; ++u)
-    if (lane + 64 * u < dv) out[(row * H + head) * (int64_t)dv + lane + 64 * u] = f2bf(res[u] * r);
+    if (lane + 64 * u < dv) out[row * o_stride + (int64_t)head * dv + lane + 64 * u] = f2bf(res[u] * r);
 }
 
 template <int DK, int DV, int MAPS>
 void launch_sm_decode_one(float* ws, const uint16_t* q, int64_t q_stride, const uint16_t* kc, const uint16_t* vc,
                           const int32_t* block_tables, int max_blocks, const int32_t* tok_seq, const int32_t* pos,
-                          int H, int G, float scale_log2, float cap_log2, int window, int v_row, dim3 grid, hipStream_t stream) {
+                          int H, int G, float scale_log2, float cap_log2, int window, int v_row, int chunk, dim3 grid, hipStream_t stream) {
   constexpr size_t tiles = (size_t)4 * DV * 64 * sizeof(uint16_t);
   constexpr size_t merge = (size_t)(4 * MAPS * 2 * 16 + MAPS * 16 * DV) * sizeof(float);
   constexpr size_t smem = tiles > merge ? tiles : merge;
@@ -912,7 +925,7 @@ void launch_sm_decode_one(float* ws, const uint16_t* q, int64_t q_stride, const 
     }
     softmax_decode_mfma_kernel_w2<DK, DV, MAPS><<<grid, 256, smem, stream>>>(ws, q, q_stride, kc, vc, block_tables,
                                                                             max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2,
-                                                                            window, v_row);
+                                                                            window, v_row, chunk);
   } else {
     if (smem > 65536 && !attr_set) {
       (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&softmax_decode_mfma_kernel<DK, DV, MAPS>),
@@ -921,15 +934,15 @@ void launch_sm_decode_one(float* ws, const uint16_t* q, int64_t q_stride, const 
     }
     softmax_decode_mfma_kernel<DK, DV, MAPS><<<grid, 256, smem, stream>>>(ws, q, q_stride, kc, vc, block_tables,
                                                                          max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2,
-                                                                         window, v_row);
+                                                                         window, v_row, chunk);
   }
 }
 
-#define NGA_SM_DEC_ARGS ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2, window, v_row, grid, stream
+#define NGA_SM_DEC_ARGS ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2, window, v_row, chunk, grid, stream
 template <int DK, int MAPS>
 bool launch_sm_decode_dv(float* ws, const uint16_t* q, int64_t q_stride, const uint16_t* kc, const uint16_t* vc,
                          const int32_t* block_tables, int max_blocks, const int32_t* tok_seq, const int32_t* pos, int H,
-                         int G, float scale_log2, float cap_log2, int window, int v_row, int dv, dim3 grid, hipStream_t stream) {
+                         int G, float scale_log2, float cap_log2, int window, int v_row, int chunk, int dv, dim3 grid, hipStream_t stream) {
   switch (dv) {
     case 32: launch_sm_decode_one<DK, 32, MAPS>(NGA_SM_DEC_ARGS); return true;
     case 64: launch_sm_decode_one<DK, 64, MAPS>(NGA_SM_DEC_ARGS); return true;
@@ -947,8 +960,8 @@ bool launch_sm_decode_dv(float* ws, const uint16_t* q, int64_t q_stride, const u
 template <int MAPS>
 bool launch_sm_decode_dk(float* ws, const uint16_t* q, int64_t q_stride, const uint16_t* kc, const uint16_t* vc,
                          const int32_t* block_tables, int max_blocks, const int32_t* tok_seq, const int32_t* pos, int H,
-                         int G, float scale_log2, float cap_log2, int window, int v_row, int dk, int dv, dim3 grid, hipStream_t stream) {
-#define NGA_SM_DEC_DV(DKV) launch_sm_decode_dv<DKV, MAPS>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2, window, v_row, dv, grid, stream)
+                         int G, float scale_log2, float cap_log2, int window, int v_row, int chunk, int dk, int dv, dim3 grid, hipStream_t stream) {
+#define NGA_SM_DEC_DV(DKV) launch_sm_decode_dv<DKV, MAPS>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2, window, v_row, chunk, dv, grid, stream)
   if (MAPS == 1) {   // key sizes of a latent plus a rotated part: one value size each
     if (dk == 96 && dv == 64) { launch_sm_decode_one<96, 64, 1>(NGA_SM_DEC_ARGS); return true; }
     if (dk == 192 && dv == 128) { launch_sm_decode_one<192, 128, 1>(NGA_SM_DEC_ARGS); return true; }
@@ -958,7 +971,7 @@ bool launch_sm_decode_dk(float* ws, const uint16_t* q, int64_t q_stride, const u
     case 32: return NGA_SM_DEC_DV(32);
     case 64: return NGA_SM_DEC_DV(64);
     case 128: return NGA_SM_DEC_DV(128);
-    case 256: return MAPS == 1 ? launch_sm_decode_dv<256, 1>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2, window, v_row, dv, grid, stream) : false;
+    case 256: return MAPS == 1 ? launch_sm_decode_dv<256, 1>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G, scale_log2, cap_log2, window, v_row, chunk, dv, grid, stream) : false;
     default: return false;
   }
 #undef NGA_SM_DEC_DV
@@ -981,24 +994,25 @@ int softmax_decode_parts(int rows, int G, int max_ctx, int window) {
 }
 
 // ws: fp32 [T, H, maps, parts, dv + 4]
-void launch_softmax_decode_mfma(uint16_t* out, float* ws, int parts, const uint16_t* q, int64_t q_stride,
+void launch_softmax_decode_mfma(uint16_t* out, int64_t o_stride, float* ws, int parts, const uint16_t* q, int64_t q_stride,
                                 const uint16_t* gate, int64_t g_stride, const uint16_t* kc, const uint16_t* vc,
                                 const int32_t* block_tables, int max_blocks, const int32_t* tok_seq,
                                 const int32_t* pos, int64_t T, int H, int G, int dk, int dv, float scale, int window,
                                 int maps, float lam, float unit_eps, float out_scale, bool v_in_k, float softcap,
-                                hipStream_t stream) {
+                                int chunk, float sink, hipStream_t stream) {
   if (T == 0) return;
   const dim3 grid((unsigned)parts, (unsigned)(G * ((H / G + 15) / 16)), (unsigned)T);
   const float scale_log2 = scale * 1.4426950408889634f;
   const float cap_log2 = softcap > 0.f ? softcap * 1.4426950408889634f : 0.f;
   const int v_row = v_in_k ? dk : dv;
   const bool ok = maps == 2 ? launch_sm_decode_dk<2>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G,
-                                                     scale_log2, cap_log2, window, v_row, dk, dv, grid, stream)
+                                                     scale_log2, cap_log2, window, v_row, chunk, dk, dv, grid, stream)
                             : launch_sm_decode_dk<1>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G,
-                                                     scale_log2, cap_log2, window, v_row, dk, dv, grid, stream);
+                                                     scale_log2, cap_log2, window, v_row, chunk, dk, dv, grid, stream);
   if (!ok) abort();   // the caller checks softmax_attention_mfma_supported
   softmax_decode_reduce_kernel<<<dim3((unsigned)T, (unsigned)H), 64, 0, stream>>>(out, ws, parts, gate, g_stride, H,
-                                                                                   dv, maps, lam, unit_eps, out_scale);
+                                                                                   dv, maps, lam, unit_eps, out_scale,
+                                                                                   sink * 1.4426950408889634f, o_stride);
 }
 
 // Head sizes of the MFMA forms: dk, dv in {32, 64, 128} (one map: also 256, and the pairs
@@ -1012,16 +1026,17 @@ bool softmax_attention_mfma_supported(int dk, int dv, int group, int maps) {
 
 // prompt portions: sequence b owns rows [cu_q[b], cu_q[b + 1]) of q / gate / out, the last ones of
 // its ctx_lens[b] keys. q rows must be 16-byte aligned (checked by the caller).
-void launch_softmax_attention_mfma(uint16_t* out, const uint16_t* q, int64_t q_stride, const uint16_t* gate,
+void launch_softmax_attention_mfma(uint16_t* out, int64_t o_stride, const uint16_t* q, int64_t q_stride, const uint16_t* gate,
                                    int64_t g_stride, const uint16_t* kc, const uint16_t* vc,
                                    const int32_t* block_tables, int max_blocks, const int32_t* cu_q,
                                    const int32_t* ctx_lens, int B, int max_q_len, int H, int G, int dk, int dv,
                                    float scale, int window, int maps, float lam, float unit_eps, float out_scale,
-                                   bool v_in_k, float softcap, hipStream_t stream) {
+                                   bool v_in_k, float softcap, int chunk, float sink, hipStream_t stream) {
   if (B == 0 || max_q_len == 0) return;
   SmMfmaParams P{out, q, gate, kc, vc, block_tables, cu_q, ctx_lens, q_stride, g_stride, max_blocks, H, G, window,
                  scale * 1.4426950408889634f, lam, unit_eps, out_scale,
-                 softcap > 0.f ? softcap * 1.4426950408889634f : 0.f, v_in_k ? dk : dv};
+                 softcap > 0.f ? softcap * 1.4426950408889634f : 0.f, v_in_k ? dk : dv, chunk,
+                 sink * 1.4426950408889634f, o_stride};
   const dim3 grid((unsigned)H, (unsigned)B, (unsigned)((max_q_len + 63) / 64));   // (head, sequence, row block)
   const bool ok = maps == 2 ? launch_sm_mfma_dk<2>(P, dk, dv, grid, stream) : launch_sm_mfma_dk<1>(P, dk, dv, grid, stream);
   if (!ok) abort();   // the caller checks softmax_attention_mfma_supported
@@ -1041,11 +1056,11 @@ void launch_headnorm_cache(void* proj, int64_t stride, const int32_t* slots, voi
                                                                           dv, eps, qw, kw, bias, pos, coef, every);
 }
 
-void launch_softmax_attention(void* out, const void* q, int64_t q_stride, const void* gate, int64_t g_stride,
+void launch_softmax_attention(void* out, int64_t o_stride, const void* q, int64_t q_stride, const void* gate, int64_t g_stride,
                               const void* kc, const void* vc, const int32_t* block_tables, int max_blocks,
                               const int32_t* tok_seq, const int32_t* pos, int64_t T, int H, int G, int dk, int dv,
                               float scale, int window, int maps, float lam, float unit_eps, float out_scale, bool v_in_k,
-                              float softcap, bool f32, hipStream_t stream) {
+                              float softcap, int chunk, float sink, bool f32, hipStream_t stream) {
   if (T == 0) return;
   const int v_row = v_in_k ? dk : dv;
   const dim3 grid((unsigned)T, (unsigned)H);
@@ -1054,12 +1069,12 @@ void launch_softmax_attention(void* out, const void* q, int64_t q_stride, const 
     softmax_attention_kernel<float><<<grid, 64, smem, stream>>>(
         (float*)out, (const float*)q, q_stride, (const float*)gate, g_stride, (const float*)kc, (const float*)vc,
         block_tables, max_blocks, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam, unit_eps, out_scale, v_row,
-        softcap);
+        softcap, chunk, sink, o_stride);
   else
     softmax_attention_kernel<uint16_t><<<grid, 64, smem, stream>>>(
         (uint16_t*)out, (const uint16_t*)q, q_stride, (const uint16_t*)gate, g_stride, (const uint16_t*)kc,
         (const uint16_t*)vc, block_tables, max_blocks, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam, unit_eps,
-        out_scale, v_row, softcap);
+        out_scale, v_row, softcap, chunk, sink, o_stride);
 }
 
 }  // namespace nga

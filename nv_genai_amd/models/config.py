@@ -562,12 +562,15 @@ class RotarySpec:
     ``p * f_i`` at position p, ``f_i = base^(-2i / dims)``. ``interleaved``: pair i is elements
     (2i, 2i + 1), else (i, i + dims / 2). ``yarn`` = (factor, original, fast, slow) or None: the
     frequencies of slow pairs are divided by ``factor`` along a linear ramp over the pair index,
-    and cos / sin are multiplied by ``0.1 ln(factor) + 1`` (:func:`ops.rotary_frequencies`)."""
+    and cos / sin are multiplied by ``0.1 ln(factor) + 1``. ``bands`` = (factor, low, high, original)
+    or None: the frequencies are divided by ``factor`` along a ramp over the wavelength, from
+    ``original / high`` to ``original / low`` (:func:`ops.rotary_frequencies`)."""
 
     dims: int
     base: float
     interleaved: bool = False
     yarn: Optional[tuple] = None
+    bands: Optional[tuple] = None
 
 
 @dataclass(frozen=True)
@@ -1048,3 +1051,246 @@ def lizezen_layers(pattern: Sequence[str], hidden: int, heads: int, kv_heads: in
         blocks.append(LizezenLayer(t, m, mlp))
     return LizezenConfig(name=name, vocab_size=vocab_size, hidden=hidden, eps=eps, blocks=tuple(blocks),
                          loop=None if not loop else LoopSpec(*loop))
+
+
+# ---------------------------------------------------------------------------------------------
+# Vivesun: pre-norm layers on an fp32 stream with a bigram embedding and a per-layer token input;
+# delta-rule recurrences, one of them side by side with chunked attention.
+@dataclass(frozen=True)
+class GatedDeltaSpec:
+    """Mixer ``delta``: per head a matrix memory with one decay per token, ``S <- g S``,
+    ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q`` on unit keys and queries; q, k, v pass a
+    causal convolution of ``conv`` taps per channel and silu; head h reads q / k head
+    ``h // (heads / kv_heads)``."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+
+
+@dataclass(frozen=True)
+class ChunkedAttentionSpec:
+    """Softmax attention with GQA, rotary positions on the first ``rot.dims`` elements and a sink of
+    score 0 without a value (one added to the denominator). ``chunk`` > 0: position i sees
+    ``j <= i`` of its own chunk of ``chunk`` positions only (0: all of them)."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot: RotarySpec
+    chunk: int = 0
+
+
+@dataclass(frozen=True)
+class ChannelDeltaSpec:
+    """Generalised delta rule with a decay and a removal rate per key channel:
+    ``S <- diag(w) S - (a u)(u^T S) + k v^T``, ``o = S^T r`` with u the unit key. ``decay_rank``: rank
+    of the decay's low-rank projection (0: as the checkpoint's tensors have it)."""
+
+    heads: int
+    dim: int
+    decay_rank: int = 0
+
+
+@dataclass(frozen=True)
+class ParallelSpec:
+    """Mixer ``parallel``: ``left_scale * left(h) + right_scale * right(h)``."""
+
+    left: ChunkedAttentionSpec
+    right: ChannelDeltaSpec
+    left_scale: float
+    right_scale: float
+
+
+@dataclass(frozen=True)
+class PlainMoeSpec:
+    """``experts`` experts ``down(gelu(up x))`` (erf gelu) of ``ff`` features of which a token uses the
+    ``top`` with the largest softmax score; weights: the chosen scores divided by their sum, times
+    ``scale``."""
+
+    experts: int
+    top: int
+    ff: int
+    scale: float = 1.0
+    kind: str = "moe"
+
+
+@dataclass(frozen=True)
+class BigramSpec:
+    """Bigram embedding: row ``(previous * mul_prev + current * mul_cur) mod buckets``; row
+    ``buckets`` for a sequence's first token."""
+
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+
+
+@dataclass(frozen=True)
+class VivesunLayer:
+    type: str                 # "delta" | "parallel"
+    mixer: object
+    mlp: Optional[PlainMoeSpec] = None
+
+
+_VIVESUN_MIXERS = ("delta", "parallel")
+
+
+@dataclass(frozen=True)
+class VivesunConfig:
+    """Vivesun: ``x += mixer(norm1(x))``, ``x += ff(norm2(x))`` on an fp32 stream, then a per-layer
+    token input of ``side_dim`` elements (0: none); RMS norms with weights stored around zero,
+    logits from the embedding table. Every size and every constant that can differ between models
+    comes from config.json (:meth:`from_dict`)."""
+
+    name: str = "vivesun"
+    vocab_size: int = 512
+    hidden: int = 128
+    eps: float = 1e-6
+    blocks: tuple = ()
+    bigram: Optional[BigramSpec] = None
+    side_dim: int = 0
+    max_position: int = 1 << 20     # no position table: only the engine's bookkeeping is bounded
+    arch: str = "vivesun"
+    bos_id: int = 0
+    eos_ids: tuple = ()
+    chat_format: str = "plain"
+
+    @property
+    def layers(self) -> int:
+        return len(self.blocks)
+
+    @property
+    def is_moe(self) -> bool:
+        return any(b.mlp is not None for b in self.blocks)
+
+    @property
+    def experts_per_tok(self) -> int:
+        """Largest top-k of any layer (sizes the engine's routing workspace)."""
+        return max([b.mlp.top for b in self.blocks if b.mlp is not None] or [1])
+
+    @property
+    def num_experts(self) -> int:
+        return max([b.mlp.experts for b in self.blocks if b.mlp is not None] or [0])
+
+    @staticmethod
+    def _rot(r: dict, what: str, dim: int) -> RotarySpec:
+        sc = r.get("scaling")
+        rot = RotarySpec(dims=int(r["dims"]), base=float(r["base"]),
+                         bands=None if not sc else tuple(float(sc[k]) for k in ("factor", "low", "high", "original")))
+        if rot.dims % 2 or not 0 < rot.dims <= dim:
+            raise ValueError(f"{what}: rot.dims must be even and at most dim")
+        return rot
+
+    @classmethod
+    def _attention(cls, m: dict, what: str) -> ChunkedAttentionSpec:
+        dim = int(m["dim"])
+        a = ChunkedAttentionSpec(heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=dim,
+                                 vdim=int(m.get("vdim", dim)), scale=float(m["scale"]), rot=cls._rot(m["rot"], what, dim),
+                                 chunk=int((m.get("mask") or {}).get("size") or 0))
+        if min(a.heads, a.kv_heads, a.dim, a.vdim) < 1 or a.heads % a.kv_heads or a.chunk < 0:
+            raise ValueError(f"{what}: heads must be a multiple of kv_heads and sizes positive")
+        return a
+
+    @classmethod
+    def from_dict(cls, d: dict, name: str = "vivesun") -> "VivesunConfig":
+        blocks = []
+        for i, b in enumerate(d["layers"]):
+            t, m, what = b["type"], b["mixer"], f"layer {i}"
+            if t == "delta":
+                mixer = GatedDeltaSpec(heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]),
+                                       vdim=int(m.get("vdim", m["dim"])), conv=int(m["conv"]))
+                if min(mixer.heads, mixer.kv_heads, mixer.dim, mixer.vdim, mixer.conv) < 1 or mixer.heads % mixer.kv_heads:
+                    raise ValueError(f"{what}: heads must be a multiple of kv_heads and sizes positive")
+            elif t == "parallel":
+                r = m["right"]
+                mixer = ParallelSpec(left=cls._attention(m["left"], what),
+                                     right=ChannelDeltaSpec(heads=int(r["heads"]), dim=int(r["dim"]),
+                                                            decay_rank=int(r.get("decay_rank") or 0)),
+                                     left_scale=float(m["left_scale"]), right_scale=float(m["right_scale"]))
+                if min(mixer.right.heads, mixer.right.dim) < 1:
+                    raise ValueError(f"{what}: sizes must be positive")
+            else:
+                raise ValueError(f"{what}: unknown mixer type {t!r} (known: {_VIVESUN_MIXERS})")
+            mlp = b.get("mlp")
+            if mlp is not None:
+                if mlp.get("kind", "moe") != "moe":
+                    raise ValueError(f"{what}: unknown feed-forward kind {mlp['kind']!r}")
+                r = mlp["router"]
+                mlp = PlainMoeSpec(experts=int(r["experts"]), top=int(r["top"]), ff=int(mlp["expert"]["ff"]),
+                                   scale=float(r.get("scale", 1.0)))
+                if not 1 <= mlp.top <= mlp.experts or mlp.ff < 1:
+                    raise ValueError(f"{what}: top {mlp.top} of {mlp.experts} experts")
+            blocks.append(VivesunLayer(type=t, mixer=mixer, mlp=mlp))
+        bg = (d.get("embedding") or {}).get("bigram")
+        bigram = None
+        if bg:
+            bigram = BigramSpec(buckets=int(bg["buckets"]), mul_prev=int(bg["mul_prev"]), mul_cur=int(bg["mul_cur"]))
+            if bigram.buckets < 1 or min(bigram.mul_prev, bigram.mul_cur) < 0:
+                raise ValueError("bigram embedding: buckets must be positive, multipliers not negative")
+        return cls(name=name, vocab_size=int(d["vocab"]), hidden=int(d["width"]), eps=float(d["norm"]["eps"]),
+                   blocks=tuple(blocks), bigram=bigram, side_dim=int((d.get("token_side") or {}).get("dim") or 0))
+
+    def to_json_dict(self) -> dict:
+        """The config.json form (inverse of :meth:`from_dict`)."""
+        layers = []
+        for b in self.blocks:
+            m = b.mixer
+            if b.type == "delta":
+                mx = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim, "vdim": m.vdim, "conv": m.conv}
+            else:
+                a, r = m.left, m.right
+                rot = {"base": a.rot.base, "dims": a.rot.dims}
+                if a.rot.bands:
+                    rot["scaling"] = dict(zip(("factor", "low", "high", "original"), a.rot.bands))
+                left = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim, "scale": a.scale, "rot": rot}
+                if a.chunk:
+                    left["mask"] = {"size": a.chunk}
+                right = {"heads": r.heads, "dim": r.dim}
+                if r.decay_rank:
+                    right["decay_rank"] = r.decay_rank
+                mx = {"left": left, "right": right, "left_scale": m.left_scale, "right_scale": m.right_scale}
+            f = b.mlp
+            ff = None if f is None else {"kind": "moe", "router": {"experts": f.experts, "top": f.top, "scale": f.scale},
+                                         "expert": {"ff": f.ff}}
+            layers.append({"type": b.type, "mixer": mx, "mlp": ff})
+        out = {"architecture": "Vivesun", "vocab": self.vocab_size, "width": self.hidden, "norm": {"eps": self.eps},
+               "layers": layers}
+        if self.bigram is not None:
+            g = self.bigram
+            out["embedding"] = {"bigram": {"buckets": g.buckets, "mul_prev": g.mul_prev, "mul_cur": g.mul_cur}}
+        if self.side_dim:
+            out["token_side"] = {"dim": self.side_dim}
+        return out
+
+    def to_dict(self):
+        return asdict(self)
+
+
+def vivesun_layers(pattern: Sequence[str], hidden: int, heads: int, kv_heads: int, dim: int, vdim: int, chunk: int = 0,
+                   delta_heads: int = 0, delta_kv_heads: int = 0, delta_dim: int = 0, delta_vdim: int = 0, conv: int = 4,
+                   right_heads: int = 0, right_dim: int = 0, decay_rank: int = 64, left_scale: float = 1.0,
+                   right_scale: float = 1.0, experts: int = 0, top: int = 2, expert_ff: int = 0, route_scale: float = 1.0,
+                   rot_base: float = 500000.0, rot_dims: int = 0, bands: Optional[tuple] = None,
+                   bigram: Optional[tuple] = None, side_dim: int = 0, vocab_size: int = 32768, eps: float = 1e-6,
+                   name: str = "vivesun") -> VivesunConfig:
+    """A Vivesun config from a pattern of mixer types with the same sizes in every layer of a kind
+    (benchmarks, tests). ``experts`` 0: no feed-forwards. ``bigram`` = (buckets, mul_prev, mul_cur)."""
+    blocks = []
+    for t in pattern:
+        if t == "delta":
+            m = GatedDeltaSpec(delta_heads or heads, delta_kv_heads or delta_heads or heads, delta_dim or dim,
+                               delta_vdim or vdim, conv)
+        elif t == "parallel":
+            left = ChunkedAttentionSpec(heads, kv_heads, dim, vdim, dim ** -0.5,
+                                        RotarySpec(rot_dims or dim, rot_base, bands=bands), chunk)
+            m = ParallelSpec(left, ChannelDeltaSpec(right_heads or heads, right_dim or dim, decay_rank), left_scale,
+                             right_scale)
+        else:
+            raise ValueError(f"unknown mixer type {t!r}")
+        blocks.append(VivesunLayer(t, m, PlainMoeSpec(experts, top, expert_ff, route_scale) if experts else None))
+    return VivesunConfig(name=name, vocab_size=vocab_size, hidden=hidden, eps=eps, blocks=tuple(blocks),
+                         bigram=None if not bigram else BigramSpec(*bigram), side_dim=side_dim)

@@ -503,17 +503,22 @@ def softcap_(z: torch.Tensor, cap: float) -> torch.Tensor:
 
 
 def group_rmsnorm(x: torch.Tensor, w: torch.Tensor, groups: int, eps: float, dtype: torch.dtype,
-                  gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  gate: Optional[torch.Tensor] = None, gate_act: str = "sigmoid",
+                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """RMS norm of each of ``groups`` equal column groups of fp32 rows, written in ``dtype``. ``w``
     (fp32) holds one weight per element of a group, shared by the groups, or one per column of the
     row. ``gate`` [T, columns] (rows of the activation type, any row stride): the result is
-    multiplied by ``sigmoid(gate)``."""
+    multiplied by ``sigmoid(gate)`` or ``silu(gate)`` (``gate_act``). ``out``: rows of any stride."""
+    if gate_act not in ("sigmoid", "silu"):
+        raise ValueError(f"unknown gate activation {gate_act!r}")
     if w.numel() not in (x.shape[1] // groups, x.shape[1]):
         raise ValueError("group_rmsnorm: one weight per group element or per column")
     if not _gpu(x):
-        return ref.group_rmsnorm(x, w, groups, eps, dtype, gate)
-    out = torch.empty(x.shape, dtype=dtype, device=x.device)
-    kernels().group_rmsnorm(out, x, w, int(groups), float(eps), gate)
+        r = ref.group_rmsnorm(x, w, groups, eps, dtype, gate, gate_act)
+        return r if out is None else out.copy_(r)
+    if out is None:
+        out = torch.empty(x.shape, dtype=dtype, device=x.device)
+    kernels().group_rmsnorm(out, x, w, int(groups), float(eps), gate, gate_act == "silu")
     return out
 
 
@@ -536,30 +541,35 @@ def headnorm_cache_(proj, slots, kc, vc, nq: int, nk: int, dk: int, nv: int, dv:
 
 def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk: int, dv: int, scale: float,
                       window: int = 0, maps: int = 1, lam: float = 0.0, unit_eps: Optional[float] = None,
-                      out_scale: float = 1.0, gate=None, out=None, v_in_k: bool = False, softcap: float = 0.0):
+                      out_scale: float = 1.0, gate=None, out=None, v_in_k: bool = False, softcap: float = 0.0,
+                      chunk: int = 0, sink: Optional[float] = None):
     """Softmax attention of token rows (prompt portions and single-token rows alike) over row-
     major pages K [blocks, G * maps, 64, dk], V [blocks, G, 64, dv]. The query at position i
     sees keys ``j <= i`` (``window`` > 0: and ``i - j < window``). ``maps`` (1 or 2) score maps per
     head: q head (h, m) is column block ``h * maps + m``, its keys are k head
     ``(h // (H / G)) * maps + m``, both maps read v head ``h // (H / G)``; two maps combine as
     ``a_0 - lam * a_1`` (differential attention). ``unit_eps``: divide every head's output by its
-    root mean square (eps inside the root) and multiply by ``out_scale``. ``gate`` [T, H]: the
-    head outputs are multiplied by ``sigmoid(gate)``. ``tok_seq[t]`` is the block-table row of
+    root mean square (eps inside the root). The outputs are multiplied by ``out_scale``, and with
+    ``gate`` [T, H] by ``sigmoid(gate)`` of their head. ``tok_seq[t]`` is the block-table row of
     token t, ``pos[t]`` its position (negative: padding row, zeros out). Scores, softmax and
     accumulation are fp32. ``v_in_k`` (one map, dv <= dk): the values are the first dv elements of
     the key rows (``vc`` is not read) - keys with extra key-only columns behind a shared latent.
-    ``softcap`` > 0: a score s becomes ``softcap * tanh(s / softcap)`` before the softmax."""
+    ``softcap`` > 0: a score s becomes ``softcap * tanh(s / softcap)`` before the softmax. ``chunk``
+    > 0: only keys of the query's own chunk of ``chunk`` positions (counted from position 0) are
+    seen. ``sink``: score of one more key that has no value (0.0: one added to the denominator).
+    ``out``: rows of any stride."""
     if v_in_k and (maps != 1 or dv > dk):
         raise ValueError("values inside the key rows: one map and dv <= dk")
     if not _gpu(q):
-        return ref.softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam,
-                                     unit_eps, out_scale, gate, v_in_k, softcap)
+        r = ref.softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam,
+                                  unit_eps, out_scale, gate, v_in_k, softcap, chunk, sink)
+        return r if out is None else out.copy_(r)
     if out is None:
         out = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
     kernels().softmax_attention(out, q, gate, kc, kc if v_in_k else vc, block_tables, tok_seq, pos, H, G, dk, dv,
                                 float(scale), int(window), int(maps), float(lam),
                                 -1.0 if unit_eps is None else float(unit_eps), float(out_scale), bool(v_in_k),
-                                float(softcap))
+                                float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 
 
@@ -583,14 +593,15 @@ def _rows_of_portions(cu_q, ctx_lens, T: int, dev):
 def softmax_attention_prefill(q, kc, vc, block_tables, cu_q, ctx_lens, max_q_len: int, H: int, G: int, dk: int,
                               dv: int, scale: float, window: int = 0, maps: int = 1, lam: float = 0.0,
                               unit_eps: Optional[float] = None, out_scale: float = 1.0, gate=None, out=None,
-                              v_in_k: bool = False, softcap: float = 0.0):
+                              v_in_k: bool = False, softcap: float = 0.0, chunk: int = 0,
+                              sink: Optional[float] = None):
     """:func:`softmax_attention` of prompt portions on MFMA tiles: sequence b owns token rows
     ``[cu_q[b], cu_q[b + 1])``, the last ones of its ``ctx_lens[b]`` keys. Rows the tile kernel
     does not take (fp32, other head sizes, CPU) run the row form."""
     if not softmax_attention_mfma_ok(q, dk, dv, H // G, maps):
         seq, pos = _rows_of_portions(cu_q, ctx_lens, q.shape[0], q.device)
         return softmax_attention(q, kc, vc, block_tables, seq, pos, H, G, dk, dv, scale, window, maps, lam, unit_eps,
-                                 out_scale, gate, out=out, v_in_k=v_in_k, softcap=softcap)
+                                 out_scale, gate, out=out, v_in_k=v_in_k, softcap=softcap, chunk=chunk, sink=sink)
     if v_in_k and (maps != 1 or dv > dk):
         raise ValueError("values inside the key rows: one map and dv <= dk")
     if out is None:
@@ -598,14 +609,14 @@ def softmax_attention_prefill(q, kc, vc, block_tables, cu_q, ctx_lens, max_q_len
     kernels().softmax_attention_prefill(out, q, gate, kc, kc if v_in_k else vc, block_tables, cu_q, ctx_lens,
                                         int(max_q_len), H, G, dk, dv, float(scale), int(window), int(maps), float(lam),
                                         -1.0 if unit_eps is None else float(unit_eps), float(out_scale), bool(v_in_k),
-                                        float(softcap))
+                                        float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 
 
 def softmax_attention_rows(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk: int, dv: int, scale: float,
                            max_ctx: int, window: int = 0, maps: int = 1, lam: float = 0.0,
                            unit_eps: Optional[float] = None, out_scale: float = 1.0, gate=None, out=None,
-                           v_in_k: bool = False, softcap: float = 0.0):
+                           v_in_k: bool = False, softcap: float = 0.0, chunk: int = 0, sink: Optional[float] = None):
     """:func:`softmax_attention` of single-token rows (decode rows; any rows work) on the page-
     parallel MFMA kernel: the query heads that share a KV head are the columns of one tile, so a
     page is read once per group; the visible pages of a row are split over several workgroups
@@ -613,19 +624,20 @@ def softmax_attention_rows(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int
     normalises and gates. ``max_ctx`` bounds the rows' positions (launch shape)."""
     if not softmax_attention_mfma_ok(q, dk, dv, H // G, maps):
         return softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam,
-                                 unit_eps, out_scale, gate, out=out, v_in_k=v_in_k, softcap=softcap)
+                                 unit_eps, out_scale, gate, out=out, v_in_k=v_in_k, softcap=softcap, chunk=chunk,
+                                 sink=sink)
     if v_in_k and (maps != 1 or dv > dk):
         raise ValueError("values inside the key rows: one map and dv <= dk")
     C = kernels()
     T = q.shape[0]
-    parts = int(C.softmax_decode_parts(max(T, 1), G * -(-(H // G) // 16), int(max_ctx), int(window)))
+    parts = int(C.softmax_decode_parts(max(T, 1), G * -(-(H // G) // 16), int(max_ctx), int(min(window or chunk, chunk or window))))
     ws = torch.empty(T * H * maps * parts * (dv + 4), dtype=torch.float32, device=q.device)
     if out is None:
         out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
     C.softmax_attention_decode(out, ws, parts, q, gate, kc, kc if v_in_k else vc, block_tables, tok_seq, pos, H, G, dk,
                                dv, float(scale), int(window), int(maps), float(lam),
                                -1.0 if unit_eps is None else float(unit_eps), float(out_scale), bool(v_in_k),
-                               float(softcap))
+                               float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 
 
@@ -643,18 +655,24 @@ def residual_add_rmsnorm_(x: torch.Tensor, y: torch.Tensor, w: Optional[torch.Te
     return out
 
 
-def rotary_frequencies(dims: int, base: float, yarn=None) -> Tuple[torch.Tensor, float]:
+def rotary_frequencies(dims: int, base: float, yarn=None, bands=None) -> Tuple[torch.Tensor, float]:
     """(float64 frequencies [dims / 2], factor on cos and sin) of rotary positions on ``dims``
     elements: ``f_i = base^(-2i / dims)``. ``yarn`` = (factor, original, fast, slow): with
     ``pair(t) = dims ln(original / (2 pi t)) / (2 ln base)`` the index of the pair that turns t
     times in ``original`` positions, ``lo = max(floor(pair(fast)), 0)``,
     ``hi = min(ceil(pair(slow)), dims - 1)`` and ``ramp_i = clamp((i - lo) / max(hi - lo, 0.001),
     0, 1)``, the frequency is ``f_i / factor * ramp_i + f_i (1 - ramp_i)`` and cos / sin are
-    multiplied by ``0.1 ln(factor) + 1``."""
-    import math
-
+    multiplied by ``0.1 ln(factor) + 1``. ``bands`` = (factor, low, high, original): by wavelength
+    ``l = 2 pi / f`` a frequency stays (``l < original / high``), is divided by ``factor``
+    (``l > original / low``) or is ``(1 - s) f / factor + s f`` with
+    ``s = (original / l - low) / (high - low)`` in between."""
     i = torch.arange(dims // 2, dtype=torch.float64)
     f = torch.tensor([float(base) ** (-2.0 * k / dims) for k in range(dims // 2)], dtype=torch.float64)
+    if bands:
+        factor, low, high, orig = (float(v) for v in bands)
+        turns = orig * f / (2.0 * math.pi)                       # original / wavelength
+        t = ((turns - low) / (high - low)).clamp(0.0, 1.0) if high != low else (turns > high).double()
+        f = (1.0 - t) * f / factor + t * f
     if not yarn:
         return f, 1.0
     factor, orig, fast, slow = (float(v) for v in yarn)
@@ -833,6 +851,145 @@ def mlstm_scan(proj, gate_bias, state, H: int, d: int, dv: int, cap: float, cu, 
     kernels().mlstm_scan(out, proj, gate_bias, state, int(H), int(d), int(dv), float(cap), cu, slots, pos, q_off, k_off,
                          v_off, g_off)
     return out
+
+
+# ------------------------------------------------------------------------- bigram embedding, token inputs, short convolution
+def bigram_embed(ids: torch.Tensor, embed: torch.Tensor, table: torch.Tensor, src: torch.Tensor, prev: torch.Tensor,
+                 mul_prev: int, mul_cur: int, save_slots: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """fp32 residual rows ``embed[id] + table[row]`` with
+    ``row = (previous id * mul_prev + id * mul_cur) mod buckets`` (``buckets`` = table rows - 1; 64-bit
+    integers), or the table's last row for a sequence's first token. ``src`` says where a row's
+    previous token is (as in :func:`token_shift`): a row of this step (>= 0), nowhere (-1), or the
+    sequence's slot ``-(src + 2)`` of ``prev`` (int32). ``save_slots`` (steps of single rows only): the slot
+    that takes the row's id afterwards; longer portions save with :func:`token_save_`."""
+    if table.shape[0] < 2 or table.shape[1] != embed.shape[1]:
+        raise ValueError("bigram table: [buckets + 1, width] with at least one bucket")
+    if not _gpu(embed):
+        x = ref.bigram_embed(ids, embed, table, src, prev, mul_prev, mul_cur)
+        if save_slots is not None:
+            ref.token_save_(prev, ids, torch.arange(ids.numel(), device=ids.device), save_slots)
+        return x
+    x = torch.empty(ids.numel(), embed.shape[1], dtype=torch.float32, device=embed.device)
+    kernels().bigram_embed(x, ids, embed, table, src, prev, int(mul_prev), int(mul_cur), save_slots)
+    return x
+
+
+def token_save_(prev: torch.Tensor, ids: torch.Tensor, last_row: torch.Tensor, slot: torch.Tensor) -> torch.Tensor:
+    """``prev[slot[i]] = ids[last_row[i]]`` for every sequence of the step (negative: skipped)."""
+    if not _gpu(prev):
+        return ref.token_save_(prev, ids, last_row, slot)
+    kernels().token_save(prev, ids, last_row, slot)
+    return prev
+
+
+def gelu_gate_rows(z: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, off: int) -> torch.Tensor:
+    """``gelu_tanh(z) * table[id, off : off + columns]``: rows gated on their token's own vector."""
+    if off < 0 or off + z.shape[1] > table.shape[1]:
+        raise ValueError("columns outside the token table")
+    if not _gpu(z):
+        return ref.gelu_gate_rows(z, ids, table, off)
+    out = torch.empty(z.shape, dtype=z.dtype, device=z.device)
+    kernels().gelu_gate_rows(out, z, ids, table, int(off))
+    return out
+
+
+def residual_add_cast_(x: torch.Tensor, y: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
+    """``x += y`` on an fp32 stream in place, and a copy of the sum in ``dtype``."""
+    out = torch.empty(x.shape, dtype=dtype, device=x.device)
+    if not _gpu(x):
+        return ref.residual_add_cast_(x, y, out)
+    kernels().residual_add_rmsnorm(x, y, None, 0.0, out)
+    return out
+
+
+def tanh_rows(x: torch.Tensor) -> torch.Tensor:
+    """tanh of rows of any stride (a column slice), contiguous result."""
+    if not _gpu(x):
+        return ref.tanh_rows(x)
+    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    kernels().tanh_rows(out, x)
+    return out
+
+
+def short_conv(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, cu, slots, seq, pos) -> torch.Tensor:
+    """Causal convolution over time per channel, then silu: ``silu(sum_j taps[n - 1 - j, c] x[t - j, c])``
+    of rows x [T, C] (any row stride), ``taps`` fp32 [n, C] (last row: the current input), zeros
+    before the start. Segments as in the scans: rows ``cu[b] .. cu[b + 1]`` (``cu`` None: row b
+    alone) of one sequence, ``seq`` the segment of every row; the n - 1 inputs in front of a segment
+    come from ``state[slots[b]]`` ([slots, n - 1, C] of the rows' type, oldest first) and the slot
+    takes the segment's last n - 1. fp32 sums, result [T, C] in the rows' type."""
+    n = taps.shape[0]
+    if state.shape[1:] != (n - 1, x.shape[1]) or taps.shape[1] != x.shape[1] or not 1 <= n <= 16:
+        raise ValueError("short_conv: state [slots, taps - 1, channels], at most 16 taps")
+    if not _gpu(x):
+        return ref.short_conv(x, taps, state, cu, slots, seq, pos)
+    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    kernels().short_conv(out, x, taps, state, cu, slots, seq, pos)
+    return out
+
+
+# ------------------------------------------------------------------------- delta-rule recurrences
+DELTA_CHUNK = 16        # rows per block of the matrix form
+
+
+def _delta_workspace(T: int, n_seg: int, H: int, d: int, device) -> torch.Tensor:
+    """Block operands of the matrix form: one entry per (block, head), see csrc/kernels/delta.hip."""
+    D = 16 * int(kernels().delta_key_tiles(d))
+    return torch.empty((T // DELTA_CHUNK + n_seg) * H * (65 * D + 256), dtype=torch.float32, device=device)
+
+
+def gated_delta_scan(x, ba, a_log, dt_bias, state, H: int, G: int, d: int, dv: int, cu, slots, pos, n_single: int = 0,
+                     max_q: int = 0) -> torch.Tensor:
+    """Gated delta rule over a step's rows. ``x`` rows ``[q (G*d) | k (G*d) | v (H*dv)]`` (convolved), ``ba``
+    rows ``[b (H) | a (H)]``; head h reads q / k head ``h // (H / G)``. In fp32: q and k to unit vectors
+    (``/ sqrt(sum x^2 + 1e-6)``), ``q *= d^-0.5``, ``beta = sigmoid(b)``,
+    ``g = exp(-exp(a_log) softplus(a + dt_bias))``, then per row ``S <- g S``, ``u = beta (v - S^T k)``,
+    ``S <- S + k u^T``, ``o = S^T q``. Segment b is rows ``cu[b] .. cu[b + 1]`` (``cu`` None: row b alone) of one
+    sequence; its state [H, d, dv] (fp32) comes from ``state[slots[b]]``, or zeros when the segment
+    starts at position 0 - a reused slot needs no clearing - and goes back there. ``slots[b]`` < 0:
+    nothing is read or kept. Returns the fp32 outputs [T, H*dv].
+
+    GPU: single rows (``cu`` None, or the first ``n_single`` segments) take the row kernel; portions (at
+    most ``max_q`` rows each) the matrix form: blocks of 16 rows become fp32 MFMA operands that do
+    not depend on the state, and a second kernel walks the blocks with the state in registers."""
+    if not _gpu(x):
+        return ref.gated_delta_scan(x, ba, a_log, dt_bias, state, H, G, d, dv, cu, slots, pos)
+    T = x.shape[0]
+    out = torch.empty(T, H * dv, dtype=torch.float32, device=x.device)
+    q, k, v = x[:, :G * d], x[:, G * d:2 * G * d], x[:, 2 * G * d:2 * G * d + H * dv]
+    _delta(out, q, k, v, ba[:, H:2 * H], ba[:, :H], a_log, dt_bias, state, 0, H, G, d, dv, 0.0, cu, slots, pos, n_single, max_q)
+    return out
+
+
+def channel_delta_scan(r, k, v, a, w, a_bias, w_bias, state, H: int, d: int, dv: int, decay: float, cu, slots, pos,
+                       n_single: int = 0, max_q: int = 0) -> torch.Tensor:
+    """Delta rule with a decay and a removal rate per key channel over a step's rows: r, k, a, w rows
+    [T, H*d], v [T, H*dv] (any row strides). In fp32: ``a = sigmoid(a + a_bias)``,
+    ``w = exp(-decay sigmoid(w + w_bias))``, ``u = k / sqrt(sum k^2 + 1e-6)`` per head, then per row
+    ``S <- diag(w) S - (a u)(u^T S) + k v^T`` (both terms on the old state), ``o = S^T r``. Segments, state
+    and forms as in :func:`gated_delta_scan`. ``decay`` is at most 4: the matrix form divides by the
+    decay of up to 16 rows."""
+    if not 0.0 <= decay <= 4.0:
+        raise ValueError("channel_delta_scan: decay in [0, 4]")
+    if not _gpu(r):
+        return ref.channel_delta_scan(r, k, v, a, w, a_bias, w_bias, state, H, d, dv, decay, cu, slots, pos)
+    out = torch.empty(r.shape[0], H * dv, dtype=torch.float32, device=r.device)
+    _delta(out, r, k, v, w, a, w_bias, a_bias, state, 1, H, H, d, dv, decay, cu, slots, pos, n_single, max_q)
+    return out
+
+
+def _delta(out, q, k, v, w, b, w_vec, b_vec, state, mode, H, G, d, dv, decay, cu, slots, pos, n_single, max_q) -> None:
+    C = kernels()
+    T, n = out.shape[0], slots.numel()
+    args = (w_vec, b_vec, state, int(mode), int(H), int(G), int(d), int(dv), float(decay))
+    ns = n if cu is None else int(n_single)
+    if ns:   # single rows: the first ns segments are the first ns rows
+        C.delta_rows(out[:ns], q[:ns], k[:ns], v[:ns], w[:ns], b[:ns], *args, slots[:ns], pos[:ns])
+    if ns < n:
+        if max_q < 1:
+            raise ValueError("delta scans of portions need max_q, the rows of the longest one")
+        ws = _delta_workspace(T, n - ns, H, d, out.device)
+        C.delta_blocks(out, ws, q, k, v, w, b, *args, cu[ns:], slots[ns:], pos, int(max_q))
 
 
 class DecodeWorkspace:
@@ -1148,16 +1305,17 @@ def moe_route_scores(logits: torch.Tensor, k: int, score: str = "sigmoid", renor
     return ids, w
 
 
-def moe_route_grouped(logits: torch.Tensor, correction: torch.Tensor, k: int, groups: int = 1, keep: int = 1,
+def moe_route_grouped(logits: torch.Tensor, correction: Optional[torch.Tensor], k: int, groups: int = 1, keep: int = 1,
                       scale: float = 1.0, ws: Optional["MoEWorkspace"] = None) -> Tuple[torch.Tensor, torch.Tensor]:
     """Group-limited routing from fp32 logits [T, E]: scores ``s = softmax(logits)`` over all E;
     experts are chosen by ``s + correction`` (fp32 [E]) among the ``keep`` of ``groups`` equal
     groups of neighbouring experts whose largest corrected score is largest (the others cannot be
     chosen, however their corrected scores compare); the ``k`` chosen (ties: the lower index) get
     the weights ``s / (sum of the chosen s + 1e-20) * scale``. ids int32 [T, k], weights fp32
-    [T, k]. ``groups = 1``: plain top-k by corrected score."""
+    [T, k]. ``groups = 1``: plain top-k by corrected score; ``correction`` None: none."""
     T, E = logits.shape
-    if logits.dtype != torch.float32 or correction.dtype != torch.float32 or correction.numel() != E:
+    if logits.dtype != torch.float32 or (correction is not None and (correction.dtype != torch.float32
+                                                                     or correction.numel() != E)):
         raise ValueError("router logits and the correction are fp32, one correction per expert")
     if groups < 1 or E % groups or not 1 <= keep <= groups or not 1 <= k <= keep * (E // groups):
         raise ValueError(f"{E} experts in {groups} groups, keep {keep}, top {k}")
@@ -1232,6 +1390,49 @@ def moe_glu_experts(x: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w13: 
         C.moe_combine_rows(y, ws.inv, T, int(k), add, out, x, ids.reshape(-1), wts.reshape(-1), E)
     else:
         C.moe_combine_rows(y, ws.inv, T, int(k), add, out, None, None, None, E)
+    return out
+
+
+def moe_plain_mfma_ok(x: torch.Tensor, F: int) -> bool:
+    """The grouped MFMA GEMMs take bf16 rows with width % 256 == 0 and expert ff % 64 == 0."""
+    return _gpu(x) and x.dtype == torch.bfloat16 and x.shape[1] % 256 == 0 and F % 64 == 0
+
+
+def moe_plain_experts(x: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor,
+                      ws: Optional["MoEWorkspace"] = None) -> torch.Tensor:
+    """Routed experts without a gate on rows x [T, H] -> [T, H]: the sum over a row's experts (``ids`` / ``wts``
+    [T, k]) of ``weight * down_e(gelu(up_e x))`` (erf gelu). ``w1`` [E, F, H], ``w2`` [E, H, F]. GPU: the
+    order of :func:`moe_glu_experts` (align, gathered up GEMM with the activation in its epilogue, down
+    GEMM times the weight, combine), on MFMA tiles where the sizes fit (:func:`moe_plain_mfma_ok`),
+    else on fp32-accumulating VALU tiles."""
+    if not _gpu(x):
+        return ref.moe_plain_experts(x, ids, wts, w1, w2)
+    C = kernels()
+    T, H = x.shape
+    E, F, _ = w1.shape
+    k = ids.shape[1]
+    out = torch.empty(T, H, dtype=x.dtype, device=x.device)
+    if T == 0:
+        return out
+    M = T * k
+    if ws is None:
+        ws = MoEWorkspace.get(T, k, E, x.device)
+    if ws.rows * ws.k < M or ws.E < E:
+        raise ValueError(f"MoE workspace for {ws.rows} rows x top-{ws.k} / {ws.E} experts cannot take "
+                         f"{T} rows x top-{k} / {E} experts")
+    mfma = moe_plain_mfma_ok(x, F)
+    bm = 64 if (not mfma or M <= 256 * E) else 128
+    mt = -(-M // bm) + E
+    C.moe_align(ids.reshape(-1), wts.reshape(-1), T, int(k), 0, E, bm, ws.sorted_tok, ws.sorted_w, ws.inv, ws.tiles, mt)
+    h = torch.empty(M, F, dtype=x.dtype, device=x.device)
+    y = torch.empty(M, H, dtype=x.dtype, device=x.device)
+    if mfma:
+        C.moe_gemm(x, w1, ws.sorted_tok, ws.sorted_w, ws.tiles, mt, bm, h, 2, 3, 0.0, 0.0, False)
+        C.moe_gemm(h, w2, ws.sorted_tok, ws.sorted_w, ws.tiles, mt, bm, y, 1, 0, 0.0, 0.0, False)
+    else:
+        C.moe_gemm_rows(x, w1, ws.sorted_tok, ws.sorted_w, ws.tiles, mt, h, 2, 0.0, 0.0, False, 0.0)
+        C.moe_gemm_rows(h, w2, ws.sorted_tok, ws.sorted_w, ws.tiles, mt, y, 1, 0.0, 0.0, True, 0.0)
+    C.moe_combine_rows(y, ws.inv, T, int(k), None, out, None, None, None, E)
     return out
 
 

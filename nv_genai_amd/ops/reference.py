@@ -578,12 +578,13 @@ def headnorm_cache_(proj, slots, kc, vc, nq, nk, dk, nv, dv, eps, q_w=None, k_w=
 
 
 def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale, window=0, maps=1, lam=0.0,
-                      unit_eps=None, out_scale=1.0, gate=None, v_in_k=False, softcap=0.0):
+                      unit_eps=None, out_scale=1.0, gate=None, v_in_k=False, softcap=0.0, chunk=0, sink=None):
     """Softmax attention of token rows over row-major pages, one row at a time. ``maps`` score
     maps per head (q head (h, m) at column (h * maps + m) * dk, k head (h // (H / G)) * maps + m,
-    v head h // (H / G)), combined as a_0 - lam * a_1; optional unit RMS per head (times
-    ``out_scale``) and a per-head sigmoid gate. ``v_in_k``: the values are the first dv elements
-    of the key rows. ``softcap`` > 0: scores become softcap * tanh(score / softcap)."""
+    v head h // (H / G)), combined as a_0 - lam * a_1; optional unit RMS per head, then times
+    ``out_scale`` and a per-head sigmoid gate. ``v_in_k``: the values are the first dv elements
+    of the key rows. ``softcap`` > 0: scores become softcap * tanh(score / softcap). ``chunk`` > 0:
+    only keys of the query's own chunk; ``sink``: score of a key without a value."""
     T = q.shape[0]
     out = torch.zeros(T, H, dv, dtype=torch.float32, device=q.device)
     BS = kc.shape[2]
@@ -596,6 +597,8 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale
             continue
         bt = block_tables[int(tok_seq[t])]
         lo = max(0, i - window + 1) if window else 0
+        if chunk:
+            lo = max(lo, i // chunk * chunk)
         j = torch.arange(lo, i + 1, device=q.device)
         blk, off = bt[j // BS].long(), j % BS
         k = kc[blk, :, off, :].float().view(-1, G, maps, dk)[:, vh]     # [n, H, maps, dk]
@@ -603,10 +606,14 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale
         s = torch.einsum("hmd,nhmd->hmn", qf[t], k) * scale
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
-        a = torch.einsum("hmn,nhd->hmd", torch.softmax(s, -1), v)
+        if sink is not None:
+            s = torch.cat([s, torch.full_like(s[..., :1], float(sink))], -1)
+        w = torch.softmax(s, -1)[..., :j.numel()]
+        a = torch.einsum("hmn,nhd->hmd", w, v)
         out[t] = a[:, 0] - lam * a[:, 1] if maps == 2 else a[:, 0]
     if unit_eps is not None:
-        out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + unit_eps) * out_scale
+        out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + unit_eps)
+    out = out * out_scale
     if gate is not None:
         out = out * torch.sigmoid(gate.float())[:, :, None]
     return out.reshape(T, H * dv).to(q.dtype)
@@ -642,16 +649,17 @@ def hgrn2_scan(proj, f_bias, lower, state, H, d, dv, cu, slots, pos):
     return out.reshape(T, H * dv)
 
 
-def group_rmsnorm(x, w, groups, eps, dtype, gate=None):
+def group_rmsnorm(x, w, groups, eps, dtype, gate=None, gate_act="sigmoid"):
     """RMS norm of every one of ``groups`` equal column groups of fp32 rows, weight per element
     of a group (or per column of the row), written in ``dtype``; ``gate`` [T, columns]: times
-    sigmoid(gate)."""
+    sigmoid(gate) or silu(gate)."""
     T = x.shape[0]
     xg = x.view(T, groups, -1)
     y = xg * torch.rsqrt(xg.pow(2).mean(-1, keepdim=True) + eps) * w.view(-1, xg.shape[2])
     y = y.reshape(T, -1)
     if gate is not None:
-        y = y * torch.sigmoid(gate.float())
+        g = gate.float()
+        y = y * (torch.sigmoid(g) if gate_act == "sigmoid" else torch.nn.functional.silu(g))
     return y.to(dtype)
 
 
@@ -869,7 +877,7 @@ def moe_route_grouped(logits, correction, k, groups, keep, scale):
     """See :func:`nv_genai_amd.ops.moe_route_grouped`."""
     T, E = logits.shape
     s = torch.softmax(logits.float(), -1)
-    c = s + correction
+    c = s if correction is None else s + correction
     if groups > 1:
         per = E // groups
         best = c.view(T, groups, per).max(-1).values
@@ -882,3 +890,126 @@ def moe_route_grouped(logits, correction, k, groups, keep, scale):
     w = torch.gather(s, 1, ids)
     w = w / (w.sum(-1, keepdim=True) + 1e-20) * scale
     return ids.to(torch.int32), w
+
+
+# ------------------------------------------------------------------------- bigram embedding, token inputs, short
+# convolution, delta-rule recurrences, experts without a gate
+def bigram_embed(ids, embed, table, src, prev, mul_prev, mul_cur):
+    """See :func:`nv_genai_amd.ops.bigram_embed`."""
+    s, t = src.long(), ids.long()
+    buckets = table.shape[0] - 1
+    p = torch.zeros_like(t)
+    rows, st = s >= 0, s <= -2
+    p[rows] = t[s[rows]]
+    p[st] = prev[-(s[st] + 2)].long()
+    idx = torch.where(s == -1, torch.full_like(t, buckets), (p * mul_prev + t * mul_cur) % buckets)
+    return embed[t].float() + table[idx].float()
+
+
+def token_save_(prev, ids, last_row, slot):
+    ok = (slot >= 0) & (last_row >= 0)
+    prev[slot[ok].long()] = ids[last_row[ok].long()].to(prev.dtype)
+    return prev
+
+
+def gelu_gate_rows(z, ids, table, off):
+    """gelu_tanh(z) * table[id, off : off + z columns]."""
+    e = table[ids.long(), off:off + z.shape[1]].float()
+    return (torch.nn.functional.gelu(z.float(), approximate="tanh") * e).to(z.dtype)
+
+
+def residual_add_cast_(x, y, out):
+    x.add_(y.float())
+    out.copy_(x)
+    return out
+
+
+def tanh_rows(x):
+    return torch.tanh(x.float()).to(x.dtype)
+
+
+def short_conv(x, taps, state, cu, slots, seq, pos):
+    """See :func:`nv_genai_amd.ops.short_conv`."""
+    T, C = x.shape
+    n = taps.shape[0]
+    out = torch.empty(T, C, dtype=x.dtype, device=x.device)
+    for b in range(slots.numel()):
+        t0, t1 = (b, b + 1) if cu is None else (int(cu[b]), int(cu[b + 1]))
+        if t1 <= t0:
+            continue
+        sl = int(slots[b])
+        if int(pos[t0]) == 0 or sl < 0:
+            old = torch.zeros(n - 1, C, dtype=torch.float32, device=x.device)
+        else:
+            old = state[sl].float()
+        rows = torch.cat([old, x[t0:t1].float()])
+        y = sum(rows[j:j + t1 - t0] * taps[j] for j in range(n))
+        out[t0:t1] = torch.nn.functional.silu(y).to(x.dtype)
+        if sl >= 0 and n > 1:
+            state[sl] = rows[-(n - 1):].to(state.dtype)
+    return out
+
+
+def _delta_segments(state, cu, slots, pos):
+    for b in range(slots.numel()):
+        t0, t1 = (b, b + 1) if cu is None else (int(cu[b]), int(cu[b + 1]))
+        if t1 <= t0:
+            continue
+        sl = int(slots[b])
+        fresh = int(pos[t0]) == 0 or sl < 0
+        yield t0, t1, sl, (torch.zeros_like(state[0]) if fresh else state[sl].clone())
+
+
+def _unit(x):
+    return x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) + 1e-6)
+
+
+def gated_delta_scan(x, ba, a_log, dt_bias, state, H, G, d, dv, cu, slots, pos):
+    """See :func:`nv_genai_amd.ops.gated_delta_scan`."""
+    T, rep = x.shape[0], H // G
+    xf = x.float()
+    q = (_unit(xf[:, :G * d].reshape(T, G, d)) * d ** -0.5).repeat_interleave(rep, 1)
+    k = _unit(xf[:, G * d:2 * G * d].reshape(T, G, d)).repeat_interleave(rep, 1)
+    v = xf[:, 2 * G * d:2 * G * d + H * dv].reshape(T, H, dv)
+    beta = torch.sigmoid(ba[:, :H].float())
+    g = torch.exp(-torch.exp(a_log) * torch.nn.functional.softplus(ba[:, H:2 * H].float() + dt_bias))
+    out = torch.zeros(T, H, dv, dtype=torch.float32, device=x.device)
+    for t0, t1, sl, S in _delta_segments(state, cu, slots, pos):
+        for t in range(t0, t1):
+            S = g[t][:, None, None] * S
+            u = beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
+            S = S + k[t][:, :, None] * u[:, None, :]
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        if sl >= 0:
+            state[sl] = S
+    return out.reshape(T, H * dv)
+
+
+def channel_delta_scan(r, k, v, a, w, a_bias, w_bias, state, H, d, dv, decay, cu, slots, pos):
+    """See :func:`nv_genai_amd.ops.channel_delta_scan`."""
+    T = r.shape[0]
+    rf, kf, vf = r.float().reshape(T, H, d), k.float().reshape(T, H, d), v.float().reshape(T, H, dv)
+    af = torch.sigmoid(a.float() + a_bias).reshape(T, H, d)
+    wf = torch.exp(-decay * torch.sigmoid(w.float() + w_bias)).reshape(T, H, d)
+    u = _unit(kf)
+    out = torch.zeros(T, H, dv, dtype=torch.float32, device=r.device)
+    for t0, t1, sl, S in _delta_segments(state, cu, slots, pos):
+        for t in range(t0, t1):
+            y = torch.einsum("hdv,hd->hv", S, u[t])
+            S = (wf[t][:, :, None] * S - (af[t] * u[t])[:, :, None] * y[:, None, :]
+                 + kf[t][:, :, None] * vf[t][:, None, :])
+            out[t] = torch.einsum("hdv,hd->hv", S, rf[t])
+        if sl >= 0:
+            state[sl] = S
+    return out.reshape(T, H * dv)
+
+
+def moe_plain_experts(x, ids, wts, w1, w2):
+    """Sum over a row's experts of weight * down_e(gelu(up_e x)) (erf gelu)."""
+    out = torch.zeros(x.shape[0], w2.shape[1], dtype=torch.float32, device=x.device)
+    for e in range(w1.shape[0]):
+        tok, slot = torch.where(ids == e)
+        if tok.numel():
+            h = torch.nn.functional.gelu(x[tok].float() @ w1[e].float().t()).to(x.dtype)
+            out.index_add_(0, tok, (h.float() @ w2[e].float().t()) * wts[tok, slot].unsqueeze(1))
+    return out.to(x.dtype)
