@@ -313,7 +313,7 @@ class VivesunModel:
         ops.rope_headnorm_cache_(proj, pos, meta.slots, kc, vc, a.heads, a.kv_heads, a.dim, a.vdim, L["freq"], L["mag"],
                                  a.rot.dims, self.cfg.eps, v_off=(a.heads + a.kv_heads) * a.dim)
         self._attend(proj[:, :a.heads * a.dim], kc, vc, pos, meta, a, y[:, :nl], scale=a.scale, chunk=a.chunk, sink=0.0,
-                     out_scale=m.left_scale)
+                     factor=m.left_scale)
         # right: r | k | v | gate | removal rate | low-rank decay columns
         c = [L["r_off"] + j * nr for j in range(6)]
         w = self._lin(ops.tanh_rows(proj[:, c[5]:c[5] + L["rank"]]), L["w2"])

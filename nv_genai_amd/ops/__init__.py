@@ -539,18 +539,22 @@ def headnorm_cache_(proj, slots, kc, vc, nq: int, nk: int, dk: int, nv: int, dv:
     return proj
 
 
+def _out_factor(unit_eps: Optional[float], out_scale: float, factor: float) -> float:
+    return float(factor) * (1.0 if unit_eps is None else float(out_scale))
+
+
 def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk: int, dv: int, scale: float,
                       window: int = 0, maps: int = 1, lam: float = 0.0, unit_eps: Optional[float] = None,
                       out_scale: float = 1.0, gate=None, out=None, v_in_k: bool = False, softcap: float = 0.0,
-                      chunk: int = 0, sink: Optional[float] = None):
+                      chunk: int = 0, sink: Optional[float] = None, factor: float = 1.0):
     """Softmax attention of token rows (prompt portions and single-token rows alike) over row-
     major pages K [blocks, G * maps, 64, dk], V [blocks, G, 64, dv]. The query at position i
     sees keys ``j <= i`` (``window`` > 0: and ``i - j < window``). ``maps`` (1 or 2) score maps per
     head: q head (h, m) is column block ``h * maps + m``, its keys are k head
     ``(h // (H / G)) * maps + m``, both maps read v head ``h // (H / G)``; two maps combine as
     ``a_0 - lam * a_1`` (differential attention). ``unit_eps``: divide every head's output by its
-    root mean square (eps inside the root). The outputs are multiplied by ``out_scale``, and with
-    ``gate`` [T, H] by ``sigmoid(gate)`` of their head. ``tok_seq[t]`` is the block-table row of
+    root mean square (eps inside the root) and multiply by ``out_scale``. ``gate`` [T, H]: the
+    head outputs are multiplied by ``sigmoid(gate)``. ``factor``: the outputs are multiplied by it. ``tok_seq[t]`` is the block-table row of
     token t, ``pos[t]`` its position (negative: padding row, zeros out). Scores, softmax and
     accumulation are fp32. ``v_in_k`` (one map, dv <= dk): the values are the first dv elements of
     the key rows (``vc`` is not read) - keys with extra key-only columns behind a shared latent.
@@ -562,13 +566,13 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk:
         raise ValueError("values inside the key rows: one map and dv <= dk")
     if not _gpu(q):
         r = ref.softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam,
-                                  unit_eps, out_scale, gate, v_in_k, softcap, chunk, sink)
+                                  unit_eps, out_scale, gate, v_in_k, softcap, chunk, sink, factor)
         return r if out is None else out.copy_(r)
     if out is None:
         out = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
     kernels().softmax_attention(out, q, gate, kc, kc if v_in_k else vc, block_tables, tok_seq, pos, H, G, dk, dv,
                                 float(scale), int(window), int(maps), float(lam),
-                                -1.0 if unit_eps is None else float(unit_eps), float(out_scale), bool(v_in_k),
+                                -1.0 if unit_eps is None else float(unit_eps), _out_factor(unit_eps, out_scale, factor), bool(v_in_k),
                                 float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 
@@ -594,21 +598,22 @@ def softmax_attention_prefill(q, kc, vc, block_tables, cu_q, ctx_lens, max_q_len
                               dv: int, scale: float, window: int = 0, maps: int = 1, lam: float = 0.0,
                               unit_eps: Optional[float] = None, out_scale: float = 1.0, gate=None, out=None,
                               v_in_k: bool = False, softcap: float = 0.0, chunk: int = 0,
-                              sink: Optional[float] = None):
+                              sink: Optional[float] = None, factor: float = 1.0):
     """:func:`softmax_attention` of prompt portions on MFMA tiles: sequence b owns token rows
     ``[cu_q[b], cu_q[b + 1])``, the last ones of its ``ctx_lens[b]`` keys. Rows the tile kernel
     does not take (fp32, other head sizes, CPU) run the row form."""
     if not softmax_attention_mfma_ok(q, dk, dv, H // G, maps):
         seq, pos = _rows_of_portions(cu_q, ctx_lens, q.shape[0], q.device)
         return softmax_attention(q, kc, vc, block_tables, seq, pos, H, G, dk, dv, scale, window, maps, lam, unit_eps,
-                                 out_scale, gate, out=out, v_in_k=v_in_k, softcap=softcap, chunk=chunk, sink=sink)
+                                 out_scale, gate, out=out, v_in_k=v_in_k, softcap=softcap, chunk=chunk, sink=sink,
+                                 factor=factor)
     if v_in_k and (maps != 1 or dv > dk):
         raise ValueError("values inside the key rows: one map and dv <= dk")
     if out is None:
         out = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
     kernels().softmax_attention_prefill(out, q, gate, kc, kc if v_in_k else vc, block_tables, cu_q, ctx_lens,
                                         int(max_q_len), H, G, dk, dv, float(scale), int(window), int(maps), float(lam),
-                                        -1.0 if unit_eps is None else float(unit_eps), float(out_scale), bool(v_in_k),
+                                        -1.0 if unit_eps is None else float(unit_eps), _out_factor(unit_eps, out_scale, factor), bool(v_in_k),
                                         float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 
@@ -616,7 +621,8 @@ def softmax_attention_prefill(q, kc, vc, block_tables, cu_q, ctx_lens, max_q_len
 def softmax_attention_rows(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk: int, dv: int, scale: float,
                            max_ctx: int, window: int = 0, maps: int = 1, lam: float = 0.0,
                            unit_eps: Optional[float] = None, out_scale: float = 1.0, gate=None, out=None,
-                           v_in_k: bool = False, softcap: float = 0.0, chunk: int = 0, sink: Optional[float] = None):
+                           v_in_k: bool = False, softcap: float = 0.0, chunk: int = 0, sink: Optional[float] = None,
+                           factor: float = 1.0):
     """:func:`softmax_attention` of single-token rows (decode rows; any rows work) on the page-
     parallel MFMA kernel: the query heads that share a KV head are the columns of one tile, so a
     page is read once per group; the visible pages of a row are split over several workgroups
@@ -625,7 +631,7 @@ def softmax_attention_rows(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int
     if not softmax_attention_mfma_ok(q, dk, dv, H // G, maps):
         return softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam,
                                  unit_eps, out_scale, gate, out=out, v_in_k=v_in_k, softcap=softcap, chunk=chunk,
-                                 sink=sink)
+                                 sink=sink, factor=factor)
     if v_in_k and (maps != 1 or dv > dk):
         raise ValueError("values inside the key rows: one map and dv <= dk")
     C = kernels()
@@ -636,7 +642,7 @@ def softmax_attention_rows(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int
         out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
     C.softmax_attention_decode(out, ws, parts, q, gate, kc, kc if v_in_k else vc, block_tables, tok_seq, pos, H, G, dk,
                                dv, float(scale), int(window), int(maps), float(lam),
-                               -1.0 if unit_eps is None else float(unit_eps), float(out_scale), bool(v_in_k),
+                               -1.0 if unit_eps is None else float(unit_eps), _out_factor(unit_eps, out_scale, factor), bool(v_in_k),
                                float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 

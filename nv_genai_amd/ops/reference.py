@@ -578,13 +578,15 @@ def headnorm_cache_(proj, slots, kc, vc, nq, nk, dk, nv, dv, eps, q_w=None, k_w=
 
 
 def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale, window=0, maps=1, lam=0.0,
-                      unit_eps=None, out_scale=1.0, gate=None, v_in_k=False, softcap=0.0, chunk=0, sink=None):
+                      unit_eps=None, out_scale=1.0, gate=None, v_in_k=False, softcap=0.0, chunk=0, sink=None,
+                      factor=1.0):
     """Softmax attention of token rows over row-major pages, one row at a time. ``maps`` score
     maps per head (q head (h, m) at column (h * maps + m) * dk, k head (h // (H / G)) * maps + m,
-    v head h // (H / G)), combined as a_0 - lam * a_1; optional unit RMS per head, then times
-    ``out_scale`` and a per-head sigmoid gate. ``v_in_k``: the values are the first dv elements
+    v head h // (H / G)), combined as a_0 - lam * a_1; optional unit RMS per head (times
+    ``out_scale``) and a per-head sigmoid gate. ``v_in_k``: the values are the first dv elements
     of the key rows. ``softcap`` > 0: scores become softcap * tanh(score / softcap). ``chunk`` > 0:
-    only keys of the query's own chunk; ``sink``: score of a key without a value."""
+    only keys of the query's own chunk; ``sink``: score of a key without a value;
+    ``factor``: multiplies the outputs."""
     T = q.shape[0]
     out = torch.zeros(T, H, dv, dtype=torch.float32, device=q.device)
     BS = kc.shape[2]
@@ -612,8 +614,8 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale
         a = torch.einsum("hmn,nhd->hmd", w, v)
         out[t] = a[:, 0] - lam * a[:, 1] if maps == 2 else a[:, 0]
     if unit_eps is not None:
-        out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + unit_eps)
-    out = out * out_scale
+        out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + unit_eps) * out_scale
+    out = out * factor
     if gate is not None:
         out = out * torch.sigmoid(gate.float())[:, :, None]
     return out.reshape(T, H * dv).to(q.dtype)
