@@ -1,10 +1,10 @@
-"""The layer-list designs (Bidasun, Biruvik, Lumepel, Lizezen) beside the closest Llama-layout model at
-equal sizes (Mistral with a sliding window; Mixtral for Lumepel and Lizezen, whose feed-forwards are
-routed experts):
+"""The layer-list designs (Bidasun, Biruvik, Lumepel, Lizezen, Vivesun) beside the closest Llama-layout model
+at equal sizes (Mistral with a sliding window; Mixtral for Lumepel, Lizezen and Vivesun, whose
+feed-forwards are routed experts):
 prefill and decode throughput through the serving engine, and the design's kernels alone with
 their distance from the roofline. Random weights, synthetic token ids.
 
-    python bench.py --workload designs [--design-sizes s,m,l] [--design-models bidasun,biruvik,lumepel,lizezen]
+    python bench.py --workload designs [--design-sizes s,m,l] [--design-models bidasun,biruvik,lumepel,lizezen,vivesun]
 
 Prints one JSON line (``metric: design_compare``); bench.py's default workload is untouched.
 """
@@ -38,14 +38,29 @@ LUMEPEL_PATTERN = ("latent_attention", "latent_attention_2")
 # with two identity experts, four groups of which two are kept, and a shared expert
 LIZEZEN_PATTERN = ("mlstm", "attention", "mlstm", "attention_2")
 LIZEZEN_MLSTM = dict(dim=64, vdim=128)
-BASELINE_OF = {"bidasun": "mistral", "biruvik": "mistral", "lumepel": "mixtral", "lizezen": "mixtral"}
+# Vivesun: gated delta heads of 128-wide keys and values (two per q / k head), chunked attention (chunk =
+# the window of the other designs, a rotation on half the head) beside 64-wide channel-decay delta
+# heads over the whole width, expert sizes of LUMEPEL, a bigram table and a token input
+VIVESUN_PATTERN = ("delta", "parallel")
+VIVESUN = dict(dim=128, vdim=128, conv=4, rdim=64, rank=64, rot=64, side=256, bigram=(65521, 31, 17))
+BASELINE_OF = {"bidasun": "mistral", "biruvik": "mistral", "lumepel": "mixtral", "lizezen": "mixtral", "vivesun": "mixtral"}
 
 
 def _engine(kind: str, z: dict, max_len: int, pages: int, seqs: int):
     from nv_genai_amd.engine.llm_engine import EngineConfig, LLMEngine
     from nv_genai_amd.models.config import LlamaConfig, bidasun_uniform, biruvik_layers, lizezen_layers, lumepel_layers
+    from nv_genai_amd.models.config import vivesun_layers
 
-    if kind == "lizezen":
+    if kind == "vivesun":
+        u, v = z["lumepel"], VIVESUN
+        pat = [VIVESUN_PATTERN[i % len(VIVESUN_PATTERN)] for i in range(z["layers"])]
+        mcfg = vivesun_layers(pat, z["hidden"], z["heads"], z["kv"], z["d"], z["d"], chunk=z["window"],
+                              delta_heads=z["heads"], delta_kv_heads=z["heads"] // 2, delta_dim=v["dim"],
+                              delta_vdim=v["vdim"], conv=v["conv"], right_heads=z["hidden"] // v["rdim"],
+                              right_dim=v["rdim"], decay_rank=v["rank"], experts=u["experts"], top=u["top"],
+                              expert_ff=u["eff"], route_scale=2.0, rot_base=5e5, rot_dims=v["rot"],
+                              bands=(8.0, 1.0, 4.0, 8192), bigram=v["bigram"], side_dim=v["side"], vocab_size=VOCAB)
+    elif kind == "lizezen":
         u = z["lumepel"]
         pat = [LIZEZEN_PATTERN[i % len(LIZEZEN_PATTERN)] for i in range(z["layers"])]
         mcfg = lizezen_layers(pat, z["hidden"], z["heads"], z["kv"], z["d"], z["d"], z["ffn"], mlstm_heads=z["heads"],
@@ -88,6 +103,23 @@ def _timed(fn, n: int) -> float:
         fn()
     torch.cuda.synchronize()
     return (time.perf_counter() - t0) / n
+
+
+def _timed_gpu(fn, n: int) -> float:
+    """Seconds per call on the GPU: n calls captured in one hipGraph, so that kernels of a few
+    microseconds are not timed by the host's launch rate."""
+    side = torch.cuda.Stream()
+    side.wait_stream(torch.cuda.current_stream())
+    with torch.cuda.stream(side):
+        fn()
+    torch.cuda.current_stream().wait_stream(side)
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for _ in range(n):
+            fn()
+    g.replay()
+    return _timed(g.replay, 3) / n
 
 
 def engine_rates(kind: str, z: dict, steps: int, warmup: int) -> dict:
@@ -514,6 +546,173 @@ def lizezen_kernel_times(z: dict, iters: int = 20) -> dict:
     return out
 
 
+def vivesun_kernel_times(z: dict, iters: int = 20) -> dict:
+    """The Vivesun kernels alone on one layer's shapes beside the like kernels of the other models: the
+    delta-rule scans against the HGRN2 scan (same state sizes; fp32 flops per state element and row:
+    7 for the gated rule, 9 with channel-wise decay, 6 for HGRN2), chunked attention with a sink
+    against windowed softmax attention of the Llama layout (visible keys each), gelu experts against
+    the Mixtral experts, and the row kernels against theirs, priced by the flops or bytes they must
+    move."""
+    from nv_genai_amd import ops
+    from nv_genai_amd.ops import reference as ref
+
+    dev, bf = "cuda", torch.bfloat16
+    u, v = z["lumepel"], VIVESUN
+    H, G, D, W, Hd = z["heads"], z["kv"], z["d"], z["window"], z["hidden"]
+    nb, L = z["pf"]
+    nd, ctx = z["dec"]
+    T = nb * L
+    cu = torch.arange(0, T + 1, L, dtype=torch.int32, device=dev)
+    posr = torch.arange(L, dtype=torch.int32, device=dev).repeat(nb)
+    tseq = torch.arange(nb, dtype=torch.int32, device=dev).repeat_interleave(L)
+    sl_p = torch.arange(nb, dtype=torch.int32, device=dev)
+    sl_d = torch.arange(nd, dtype=torch.int32, device=dev)
+    posd = torch.full((nd,), ctx - 1, dtype=torch.int32, device=dev)
+    out, scan = {}, {}
+    # ---- scans: prompts (nb segments of L rows) and single rows (nd segments)
+    d, dv, Gk = v["dim"], v["vdim"], H // 2
+    C = 2 * Gk * d + H * dv
+    proj = torch.randn(T, C + H * dv + 2 * H, device=dev).to(bf)
+    taps = torch.randn(v["conv"], C, device=dev) * 0.5
+    cst = torch.zeros(max(nb, nd), v["conv"] - 1, C, device=dev, dtype=bf)
+    t_cp = _timed_gpu(lambda: ops.short_conv(proj[:, :C], taps, cst, cu, sl_p, tseq, posr), iters)
+    t_cd = _timed_gpu(lambda: ops.short_conv(proj[:nd, :C], taps, cst, None, sl_d, sl_d, posd), iters)
+    x = ops.short_conv(proj[:, :C], taps, cst, cu, sl_p, tseq, posr)
+    ba = proj[:, C + H * dv:]
+    al, db = torch.zeros(H, device=dev), torch.full((H,), -2.0, device=dev)
+
+    def scans(name, run_p, run_d, heads, k, vv, flops):
+        hp = torch.randn(T, 2 * heads * k + heads * vv, device=dev).to(bf)
+        fb, lw = torch.randn(heads * k, device=dev), torch.rand(heads * k, device=dev) * 0.9
+        hs = torch.zeros(max(nb, nd), heads, k, vv, device=dev)
+        t_p, t_d = _timed_gpu(run_p, iters), _timed_gpu(run_d, iters)
+        t_hp = _timed_gpu(lambda: ops.hgrn2_scan(hp, fb, lw, hs, heads, k, vv, cu, sl_p, posr), iters)
+        t_hd = _timed_gpu(lambda: ops.hgrn2_scan(hp[:nd], fb, lw, hs, heads, k, vv, None, sl_d, posd), iters)
+        fl, by = T * heads * k * vv, nd * heads * k * vv * 8.0       # state read + written
+        scan[name] = {"prefill_ms": round(t_p * 1e3, 3), "hgrn2_prefill_ms": round(t_hp * 1e3, 3),
+                      "fp32_frac": round(flops * fl / t_p / PEAK_VALU, 4), "hgrn2_fp32_frac": round(6.0 * fl / t_hp / PEAK_VALU, 4),
+                      "decode_ms": round(t_d * 1e3, 4), "hgrn2_decode_ms": round(t_hd * 1e3, 4),
+                      "state_hbm_frac": round(by / t_d / PEAK_HBM, 4), "hgrn2_state_hbm_frac": round(by / t_hd / PEAK_HBM, 4)}
+
+    st = torch.zeros(max(nb, nd), H, d, dv, device=dev)
+    scans("gated_delta", lambda: ops.gated_delta_scan(x, ba, al, db, st, H, Gk, d, dv, cu, sl_p, posr, max_q=L),
+          lambda: ops.gated_delta_scan(x[:nd], ba[:nd], al, db, st, H, Gk, d, dv, None, sl_d, posd), H, d, dv, 7.0)
+    del proj, x, st
+    R, rd = Hd // v["rdim"], v["rdim"]
+    n = R * rd
+    rp = torch.randn(T, 5 * n, device=dev).to(bf)
+    cols = [rp[:, i * n:(i + 1) * n] for i in range(5)]
+    ab, wb = torch.zeros(n, device=dev), torch.full((n,), -3.0, device=dev)
+    st = torch.zeros(max(nb, nd), R, rd, rd, device=dev)
+    dcy = 0.6065306597126334
+    scans("channel_delta", lambda: ops.channel_delta_scan(*cols, ab, wb, st, R, rd, rd, dcy, cu, sl_p, posr, max_q=L),
+          lambda: ops.channel_delta_scan(*(c[:nd] for c in cols), ab, wb, st, R, rd, rd, dcy, None, sl_d, posd), R, rd, rd, 9.0)
+    del rp, cols, st
+    out["scan"] = scan
+    # ---- attention: chunks and a sink on row-major pages against the windowed Llama-layout kernels
+    pages_seq = -(-max(L, ctx) // 64)
+    nseq = max(nb, nd)
+    npg = nseq * pages_seq
+    bt = torch.arange(npg, dtype=torch.int32, device=dev).view(nseq, pages_seq)
+    kr = (torch.randn(npg, G, 64, D, device=dev) * 0.5).to(bf)
+    vr = (torch.randn(npg, G, 64, D, device=dev) * 0.5).to(bf)
+    vt = (torch.randn(npg, G, D, 64, device=dev) * 0.5).to(bf)
+    cx = torch.full((nb,), L, dtype=torch.int32, device=dev)
+    q1 = torch.randn(T, H * D, device=dev).to(bf)
+    pairs_c = nb * sum(i % W + 1 for i in range(L)) * H
+    pairs_w = nb * sum(min(i + 1, W) for i in range(L)) * H
+    sc = D ** -0.5
+    out["mfma_attention"] = bool(ops.softmax_attention_mfma_ok(q1, D, D, H // G, 1))
+    kw = dict(scale=sc, chunk=W, sink=0.0)
+    t_ch = _timed_gpu(lambda: ops.softmax_attention_prefill(q1, kr, vr, bt, cu, cx, L, H, G, D, D, **kw), iters)
+    t_wi = _timed_gpu(lambda: ops.prefill_attention_paged(q1, kr, vt, bt, cu, cx, H, G, D, L, sc, window=W, impl=4), iters)
+    out["prefill"] = {"chunked_ms": round(t_ch * 1e3, 3), "windowed_llama_layout_ms": round(t_wi * 1e3, 3),
+                      "chunked_mfma_frac": round(4.0 * pairs_c * D / t_ch / PEAK_BF16, 4),
+                      "windowed_llama_layout_mfma_frac": round(4.0 * pairs_w * D / t_wi / PEAK_BF16, 4)}
+    cxd = torch.full((nd,), ctx, dtype=torch.int32, device=dev)
+    ws = ops.DecodeWorkspace(nd, H, G, ctx, dev, None, D=D)
+    t_chd = _timed_gpu(lambda: ops.softmax_attention_rows(q1[:nd], kr, vr, bt, sl_d, posd, H, G, D, D, max_ctx=ctx, **kw), iters)
+    t_wid = _timed_gpu(lambda: ops.decode_attention(q1[:nd], kr, vt, bt, cxd, H, G, ctx, sc, ws=ws, window=W), iters)
+    kvb = nd * G * 2 * D * 2.0
+    out["decode"] = {"chunked_ms": round(t_chd * 1e3, 4), "windowed_llama_layout_ms": round(t_wid * 1e3, 4),
+                     "chunked_hbm_frac": round(kvb * ((ctx - 1) % W + 1) / t_chd / PEAK_HBM, 4),
+                     "windowed_llama_layout_hbm_frac": round(kvb * min(ctx, W) / t_wid / PEAK_HBM, 4)}
+    # ---- experts: T rows (prompts) and nd rows (single tokens)
+    E, k, F = u["experts"], u["top"], u["eff"]
+    x = torch.randn(T, Hd, device=dev).to(bf)
+    router = (torch.randn(E, Hd, device=dev) * Hd ** -0.5)
+    w13 = (torch.randn(E, 2 * F, Hd, device=dev) * Hd ** -0.5).to(bf)
+    w1 = w13[:, :F].contiguous()
+    w2 = (torch.randn(E, Hd, F, device=dev) * F ** -0.5).to(bf)
+    rb = router.to(bf)
+
+    def viv(xx):
+        ids, wts = ops.moe_route_grouped(ops.linear(xx.float(), router), None, k, 1, 1, 2.0)
+        return ops.moe_plain_experts(xx, ids, wts, w1, w2)
+
+    ex = {}
+    for name, rows in (("prefill", T), ("decode", nd)):
+        xx = x[:rows]
+        fl, by = 2.0 * rows * k * Hd * F, min(E, rows * k) * Hd * F * 2.0
+        t_v = _timed_gpu(lambda: viv(xx), iters)
+        t_m = _timed_gpu(lambda: ops.moe_ffn(xx, rb, w13, w2, k), iters)
+        ex[name] = {"vivesun_ms": round(t_v * 1e3, 3), "mixtral_ms": round(t_m * 1e3, 3),
+                    "vivesun_mfma_frac": round(2 * fl / t_v / PEAK_BF16, 4), "mixtral_mfma_frac": round(3 * fl / t_m / PEAK_BF16, 4),
+                    "vivesun_weight_hbm_frac": round(2 * by / t_v / PEAK_HBM, 4),
+                    "mixtral_weight_hbm_frac": round(3 * by / t_m / PEAK_HBM, 4)}
+    out["experts"] = ex
+    del w13, w1, w2
+    # ---- row kernels (prompt rows): bytes that must move over the time, against 8 TB/s
+    qkv = torch.randn(T, (H + 2 * G) * D, device=dev).to(bf)
+    slots = torch.arange(T, dtype=torch.int32, device=dev)
+    freq, mag = ops.rotary_frequencies(v["rot"], 5e5, bands=(8.0, 1.0, 4.0, 8192))
+    freq = freq.to(dev)
+    t_rh = _timed_gpu(lambda: ops.rope_headnorm_cache_(qkv, posr, slots, kr, vr, H, G, D, D, freq, mag, v["rot"], 1e-5,
+                                                   v_off=(H + G) * D), iters)
+    cs = ref.rope_cos_sin(L, D, 1e6).to(dev)
+    t_rk = _timed_gpu(lambda: ops.rope_cache_(qkv, posr, cs, slots, kr, vt, H, G, D), iters)
+    by_rk = T * (2 * (H + G) * D + 2 * G * D) * 2.0      # q, k read + written, k and v pages written, v read
+    by_rh = T * (2 * H * v["rot"] + G * (D + v["rot"]) + G * D + 2 * G * D) * 2.0   # only rotated parts written back
+    xs = torch.randn(T, Hd, device=dev)
+    y1 = torch.randn(T, Hd, device=dev).to(bf)
+    wn = torch.ones(Hd, device=dev)
+    ids = torch.randint(0, VOCAB, (T,), device=dev, dtype=torch.int32)
+    emb = torch.randn(VOCAB, Hd, device=dev).to(bf)
+    bg = torch.randn(v["bigram"][0] + 1, Hd, device=dev).to(bf)
+    src = torch.arange(-1, T - 1, dtype=torch.int32, device=dev)
+    prev = torch.zeros(nseq, dtype=torch.int32, device=dev)
+    se = torch.randn(VOCAB, 2 * v["side"], device=dev).to(bf)
+    zz = torch.randn(T, v["side"], device=dev).to(bf)
+    o = torch.randn(T, H * dv, device=dev)
+    gg = torch.randn(T, H * dv, device=dev).to(bf)
+    won = torch.ones(dv, device=dev)
+    lr = torch.randn(T, 4 * v["rank"], device=dev).to(bf)
+    xb, wbf = xs.to(bf), wn.to(bf)
+    Fd = z["ffn"] // 8 * 8
+    gu = torch.randn(T, 2 * Fd, device=dev).to(bf)
+    rows = {
+        # name: (call, bytes)
+        "rope_partial_cache": (t_rh, by_rh), "rope_cache": (t_rk, by_rk),
+        "short_conv": (t_cp, T * C * 4.0),
+        "bigram_embed": (lambda: ops.bigram_embed(ids, emb, bg, src, prev, 31, 17), T * Hd * 8.0),   # two bf16 in, fp32 out
+        "embed_rows": (lambda: ops.embed_rows(ids, emb), T * Hd * 6.0),
+        "residual_add_rmsnorm": (lambda: ops.residual_add_rmsnorm_(xs, y1, wn, 1e-5, bf), T * Hd * 12.0),
+        "residual_add_cast": (lambda: ops.residual_add_cast_(xs, y1, bf), T * Hd * 12.0),
+        "rmsnorm_residual_next": (lambda: ops.rmsnorm_residual_next_(xs, y1, wn, 1e-5, wn, bf), T * Hd * 12.0),
+        "add_rmsnorm": (lambda: ops.add_rmsnorm(xb, y1, wbf, 1e-5), T * Hd * 8.0),
+        "gelu_gate_rows": (lambda: ops.gelu_gate_rows(zz, ids, se, v["side"]), T * v["side"] * 6.0),
+        "tanh_rows": (lambda: ops.tanh_rows(lr[:, v["rank"]:2 * v["rank"]]), T * v["rank"] * 4.0),
+        "silu_gated_head_norm": (lambda: ops.group_rmsnorm(o, won, H, 1e-5, bf, gate=gg, gate_act="silu"), T * H * dv * 8.0),
+        "silu_mul": (lambda: ops.silu_mul(gu), T * Fd * 6.0)}
+    out["rows"] = {}
+    for name, (c, by) in rows.items():
+        t = c if isinstance(c, float) else _timed_gpu(c, iters)
+        out["rows"][name] = {"ms": round(t * 1e3, 4), "hbm_frac": round(by / t / PEAK_HBM, 4)}
+    out["rows"]["short_conv_decode"] = {"ms": round(t_cd * 1e3, 4), "hbm_frac": round(
+        nd * C * (4.0 + 4.0 * (v["conv"] - 1)) / t_cd / PEAK_HBM, 4)}
+    return out
+
+
 def run(args) -> None:
     names = [s for s in (args.design_sizes or "s,m,l").split(",") if s]
     models = [m for m in (getattr(args, "design_models", None) or "bidasun").split(",") if m]
@@ -537,6 +736,9 @@ def run(args) -> None:
             torch.cuda.empty_cache()
         if "lizezen" in models:
             res[n]["lizezen_kernels"] = lizezen_kernel_times(z)
+            torch.cuda.empty_cache()
+        if "vivesun" in models:
+            res[n]["vivesun_kernels"] = vivesun_kernel_times(z)
             torch.cuda.empty_cache()
         print(f"[designs] {n}: {json.dumps(res[n])}", flush=True)
     line = {"metric": "design_compare", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,

@@ -428,7 +428,7 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, fl
 template <typename T, int DT>
 struct BlockRegs {
   f32x4 c[DT], r[DT], a[DT], k[DT], p[DT], n;
-  float v[4];
+  T v[4];      // raw values (converted at their use: a conversion behind the load would wait for it)
 };
 
 template <typename T, int DT>
@@ -454,6 +454,8 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1)))
     }
   const int64_t ent = (int64_t)P.H * (65 * D + 256);       // one block of all heads
   const float* wp = ws + ((int64_t)((t0 - P.cu[0]) / 16 + b) * P.H + h) * (int64_t)(65 * D + 256);
+  // no branch around a load (each would wait for all loads in flight): rows past the segment read its
+  // last row - the block operands are zero there -, columns past dv the first one, and are not stored
   const T* vp = (const T*)P.v + (int64_t)t0 * P.vs + h * dv + (colok ? col : 0);
   auto load = [&](BlockRegs<T, DT>& B, int blk) {
     const float* w = wp + blk * ent;
@@ -464,8 +466,8 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1)))
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int t = blk * 16 + 4 * hh + r;
-      B.v[r] = (colok && t0 + t < t1) ? ldf(vp + (int64_t)t * P.vs) : 0.f;
+      const int t = min(blk * 16 + 4 * hh + r, t1 - t0 - 1);
+      B.v[r] = vp[(int64_t)t * P.vs];
     }
     B.n = *reinterpret_cast<const f32x4*>(w + 64 * D + 4 * lane);
 #pragma unroll
@@ -486,20 +488,29 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1)))
       }
 #pragma unroll
     for (int i = 0; i < DT; ++i) S[i] *= B.p[i];
+    float v[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = ldf(&B.v[r]);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      o = mfma32(B.n[r], B.v[r], o);
+      o = mfma32(B.n[r], v[r], o);
 #pragma unroll
-      for (int i = 0; i < DT; ++i) S[i] = mfma32(B.k[i][r], B.v[r], S[i]);
+      for (int i = 0; i < DT; ++i) S[i] = mfma32(B.k[i][r], v[r], S[i]);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r)
 #pragma unroll
       for (int i = 0; i < DT; ++i) S[i] = mfma32(B.a[i][r], y[r], S[i]);
+    float* op = P.out + (int64_t)(t0 + blk * 16) * P.H * dv + h * dv + col;
+    if (blk * 16 + 16 <= t1 - t0) {
+      if (colok) {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = t0 + blk * 16 + 4 * hh + r;
-      if (colok && t < t1) P.out[(int64_t)t * P.H * dv + h * dv + col] = o[r];
+        for (int r = 0; r < 4; ++r) op[(int64_t)(4 * hh + r) * P.H * dv] = o[r];
+      }
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (colok && blk * 16 + 4 * hh + r < t1 - t0) op[(int64_t)(4 * hh + r) * P.H * dv] = o[r];
     }
   };
   const int nblk = (t1 - t0 + 15) / 16;

@@ -257,12 +257,13 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_kernel(const RopeHead
   }
 }
 
-// bf16 rows, the rotation over the whole head (rot_dims = dk, dk % 16 == 0, dk / 2 a power of two
-// up to 512), 16-byte aligned rows, columns and pages: a lane owns 8 neighbouring pairs - elements
-// 8c .. 8c + 7 and the 8 elements half a head further - so every access is 16 bytes, a head takes
-// CPH = dk / 16 lanes and a wave works on 64 / CPH heads at a time. cos / sin of the token go
-// through the wave's LDS row (one sincos per lane). A wave takes the head rounds r = blockIdx.y,
-// + gridDim.y, ...; the last y also copies value columns of their own into the V page.
+// bf16 rows, rot_dims % 16 == 0, dk % 16 == 0, dk / 2 a power of two up to 512, 16-byte aligned rows,
+// columns and pages: a lane owns two runs of 8 elements, so every access is 16 bytes, a head takes
+// CPH = dk / 16 lanes and a wave works on 64 / CPH heads at a time. The first rot_dims / 16 lanes of a
+// head own 8 neighbouring pairs (elements 8c .. 8c + 7 and those rot_dims / 2 further), the others 16
+// unrotated elements (cos 1, sin 0). cos / sin of the token go through the wave's LDS row (one sincos
+// per lane). A wave takes the head rounds r = blockIdx.y, + gridDim.y, ...; the last y also copies
+// value columns of their own into the V page.
 __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const RopeHeadnormParams P, int64_t T_rows) {
   __shared__ __attribute__((aligned(16))) float cs_all[4][MAX_PAIRS], sn_all[4][MAX_PAIRS];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -272,8 +273,8 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const R
   float* sn = sn_all[wave];
   uint16_t* pr = (uint16_t*)P.proj + row * P.stride;
   const int p = P.pos[row] < 0 ? 0 : P.pos[row];
-  const int dk = P.dk, half = dk >> 1;
-  for (int i = lane; i < half; i += 64) {
+  const int dk = P.dk, half = dk >> 1, rhalf = P.rot_dims >> 1;
+  for (int i = lane; i < rhalf; i += 64) {
     const double turns = (double)p * P.freq[i] * 0.15915494309189535;   // angle / 2 pi
     const float a = (float)((turns - floor(turns)) * 6.283185307179586);
     float s, c;
@@ -288,11 +289,17 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const R
   const int CPH = half >> 3;               // lanes per head (a power of two <= 64)
   const int hpr = 64 / CPH;                // heads per round
   const int c8 = (lane & (CPH - 1)) * 8, hsub = lane / CPH;
+  const bool rot = c8 < rhalf;                       // (a lane's pairs are all rotated or none is)
+  const int ea = rot ? c8 : 2 * c8, eb = rot ? rhalf + c8 : 2 * c8 + 8;   // the lane's two runs of the head
   const int heads = P.H + P.G;
   float cc[8], sv[8];
 #pragma unroll
   for (int j = 0; j < 8; j += 4) {
-    const float4 c4 = *reinterpret_cast<const float4*>(cs + c8 + j), s4 = *reinterpret_cast<const float4*>(sn + c8 + j);
+    float4 c4 = make_float4(1.f, 1.f, 1.f, 1.f), s4 = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (rot) {
+      c4 = *reinterpret_cast<const float4*>(cs + c8 + j);
+      s4 = *reinterpret_cast<const float4*>(sn + c8 + j);
+    }
     cc[j] = c4.x, cc[j + 1] = c4.y, cc[j + 2] = c4.z, cc[j + 3] = c4.w;
     sv[j] = s4.x, sv[j + 1] = s4.y, sv[j + 2] = s4.z, sv[j + 3] = s4.w;
   }
@@ -302,11 +309,11 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const R
     const bool is_k = hh >= P.H;
     const int g = hh - P.H;
     uint16_t* src = pr + (int64_t)(live ? hh : 0) * dk;
-    const u16x8 ra = load8(src + c8), rb = load8(src + half + c8);
+    const u16x8 ra = load8(src + ea), rb = load8(src + eb);
     if (live && is_k && P.v_off < 0 && slot >= 0) {   // values = the keys as projected
       uint16_t* vd = (uint16_t*)P.vc + ((page * P.G + g) * 64 + in_page) * (int64_t)P.dv;
-      store8(vd + c8, ra);
-      store8(vd + half + c8, rb);
+      store8(vd + ea, ra);
+      store8(vd + eb, rb);
     }
     float xa[8], xb[8], ss = 0.f;
 #pragma unroll
@@ -322,8 +329,8 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const R
         const float r = 1.0f / sqrtf(ss / (float)dk + P.eps);
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          xa[j] *= r * w[c8 + j];
-          xb[j] *= r * w[half + c8 + j];
+          xa[j] *= r * w[ea + j];
+          xb[j] *= r * w[eb + j];
         }
       }
     }
@@ -334,12 +341,14 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const R
       oa[j] = f2bf(xa[j] * cc[j] - xb[j] * sv[j]);
       ob[j] = f2bf(xb[j] * cc[j] + xa[j] * sv[j]);
     }
-    store8(src + c8, oa);
-    store8(src + half + c8, ob);
+    if (rot || w != nullptr) {
+      store8(src + ea, oa);
+      store8(src + eb, ob);
+    }
     if (is_k && slot >= 0) {
       uint16_t* kd = (uint16_t*)P.kc + ((page * P.G + g) * 64 + in_page) * (int64_t)dk;
-      store8(kd + c8, oa);
-      store8(kd + half + c8, ob);
+      store8(kd + ea, oa);
+      store8(kd + eb, ob);
     }
   }
   if (P.v_off >= 0 && slot >= 0 && blockIdx.y == gridDim.y - 1) {
@@ -369,7 +378,7 @@ void launch_rope_headnorm_cache(const RopeHeadnormParams& p, int64_t T, bool f32
   if (p.rot_dims / 2 > MAX_PAIRS || p.dk > MAX_HEAD) abort();   // the binding checks both
   const int half = p.dk / 2;
   auto al16 = [](const void* q) { return ((uintptr_t)q % 16) == 0; };
-  if (!f32 && p.rot_dims == p.dk && p.dk % 16 == 0 && (half & (half - 1)) == 0 && half <= 512 && p.stride % 8 == 0 &&
+  if (!f32 && p.rot_dims % 16 == 0 && p.dk % 16 == 0 && (half & (half - 1)) == 0 && half <= 512 && p.stride % 8 == 0 &&
       al16(p.proj) && al16(p.kc) && al16(p.vc) && p.dv % 8 == 0 && (p.v_off < 0 || p.v_off % 8 == 0)) {
     const int hpr = 64 / (half / 8);
     const int rounds = (p.H + p.G + hpr - 1) / hpr;

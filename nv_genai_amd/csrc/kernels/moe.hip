@@ -54,6 +54,16 @@ __device__ __forceinline__ float gelu_tanh(float x) {
   return x - x / (1.f + __expf(2.f * u));
 }
 __device__ __forceinline__ float gelu_erf(float x) { return 0.5f * x * (1.f + erff(x * 0.7071067811865475f)); }
+// the same for results that are rounded to bf16: x Phi(x) with Phi(-|x|) = erfc(|x| / sqrt 2) / 2 from the
+// rational approximation 7.1.26 of Abramowitz and Stegun's Handbook of Mathematical Functions (absolute
+// error of erf below 1.5e-7) on the hardware exp2 and reciprocal; the tail is formed without cancellation
+__device__ __forceinline__ float gelu_erf_bf16(float x) {
+  const float z = fabsf(x) * 0.7071067811865475f;
+  const float t = __builtin_amdgcn_rcpf(1.0f + 0.3275911f * z);
+  const float p = t * (0.254829592f + t * (-0.284496736f + t * (1.421413741f + t * (-1.453152027f + t * 1.061405429f))));
+  const float tail = 0.5f * p * __builtin_amdgcn_exp2f(-1.4426950408889634f * z * z);
+  return x * (x > 0.f ? 1.0f - tail : tail);
+}
 // g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit)
 __device__ __forceinline__ float clamped_glu(float gate, float up, float limit, float alpha, float shift = 1.f) {
   const float g = fminf(gate, limit);
@@ -327,7 +337,7 @@ __global__ void __launch_bounds__(256) moe_gemm_kernel(MoeGemmParams P) {
         if (n >= P.w_rows) continue;
         u16x4 v;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) v[r] = f2bf(gelu_erf(acc[nt][mt][r]));
+        for (int r = 0; r < 4; ++r) v[r] = f2bf(gelu_erf_bf16(acc[nt][mt][r]));
         *reinterpret_cast<u16x4*>(op + n) = v;
       }
     } else {

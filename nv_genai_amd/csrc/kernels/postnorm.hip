@@ -226,6 +226,97 @@ __global__ void __launch_bounds__(256) residual_add_rmsnorm_kernel(float* __rest
   for (int c = threadIdx.x; c < H; c += blockDim.x) stf(out + row * H + c, xr[c] * r * w[c]);
 }
 
+// The two steps above for bf16 rows with H % 4 == 0 and aligned rows, the row held in registers: TPR
+// threads per row (a wave, or the workgroup when the rows are few), NV runs of four elements per
+// thread, one read and one write of the stream. POST: x += rmsnorm(y) * w and out = rmsnorm(x) * nw;
+// else x += y and out = rmsnorm(x) * nw (nw == nullptr: a copy of the sum; out == nullptr: the sum only).
+template <int TPR, int NV, bool POST>
+__global__ void __launch_bounds__(256) residual_step_bf16x4_kernel(float* __restrict__ x, const uint16_t* __restrict__ y,
+                                                                   int64_t y_stride, const float* __restrict__ w,
+                                                                   const float* __restrict__ nw, float eps, int H,
+                                                                   int64_t T_rows, uint16_t* __restrict__ out) {
+  __shared__ float red[4];
+  const int64_t row = TPR == 64 ? (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6) : (int64_t)blockIdx.x;
+  if (row >= T_rows) return;                 // (whole waves / workgroups)
+  const int l = TPR == 64 ? threadIdx.x & 63 : threadIdx.x;
+  float* xr = x + row * H;
+  const uint16_t* yr = y + row * y_stride;
+  float4 xv[NV], yv[NV];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * (l + TPR * i);
+    xv[i] = yv[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (c < H) {
+      xv[i] = *reinterpret_cast<const float4*>(xr + c);
+      const u16x4 a = *reinterpret_cast<const u16x4*>(yr + c);
+      yv[i] = make_float4(bf2f(a[0]), bf2f(a[1]), bf2f(a[2]), bf2f(a[3]));
+    }
+  }
+  auto total = [&](float v) { return TPR == 64 ? wave_sum(v) : block_sum(v, red); };
+  if (POST) {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) ss += yv[i].x * yv[i].x + yv[i].y * yv[i].y + yv[i].z * yv[i].z + yv[i].w * yv[i].w;
+    const float r = 1.0f / sqrtf(total(ss) / (float)H + eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = 4 * (l + TPR * i);
+      if (c < H) {
+        const float4 ww = *reinterpret_cast<const float4*>(w + c);
+        yv[i] = make_float4(yv[i].x * r * ww.x, yv[i].y * r * ww.y, yv[i].z * r * ww.z, yv[i].w * r * ww.w);
+      }
+    }
+  }
+  float s2 = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * (l + TPR * i);
+    xv[i].x += yv[i].x, xv[i].y += yv[i].y, xv[i].z += yv[i].z, xv[i].w += yv[i].w;
+    s2 += xv[i].x * xv[i].x + xv[i].y * xv[i].y + xv[i].z * xv[i].z + xv[i].w * xv[i].w;
+    if (c < H) *reinterpret_cast<float4*>(xr + c) = xv[i];
+  }
+  if (!out) return;
+  const float r2 = nw ? 1.0f / sqrtf(total(s2) / (float)H + eps) : 1.0f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * (l + TPR * i);
+    if (c < H) {
+      float4 ww = make_float4(1.f, 1.f, 1.f, 1.f);
+      if (nw) ww = *reinterpret_cast<const float4*>(nw + c);
+      u16x4 o;
+      o[0] = f2bf(xv[i].x * r2 * ww.x);
+      o[1] = f2bf(xv[i].y * r2 * ww.y);
+      o[2] = f2bf(xv[i].z * r2 * ww.z);
+      o[3] = f2bf(xv[i].w * r2 * ww.w);
+      *reinterpret_cast<u16x4*>(out + row * H + c) = o;
+    }
+  }
+}
+
+template <bool POST>
+bool launch_residual_step_vec(float* x, const uint16_t* y, int64_t y_stride, const float* w, const float* nw, float eps,
+                              int64_t T, int H, uint16_t* out, hipStream_t stream) {
+  auto al = [](const void* p, int a) { return ((uintptr_t)p % a) == 0; };
+  if (H % 4 || H > 8192 || y_stride % 4 || !al(x, 16) || !al(y, 8) || !al(w, 16) || !al(nw, 16) || !al(out, 8)) return false;
+#define NGA_STEP(TPR, NV)                                                                                              \
+  residual_step_bf16x4_kernel<TPR, NV, POST><<<dim3((unsigned)(TPR == 64 ? (T + 3) / 4 : T)), 256, 0, stream>>>(        \
+      x, y, y_stride, w, nw, eps, H, T, out)
+  if (T >= 4096 && H <= 4096) {      // rows enough to fill the chip with one wave each
+    if (H <= 256) NGA_STEP(64, 1);
+    else if (H <= 512) NGA_STEP(64, 2);
+    else if (H <= 1024) NGA_STEP(64, 4);
+    else if (H <= 2048) NGA_STEP(64, 8);
+    else NGA_STEP(64, 16);
+  } else {
+    if (H <= 1024) NGA_STEP(256, 1);
+    else if (H <= 2048) NGA_STEP(256, 2);
+    else if (H <= 4096) NGA_STEP(256, 4);
+    else NGA_STEP(256, 8);
+  }
+#undef NGA_STEP
+  return true;
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ in,
                                                           int64_t in_stride, int64_t T_rows, int F, float limit,
@@ -548,6 +639,28 @@ __global__ void __launch_bounds__(256) gelu_gate_rows_kernel(T* __restrict__ out
   }
 }
 
+// bf16, C % 8 == 0, aligned rows: 8 elements per thread
+__global__ void __launch_bounds__(256) gelu_gate_rows_bf16x8_kernel(uint16_t* __restrict__ out, const uint16_t* __restrict__ z,
+                                                                    int64_t z_stride, const int32_t* __restrict__ ids,
+                                                                    const uint16_t* __restrict__ table, int64_t t_stride,
+                                                                    int rows, int C8, int vocab) {
+  const int total = rows * C8;
+  for (int i = blockIdx.x * blockDim.x + threadIdx.x; i < total; i += gridDim.x * blockDim.x) {
+    const int t = i / C8, c = (i - t * C8) * 8;
+    int id = ids[t];
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    const u16x8 a = load8(z + (int64_t)t * z_stride + c), e = load8(table + (int64_t)id * t_stride + c);
+    u16x8 o;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float v = bf2f(a[j]), q = 0.7978845608028654f * (v + 0.044715f * v * v * v);
+      // gelu_tanh = v - v / (1 + e^(2q))
+      o[j] = f2bf((v - v * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.8853900817779268f * q))) * bf2f(e[j]));
+    }
+    store8(out + (int64_t)i * 8, o);
+  }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) tanh_rows_kernel(T* __restrict__ out, const T* __restrict__ x, int64_t x_stride,
                                                         int64_t total, int C) {
@@ -627,6 +740,9 @@ void launch_embed_rows(float* x, const int32_t* ids, const void* embed, float sc
 void launch_rmsnorm_residual_next(float* x, const void* y, int64_t y_stride, const float* w, int w_n, const float* nw,
                                   int nw_n, float eps, int64_t T, int H, void* out, bool f32, hipStream_t stream) {
   if (T == 0) return;
+  if (!f32 && w_n == H && nw_n == H &&
+      launch_residual_step_vec<true>(x, (const uint16_t*)y, y_stride, w, nw, eps, T, H, (uint16_t*)out, stream))
+    return;
   const int ws = w_n == 1 ? 0 : 1, nws = nw_n == 1 ? 0 : 1;
   if (f32)
     rmsnorm_residual_next_kernel<float><<<dim3((unsigned)T), 256, 0, stream>>>(x, (const float*)y, y_stride, w, ws, nw,
@@ -662,6 +778,8 @@ void launch_softcap(float* z, int64_t n, float cap, float scale, hipStream_t str
 void launch_residual_add_rmsnorm(float* x, const void* y, int64_t y_stride, const float* w, float eps, int64_t T, int H,
                                  void* out, bool f32, hipStream_t stream) {
   if (T == 0) return;
+  if (!f32 && launch_residual_step_vec<false>(x, (const uint16_t*)y, y_stride, nullptr, w, eps, T, H, (uint16_t*)out, stream))
+    return;
   if (f32)
     residual_add_rmsnorm_kernel<float><<<dim3((unsigned)T), 256, 0, stream>>>(x, (const float*)y, y_stride, w, eps, H,
                                                                              (float*)out);
@@ -793,6 +911,15 @@ void launch_gelu_gate_rows(void* out, const void* z, int64_t z_stride, const int
                            int64_t t_stride, int64_t T, int C, int vocab, bool f32, hipStream_t stream) {
   const int64_t total = T * C;
   if (total == 0) return;
+  if (!f32 && C % 8 == 0 && z_stride % 8 == 0 && t_stride % 8 == 0 && total < (1ll << 31) && ((uintptr_t)z % 16) == 0 &&
+      ((uintptr_t)table % 16) == 0 && ((uintptr_t)out % 16) == 0) {
+    int64_t g8 = (total / 8 + 255) / 256;
+    if (g8 > 8192) g8 = 8192;
+    gelu_gate_rows_bf16x8_kernel<<<dim3((unsigned)g8), 256, 0, stream>>>((uint16_t*)out, (const uint16_t*)z, z_stride, ids,
+                                                                        (const uint16_t*)table, t_stride, (int)T, C / 8,
+                                                                        vocab);
+    return;
+  }
   int64_t g = (total + 255) / 256;
   if (g > 8192) g = 8192;
   if (f32)

@@ -466,9 +466,10 @@ bool launch_mlstm_t(float* out, const T* proj, int64_t stride, const float* gate
 // ---------------------------------------------------------------------------------------------
 // Short convolution: out[t] = silu(sum_j taps[n - 1 - j][c] x[t - j]), V channels per thread. Inputs in
 // front of the segment come from the state slot [n - 1][C] (oldest first), zeros in front of
-// position 0. SINGLE = false: rows of portions (seq[t]: the row's segment), the slots are written by
-// short_conv_save_kernel behind this launch; SINGLE = true: every row is a segment, and the thread that reads
-// its channels of the slot also writes them.
+// position 0. short_conv_kernel: any row; SINGLE = true: every row is a segment, and the thread that
+// reads its channels of the slot also writes them; SINGLE = false: rows of portions (seq[t]: the row's
+// segment), the slots are written by short_conv_save_kernel behind the launch.
+// short_conv_rows_kernel: portions, CR rows per thread with the window of inputs in registers.
 constexpr int MAX_TAPS = 16;
 
 template <typename T, int V>
@@ -550,6 +551,59 @@ __global__ void __launch_bounds__(256) short_conv_kernel(T* __restrict__ out, co
   }
 }
 
+constexpr int CR = 8;
+template <int NT>
+__global__ void __launch_bounds__(256) short_conv_rows_kernel(uint16_t* __restrict__ out, const uint16_t* __restrict__ x,
+                                                              int64_t x_stride, const float* __restrict__ taps,
+                                                              const uint16_t* __restrict__ state, int C,
+                                                              const int32_t* __restrict__ cu,
+                                                              const int32_t* __restrict__ slots,
+                                                              const int32_t* __restrict__ seq,
+                                                              const int32_t* __restrict__ pos, int64_t rows) {
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 8;
+  if (c >= C) return;
+  float tp[NT][8];
+#pragma unroll
+  for (int j = 0; j < NT; ++j)
+#pragma unroll
+    for (int e = 0; e < 8; e += 4) {
+      const float4 t4 = *reinterpret_cast<const float4*>(taps + (int64_t)j * C + c + e);
+      tp[j][e] = t4.x, tp[j][e + 1] = t4.y, tp[j][e + 2] = t4.z, tp[j][e + 3] = t4.w;
+    }
+  const int64_t r0 = (int64_t)blockIdx.x * CR;
+  const int n = (int)(rows - r0 < CR ? rows - r0 : CR);
+  u16x8 w[CR + NT - 1];       // the rows and, in front of them, the inputs ahead of the first one
+#pragma unroll
+  for (int i = 0; i < CR; ++i)
+    if (i < n) w[NT - 1 + i] = load8(x + (r0 + i) * x_stride + c);
+  auto before = [&](int64_t row, int j) -> u16x8 {      // input j rows ahead of `row`, by its segment
+    const int b = seq[row], in_seg = (int)row - cu[b], slot = slots[b], p = pos[row];
+    if (j <= in_seg) return load8(x + (row - j) * x_stride + c);
+    if (p - j >= 0 && slot >= 0) return load8(state + ((int64_t)slot * (NT - 1) + NT - 1 - (j - in_seg)) * C + c);
+    return (u16x8)(0);
+  };
+#pragma unroll
+  for (int j = 1; j < NT; ++j) w[NT - 1 - j] = before(r0, j);
+  const bool one = seq[r0] == seq[r0 + n - 1];         // (uniform) all rows of one segment: the window slides
+#pragma unroll
+  for (int i = 0; i < CR; ++i) {
+    if (i >= n) break;
+    float acc[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) acc[e] = 0.f;
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+      const u16x8 v = (one || j == 0 || i == 0) ? w[NT - 1 + i - j] : before(r0 + i, j);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[e] += tp[NT - 1 - j][e] * bf2f(v[e]);
+    }
+    u16x8 o;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) o[e] = f2bf(acc[e] * sigmoid_fast(acc[e]));
+    store8(out + (r0 + i) * C + c, o);
+  }
+}
+
 // the last n - 1 inputs of every segment into its slot; entry e takes row t1 - (n - 1) + e, which may
 // lie in front of the segment: then the old entry e + rows (read in front of its own rewrite: e ascends)
 template <typename T>
@@ -595,8 +649,16 @@ void launch_short_conv_t(T* out, const T* x, int64_t x_stride, const float* taps
     else launch_short_conv_v<T, 1, true>(NGA_CONV_ARGS);
     return;
   }
-  if (vec) launch_short_conv_v<T, sizeof(T) == 2 ? 8 : 1, false>(NGA_CONV_ARGS);
-  else launch_short_conv_v<T, 1, false>(NGA_CONV_ARGS);
+  if (vec && rows >= 512 && (n == 3 || n == 4) && ((uintptr_t)taps % 16) == 0) {
+    const dim3 grid((unsigned)((rows + CR - 1) / CR), (unsigned)((C / 8 + 255) / 256));
+    auto k = n == 4 ? &short_conv_rows_kernel<4> : &short_conv_rows_kernel<3>;
+    k<<<grid, 256, 0, stream>>>((uint16_t*)out, (const uint16_t*)x, x_stride, taps, (const uint16_t*)state, C, cu, slots,
+                                seq, pos, rows);
+  } else if (vec) {
+    launch_short_conv_v<T, sizeof(T) == 2 ? 8 : 1, false>(NGA_CONV_ARGS);
+  } else {
+    launch_short_conv_v<T, 1, false>(NGA_CONV_ARGS);
+  }
 #undef NGA_CONV_ARGS
   if (n > 1)
     short_conv_save_kernel<T><<<dim3((unsigned)((C + 255) / 256), (unsigned)n_seg), 256, 0, stream>>>(x, x_stride, state, C,
