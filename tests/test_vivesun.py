@@ -805,6 +805,65 @@ def test_mfma_forms_run_and_agree_with_the_plain_kernels():
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("n", [3, 4])
+def test_convolution_of_many_rows(n):
+    """The form with the window of inputs in registers (bf16, hundreds of rows): segments of one, two and
+    many rows whose borders fall anywhere in a thread's run of rows, fresh and going on from slots."""
+    dev = "cuda"
+    g = torch.Generator().manual_seed(31)
+    C, lens = 72, [300, 1, 2, 5, 8, 250, 3, 17]
+    T = 400
+    xs = [torch.randn(T, C, generator=g).bfloat16() for _ in lens]
+    taps = torch.randn(C, n, generator=g)
+    want = [O.short_conv(x.double(), taps) for x in xs]
+    td = taps.t().contiguous().to(dev)
+    state = torch.full((len(lens), n - 1, C), 9.0, dtype=torch.bfloat16, device=dev)
+    start = [0, 40, 1, 0, 2, 100, 0, 7]            # rows of the sequence already seen
+    for i, s in enumerate(start):
+        if s:
+            pos = torch.arange(s, dtype=torch.int32, device=dev)
+            ops.short_conv(xs[i][:s].to(dev), td, state, i32(0, s, device=dev), i32(i, device=dev), torch.zeros_like(pos), pos)
+    wide = torch.zeros(sum(lens), C + 8, dtype=torch.bfloat16, device=dev)
+    x = wide[:, :C]
+    x.copy_(torch.cat([xs[i][s:s + k] for i, (s, k) in enumerate(zip(start, lens))]))
+    pos = torch.cat([torch.arange(s, s + k) for s, k in zip(start, lens)]).to(torch.int32).to(dev)
+    seq = torch.cat([torch.full((k,), i) for i, k in enumerate(lens)]).to(torch.int32).to(dev)
+    cu = torch.tensor([0] + lens).cumsum(0).to(torch.int32).to(dev)
+    assert sum(lens) >= 512
+    got = ops.short_conv(x, td, state, cu, torch.arange(len(lens), dtype=torch.int32, device=dev), seq, pos)
+    close(got, torch.cat([want[i][s:s + k] for i, (s, k) in enumerate(zip(start, lens))]), "bfloat16", "many rows")
+    for i, (s, k) in enumerate(zip(start, lens)):
+        pad = torch.cat([torch.zeros(n - 1, C).bfloat16(), xs[i][:s + k]])[-(n - 1):]
+        assert torch.equal(state[i].cpu(), pad), f"inputs left in slot {i}"
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("T,H", [(5000, 256), (4097, 1024), (4100, 3000), (37, 1024), (40, 5120), (33, 30)])
+def test_residual_steps_of_many_rows(T, H):
+    """The residual steps with the row in registers (one wave per row, one workgroup per row) and the
+    scalar form: sum, copy, norm of the sum, norm of the sub-layer's output in front of the sum."""
+    dev = "cuda"
+    g = torch.Generator().manual_seed(37)
+    x0, y = 3.0 * torch.randn(T, H, generator=g), torch.randn(T, H, generator=g).bfloat16()
+    w, nw = 1 + 0.2 * torch.randn(H, generator=g), 1 + 0.2 * torch.randn(H, generator=g)
+    xd, yd = x0.double(), y.double()
+    eps = 1e-3
+    x = x0.to(dev)
+    h = ops.residual_add_rmsnorm_(x, y.to(dev), nw.to(dev), eps, torch.bfloat16)
+    close(x, xd + yd, "float32", "sum")
+    close(h, O.unit_rms(xd + yd, eps) * nw.double(), "bfloat16", "norm of the sum")
+    assert ops.residual_add_rmsnorm_(x, y.to(dev), None, eps, torch.bfloat16) is None
+    close(x, xd + 2 * yd, "float32", "sum alone")
+    x = x0.to(dev)
+    close(ops.residual_add_cast_(x, y.to(dev), torch.bfloat16), xd + yd, "bfloat16", "copy")
+    x = x0.to(dev)
+    h = ops.rmsnorm_residual_next_(x, y.to(dev), w.to(dev), eps, nw.to(dev), torch.bfloat16)
+    xs = xd + O.unit_rms(yd, eps) * w.double()
+    close(x, xs, "float32", "sum of the normed output")
+    close(h, O.unit_rms(xs, eps) * nw.double(), "bfloat16", "next norm")
+
+
+@pytest.mark.gpu
 def test_captured_decode_graph_replays():
     """Decode steps from the captured graph, several in a row with eager steps of other sequences in
     between, against eager decoding of the same tokens: state, convolution inputs and previous
