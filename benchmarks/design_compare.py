@@ -647,7 +647,7 @@ def vivesun_kernel_times(z: dict, iters: int = 20) -> dict:
     rb = router.to(bf)
 
     def viv(xx):
-        ids, wts = ops.moe_route_grouped(ops.linear(xx.float(), router), None, k, 1, 1, 2.0)
+        ids, wts = ops.moe_router(xx, router, k, 2.0)
         return ops.moe_plain_experts(xx, ids, wts, w1, w2)
 
     ex = {}

@@ -317,6 +317,20 @@ void moe_route_grouped(Tensor logits, c10::optional<Tensor> correction, int64_t 
                                 w.data_ptr<float>(), cur_stream(logits));
 }
 
+// router product + softmax scores + top-k + weights of few rows
+void moe_router_rows(Tensor x, Tensor router, int64_t k, double scale, Tensor ids, Tensor w) {
+  const bool f32 = act_f32(x);
+  CHECK_DEV(router); CHECK_DT(router, at::kFloat); CHECK_CONTIG(router);
+  const int64_t T = x.size(0), H = x.size(1), E = router.size(0);
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && router.dim() == 2 && router.size(1) == H && H <= 8192);
+  TORCH_CHECK(E >= 1 && E <= 512 && k >= 1 && k <= E && k <= 64, "moe_router_rows: E <= 512, k <= min(E, 64)");
+  CHECK_DEV(ids); CHECK_DT(ids, at::kInt); CHECK_DEV(w); CHECK_DT(w, at::kFloat);
+  TORCH_CHECK(ids.is_contiguous() && w.is_contiguous() && ids.numel() >= T * k && w.numel() >= T * k &&
+              (uintptr_t)router.data_ptr() % 16 == 0);
+  nga::launch_moe_router_rows(x.data_ptr(), x.stride(0), router.data_ptr<float>(), (int)T, (int)H, (int)E, (int)k,
+                              (float)scale, ids.data_ptr<int32_t>(), w.data_ptr<float>(), f32, cur_stream(x));
+}
+
 void moe_combine_rows(Tensor y, Tensor inv, int64_t T, int64_t k, c10::optional<Tensor> add, Tensor out,
                       c10::optional<Tensor> id_x, c10::optional<Tensor> ids, c10::optional<Tensor> wts, int64_t E) {
   const bool f32 = act_f32(y);
@@ -1289,11 +1303,18 @@ void softcap(Tensor z, double cap, double scale) {
 void check_row_pages(const Tensor& act, const Tensor& c, int64_t heads, int64_t d, const char* what);
 const float* opt_f32(const c10::optional<Tensor>& t, int64_t n, const char* what);
 
-void residual_add_rmsnorm(Tensor x, Tensor y, c10::optional<Tensor> w, double eps, c10::optional<Tensor> out) {
+void residual_add_rmsnorm(Tensor x, Tensor y, c10::optional<Tensor> w, double eps, c10::optional<Tensor> out,
+                          c10::optional<Tensor> inv, int64_t k) {
   CHECK_F32(x);
   const bool f32 = act_f32(y);
   const int64_t H = x.size(1);
-  TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && y.size(0) == x.size(0) && y.size(1) == H && y.stride(1) == 1);
+  const int32_t* ip = nullptr;
+  if (inv.has_value()) {   // rows of y gathered by number (numbers < y rows: moe_align writes them below T * k)
+    CHECK_I32(*inv);
+    TORCH_CHECK(k >= 1 && inv->numel() >= x.size(0) * k && y.size(0) >= x.size(0) * k);
+    ip = inv->data_ptr<int32_t>();
+  }
+  TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && (ip || y.size(0) == x.size(0)) && y.size(1) == H && y.stride(1) == 1);
   TORCH_CHECK(!w.has_value() || out.has_value(), "residual_add_rmsnorm: a norm weight needs an output");
   void* op = nullptr;
   if (out.has_value()) {
@@ -1302,7 +1323,7 @@ void residual_add_rmsnorm(Tensor x, Tensor y, c10::optional<Tensor> w, double ep
     op = out->data_ptr();
   }
   nga::launch_residual_add_rmsnorm(x.data_ptr<float>(), y.data_ptr(), y.stride(0), opt_f32(w, H, "norm weight"),
-                                   (float)eps, x.size(0), (int)H, op, f32, cur_stream(x));
+                                   (float)eps, x.size(0), (int)H, op, ip, (int)k, f32, cur_stream(x));
 }
 
 void clamped_glu(Tensor out, Tensor x, int64_t F, double limit, double alpha, int64_t gate_col, double shift) {
@@ -1936,6 +1957,7 @@ PYBIND11_MODULE(_C, m) {
   m.def("moe_gemm", checked("moe_gemm", &moe_gemm));
   m.def("moe_combine", checked("moe_combine", &moe_combine));
   m.def("moe_route_scores", checked("moe_route_scores", &moe_route_scores));
+  m.def("moe_router_rows", checked("moe_router_rows", &moe_router_rows));
   m.def("moe_gemm_rows", checked("moe_gemm_rows", &moe_gemm_rows));
   m.def("moe_combine_rows", checked("moe_combine_rows", &moe_combine_rows));
   m.def("skinny_cfg", &skinny_cfg);

@@ -196,6 +196,9 @@ void launch_moe_combine_rows(const void* y, const int32_t* inv, int T, int k, in
                              const float* wts, int E, bool f32, hipStream_t stream);
 void launch_moe_route_grouped(const float* logits, int64_t ld, const float* correction, int T, int E, int k, int groups,
                               int keep, float scale, int32_t* ids, float* w, hipStream_t stream);
+// router product, softmax scores, top-k and weights of few rows in one launch (E <= 512, k <= 64)
+void launch_moe_router_rows(const void* x, int64_t ldx, const float* router, int T, int H, int E, int k, float scale,
+                            int32_t* ids, float* w, bool f32, hipStream_t stream);
 void launch_moe_route(const uint16_t* logits, int64_t ld, int T, int E, int k, int32_t* ids,
                       float* w, hipStream_t stream);
 void launch_moe_align(const int32_t* ids, const float* w, int M, int k, int e0, int E, int bm,
@@ -296,8 +299,9 @@ void launch_rmsnorm_residual_next(float* x, const void* y, int64_t y_stride, con
                                   int nw_n, float eps, int64_t T, int H, void* out, bool f32, hipStream_t stream);
 void launch_relu_sq(void* out, const void* in, int64_t n, bool f32, hipStream_t stream);
 void launch_softcap(float* z, int64_t n, float cap, float scale, hipStream_t stream);
+// inv != nullptr: row t adds the sum of the k rows inv[t k ..] of y (< 0: none)
 void launch_residual_add_rmsnorm(float* x, const void* y, int64_t y_stride, const float* w, float eps, int64_t T, int H,
-                                 void* out, bool f32, hipStream_t stream);
+                                 void* out, const int32_t* inv, int k, bool f32, hipStream_t stream);
 void launch_clamped_glu(void* out, const void* in, int64_t in_stride, int64_t T, int F, float limit, float alpha,
                         int gate_col, float shift, bool f32, hipStream_t stream);
 void launch_dyt_norm(void* out, const float* x, float alpha, const float* w, const float* b, const int64_t* rows,

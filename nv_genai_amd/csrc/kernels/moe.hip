@@ -24,6 +24,7 @@
 //                and the true-fp32 path)
 //   moe_combine_rows  moe_combine for any width and type, plus an optional added row (a shared
 //                expert's output) and identity experts (ids >= E: weight * the token's own row)
+//   moe_router_rows   router product, softmax scores, top-k and weights of few rows in one launch
 //   moe_route_grouped fp32 router logits -> softmax scores, choice by score + correction inside
 //                the best groups of experts, top-k ids + weights renormalised and scaled
 //
@@ -517,14 +518,6 @@ __global__ void __launch_bounds__(RG_THREADS) moe_route_grouped_kernel(
   for (int j = 0; j < k; ++j) w[(int64_t)t * k + j] *= r;
 }
 
-// ------------------------------------------------------------------ grouped GEMM on VALU tiles
-// Workgroup (256 threads) = one M tile of the table (<= 64 sorted rows of one expert) x 64
-// output columns; K in steps of 16 through LDS; a thread owns 4 rows x 4 columns (fp32). MODE 0:
-// gathered token rows x the expert's gate and up rows of the same 64 features (two accumulator
-// sets), epilogue = routing weight on the input (optional) and the clamped GLU; MODE 1: sorted
-// activation rows x the expert's down rows, optionally times the routing weight; MODE 2: gathered
-// token rows x the expert's rows, gelu (erf). No alignment
-// or divisibility is assumed.
 namespace {
 template <typename T> __device__ __forceinline__ float ldv(const T* p);
 template <> __device__ __forceinline__ float ldv<uint16_t>(const uint16_t* p) { return bf2f(*p); }
@@ -534,6 +527,107 @@ template <> __device__ __forceinline__ void stv<uint16_t>(uint16_t* p, float v) 
 template <> __device__ __forceinline__ void stv<float>(float* p, float v) { *p = v; }
 constexpr int RT = 64, RK = 16;
 }  // namespace
+
+// ------------------------------------------------------------------ router of few rows
+// One workgroup per row: the row as fp32 in LDS, every wave takes experts w, w + 4, ... four at a time
+// (fp32 products with the fp32 router rows), then the first wave forms the softmax over all E and picks
+// the k largest scores one after the other (ties: the lower index): weights = chosen scores / (their
+// sum + 1e-20) * scale, all fp32.
+constexpr int RR_MAX_E = 512;
+template <typename T>
+__global__ void __launch_bounds__(256) moe_router_rows_kernel(const T* __restrict__ x, int64_t ldx,
+                                                              const float* __restrict__ router, int H, int E, int k,
+                                                              float scale, int32_t* __restrict__ ids,
+                                                              float* __restrict__ w) {
+  extern __shared__ __attribute__((aligned(16))) float rr_s[];   // [H] the row, [E] logits
+  float* z = rr_s + (H + 3) / 4 * 4;
+  const int64_t t = blockIdx.x;
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+  for (int c = threadIdx.x; c < H; c += 256) rr_s[c] = ldv(x + t * ldx + c);
+  __syncthreads();
+  const bool vec = H % 4 == 0;
+  for (int e0 = wv * 4; e0 < E; e0 += 16) {
+    const int n = min(4, E - e0);
+    const float* r = router + (int64_t)e0 * H;
+    float a[4] = {0.f, 0.f, 0.f, 0.f};
+    if (vec) {
+      for (int c = 4 * lane; c < H; c += 256) {
+        const float4 xv = *reinterpret_cast<const float4*>(rr_s + c);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float4 rv = *reinterpret_cast<const float4*>(r + (int64_t)(j < n ? j : 0) * H + c);
+          a[j] += xv.x * rv.x + xv.y * rv.y + xv.z * rv.z + xv.w * rv.w;
+        }
+      }
+    } else {
+      for (int c = lane; c < H; c += 64)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) a[j] += rr_s[c] * r[(int64_t)(j < n ? j : 0) * H + c];
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      a[j] = wave_sum(a[j]);
+      if (lane == 0 && j < n) z[e0 + j] = a[j];
+    }
+  }
+  __syncthreads();
+  if (wv) return;
+  constexpr int PE = RR_MAX_E / 64;
+  float s[PE], mx = -INFINITY, den = 0.f;
+#pragma unroll
+  for (int q = 0; q < PE; ++q) {
+    s[q] = lane + 64 * q < E ? z[lane + 64 * q] : -INFINITY;
+    mx = fmaxf(mx, s[q]);
+  }
+  mx = wave_max(mx);
+#pragma unroll
+  for (int q = 0; q < PE; ++q) {
+    s[q] = lane + 64 * q < E ? expf(s[q] - mx) : -1.f;
+    if (s[q] >= 0.f) den += s[q];
+  }
+  den = wave_sum(den);
+#pragma unroll
+  for (int q = 0; q < PE; ++q)
+    if (s[q] >= 0.f) s[q] /= den;
+  float sum = 0.f, mine = 0.f;
+  for (int j = 0; j < k; ++j) {
+    float best = -1.f;
+    int bi = 1 << 30;
+#pragma unroll
+    for (int q = 0; q < PE; ++q)
+      if (s[q] > best) {
+        best = s[q];
+        bi = lane + 64 * q;
+      }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(best, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ob > best || (ob == best && oi < bi)) {
+        best = ob;
+        bi = oi;
+      }
+    }
+#pragma unroll
+    for (int q = 0; q < PE; ++q)
+      if (bi == lane + 64 * q) s[q] = -1.f;      // taken
+    sum += best;
+    if (lane == j) {      // lane j keeps choice j (k <= 64)
+      mine = best;
+      ids[t * k + j] = bi;
+    }
+  }
+  if (lane < k) w[t * k + lane] = mine * (scale / (sum + 1e-20f));
+}
+
+// ------------------------------------------------------------------ grouped GEMM on VALU tiles
+// Workgroup (256 threads) = one M tile of the table (<= 64 sorted rows of one expert) x 64
+// output columns; K in steps of 16 through LDS; a thread owns 4 rows x 4 columns (fp32). MODE 0:
+// gathered token rows x the expert's gate and up rows of the same 64 features (two accumulator
+// sets), epilogue = routing weight on the input (optional) and the clamped GLU; MODE 1: sorted
+// activation rows x the expert's down rows, optionally times the routing weight; MODE 2: gathered
+// token rows x the expert's rows, gelu (erf). No alignment
+// or divisibility is assumed.
 
 template <typename T, int MODE>
 __global__ void __launch_bounds__(256) moe_gemm_rows_kernel(MoeRowsParams P) {
@@ -699,6 +793,17 @@ void launch_moe_route_grouped(const float* logits, int64_t ld, const float* corr
   }
   moe_route_grouped_kernel<<<(T + RG_THREADS - 1) / RG_THREADS, RG_THREADS, smem, stream>>>(logits, ld, correction, T, E, k,
                                                                                            groups, keep, scale, ids, w);
+}
+
+void launch_moe_router_rows(const void* x, int64_t ldx, const float* router, int T, int H, int E, int k, float scale,
+                            int32_t* ids, float* w, bool f32, hipStream_t stream) {
+  if (T == 0) return;
+  if (E > RR_MAX_E || k > 64) abort();   // the binding checks both
+  const size_t smem = (size_t)((H + 3) / 4 * 4 + E) * sizeof(float);
+  if (f32)
+    moe_router_rows_kernel<float><<<T, 256, smem, stream>>>((const float*)x, ldx, router, H, E, k, scale, ids, w);
+  else
+    moe_router_rows_kernel<uint16_t><<<T, 256, smem, stream>>>((const uint16_t*)x, ldx, router, H, E, k, scale, ids, w);
 }
 
 void launch_moe_gemm_rows(const MoeRowsParams& p, int mode, bool f32, hipStream_t stream) {

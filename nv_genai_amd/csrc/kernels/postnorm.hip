@@ -13,7 +13,8 @@
 //   relu_sq           relu(x)^2
 //   softcap           z = cap * tanh(z * scale / cap) on fp32 logits
 //   residual_add_rmsnorm   x[t] += y[t], out[t] = rmsnorm(x[t]) * w: the residual sum of one
-//                     pre-norm sub-layer and the norm in front of the next in one pass
+//                     pre-norm sub-layer and the norm in front of the next in one pass; y[t] may be
+//                     the sum of a token's expert rows (inv: their k row numbers, < 0: none)
 //   clamped_glu       [gate F | up F | ...] -> g sigmoid(alpha g) (u + shift), g = min(gate, limit),
 //                     u = clamp(up, +-limit), optionally times sigmoid of one gate column of the row
 //   group_rmsnorm     RMS norm of each of G equal column groups of fp32 rows (heads), weight per
@@ -205,14 +206,24 @@ __global__ void __launch_bounds__(256) relu_sq_bf16x8_kernel(uint16_t* __restric
 template <typename T>
 __global__ void __launch_bounds__(256) residual_add_rmsnorm_kernel(float* __restrict__ x, const T* __restrict__ y,
                                                                    int64_t y_stride, const float* __restrict__ w,
-                                                                   float eps, int H, T* __restrict__ out) {
+                                                                   float eps, int H, T* __restrict__ out,
+                                                                   const int32_t* __restrict__ inv, int k) {
   __shared__ float red[4];
   const int64_t row = blockIdx.x;
   const T* yr = y + row * y_stride;
   float* xr = x + row * H;
   float ss = 0.f;
   for (int c = threadIdx.x; c < H; c += blockDim.x) {
-    const float v = xr[c] + ldf(yr + c);
+    float a = 0.f;
+    if (inv) {
+      for (int j = 0; j < k; ++j) {
+        const int p = inv[row * k + j];
+        if (p >= 0) a += ldf(y + (int64_t)p * y_stride + c);
+      }
+    } else {
+      a = ldf(yr + c);
+    }
+    const float v = xr[c] + a;
     xr[c] = v;
     ss += v * v;
   }
@@ -229,12 +240,14 @@ __global__ void __launch_bounds__(256) residual_add_rmsnorm_kernel(float* __rest
 // The two steps above for bf16 rows with H % 4 == 0 and aligned rows, the row held in registers: TPR
 // threads per row (a wave, or the workgroup when the rows are few), NV runs of four elements per
 // thread, one read and one write of the stream. POST: x += rmsnorm(y) * w and out = rmsnorm(x) * nw;
-// else x += y and out = rmsnorm(x) * nw (nw == nullptr: a copy of the sum; out == nullptr: the sum only).
+// else x += y and out = rmsnorm(x) * nw (nw == nullptr: a copy of the sum; out == nullptr: the sum only;
+// inv: y[t] is the sum of the k rows inv[t k ..] of y, in fp32).
 template <int TPR, int NV, bool POST>
 __global__ void __launch_bounds__(256) residual_step_bf16x4_kernel(float* __restrict__ x, const uint16_t* __restrict__ y,
                                                                    int64_t y_stride, const float* __restrict__ w,
                                                                    const float* __restrict__ nw, float eps, int H,
-                                                                   int64_t T_rows, uint16_t* __restrict__ out) {
+                                                                   int64_t T_rows, uint16_t* __restrict__ out,
+                                                                   const int32_t* __restrict__ inv, int k) {
   __shared__ float red[4];
   const int64_t row = TPR == 64 ? (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6) : (int64_t)blockIdx.x;
   if (row >= T_rows) return;                 // (whole waves / workgroups)
@@ -248,8 +261,25 @@ __global__ void __launch_bounds__(256) residual_step_bf16x4_kernel(float* __rest
     xv[i] = yv[i] = make_float4(0.f, 0.f, 0.f, 0.f);
     if (c < H) {
       xv[i] = *reinterpret_cast<const float4*>(xr + c);
-      const u16x4 a = *reinterpret_cast<const u16x4*>(yr + c);
-      yv[i] = make_float4(bf2f(a[0]), bf2f(a[1]), bf2f(a[2]), bf2f(a[3]));
+      if (!inv) {
+        const u16x4 a = *reinterpret_cast<const u16x4*>(yr + c);
+        yv[i] = make_float4(bf2f(a[0]), bf2f(a[1]), bf2f(a[2]), bf2f(a[3]));
+      }
+    }
+  }
+  if (inv) {
+    for (int j = 0; j < k; ++j) {
+      const int p = inv[row * k + j];
+      if (p < 0) continue;
+      const uint16_t* pr = y + (int64_t)p * y_stride;
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = 4 * (l + TPR * i);
+        if (c < H) {
+          const u16x4 a = *reinterpret_cast<const u16x4*>(pr + c);
+          yv[i].x += bf2f(a[0]), yv[i].y += bf2f(a[1]), yv[i].z += bf2f(a[2]), yv[i].w += bf2f(a[3]);
+        }
+      }
     }
   }
   auto total = [&](float v) { return TPR == 64 ? wave_sum(v) : block_sum(v, red); };
@@ -295,12 +325,12 @@ __global__ void __launch_bounds__(256) residual_step_bf16x4_kernel(float* __rest
 
 template <bool POST>
 bool launch_residual_step_vec(float* x, const uint16_t* y, int64_t y_stride, const float* w, const float* nw, float eps,
-                              int64_t T, int H, uint16_t* out, hipStream_t stream) {
+                              int64_t T, int H, uint16_t* out, const int32_t* inv, int k, hipStream_t stream) {
   auto al = [](const void* p, int a) { return ((uintptr_t)p % a) == 0; };
   if (H % 4 || H > 8192 || y_stride % 4 || !al(x, 16) || !al(y, 8) || !al(w, 16) || !al(nw, 16) || !al(out, 8)) return false;
 #define NGA_STEP(TPR, NV)                                                                                              \
   residual_step_bf16x4_kernel<TPR, NV, POST><<<dim3((unsigned)(TPR == 64 ? (T + 3) / 4 : T)), 256, 0, stream>>>(        \
-      x, y, y_stride, w, nw, eps, H, T, out)
+      x, y, y_stride, w, nw, eps, H, T, out, inv, k)
   if (T >= 4096 && H <= 4096) {      // rows enough to fill the chip with one wave each
     if (H <= 256) NGA_STEP(64, 1);
     else if (H <= 512) NGA_STEP(64, 2);
@@ -741,7 +771,7 @@ void launch_rmsnorm_residual_next(float* x, const void* y, int64_t y_stride, con
                                   int nw_n, float eps, int64_t T, int H, void* out, bool f32, hipStream_t stream) {
   if (T == 0) return;
   if (!f32 && w_n == H && nw_n == H &&
-      launch_residual_step_vec<true>(x, (const uint16_t*)y, y_stride, w, nw, eps, T, H, (uint16_t*)out, stream))
+      launch_residual_step_vec<true>(x, (const uint16_t*)y, y_stride, w, nw, eps, T, H, (uint16_t*)out, nullptr, 0, stream))
     return;
   const int ws = w_n == 1 ? 0 : 1, nws = nw_n == 1 ? 0 : 1;
   if (f32)
@@ -776,16 +806,17 @@ void launch_softcap(float* z, int64_t n, float cap, float scale, hipStream_t str
 }
 
 void launch_residual_add_rmsnorm(float* x, const void* y, int64_t y_stride, const float* w, float eps, int64_t T, int H,
-                                 void* out, bool f32, hipStream_t stream) {
+                                 void* out, const int32_t* inv, int k, bool f32, hipStream_t stream) {
   if (T == 0) return;
-  if (!f32 && launch_residual_step_vec<false>(x, (const uint16_t*)y, y_stride, nullptr, w, eps, T, H, (uint16_t*)out, stream))
+  if (!f32 && launch_residual_step_vec<false>(x, (const uint16_t*)y, y_stride, nullptr, w, eps, T, H, (uint16_t*)out, inv, k,
+                                              stream))
     return;
   if (f32)
     residual_add_rmsnorm_kernel<float><<<dim3((unsigned)T), 256, 0, stream>>>(x, (const float*)y, y_stride, w, eps, H,
-                                                                             (float*)out);
+                                                                             (float*)out, inv, k);
   else
     residual_add_rmsnorm_kernel<uint16_t><<<dim3((unsigned)T), 256, 0, stream>>>(x, (const uint16_t*)y, y_stride, w, eps,
-                                                                                H, (uint16_t*)out);
+                                                                                H, (uint16_t*)out, inv, k);
 }
 
 void launch_clamped_glu(void* out, const void* in, int64_t in_stride, int64_t T, int F, float limit, float alpha,

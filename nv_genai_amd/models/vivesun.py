@@ -7,7 +7,7 @@ around zero and applied as ``1 + w``):
 
     h  = norm1(x)                                    fused into the previous layer's last step
     x += mixer(h); h2 = norm2(x)                     ops.residual_add_rmsnorm_
-    x += experts(h2), copy of x for the gate         ops.residual_add_cast_
+    x += experts(h2), copy of x for the gate         ops.moe_router, ops.residual_plain_experts_
     g  = gelu_tanh(gate x) * token vector of layer i ops.gelu_gate_rows
     x += rmsnorm(proj g) * w; h = next norm1(x)      ops.rmsnorm_residual_next_
 
@@ -323,12 +323,6 @@ class VivesunModel:
         ops.group_rmsnorm(o, L["on_scaled"], r.heads, self.cfg.eps, self.dtype, gate=proj[:, c[3]:c[4]], out=y[:, nl:])
         return self._lin(y, L["wo"])
 
-    def _ff(self, L: dict, h):
-        f = L["mlp"]
-        logits = ops.linear(h if h.dtype == torch.float32 else h.float(), L["router"])
-        ids, wts = ops.moe_route_grouped(logits, None, f.top, 1, 1, f.scale, ws=self.moe_ws)
-        return ops.moe_plain_experts(h, ids, wts, L["w1"], L["wd"], ws=self.moe_ws)
-
     def _embed(self, ids, meta: AttnMeta):
         g = self.cfg.bigram
         if g is None:
@@ -354,18 +348,22 @@ class VivesunModel:
         h = ops.rmsnorm_f32(x, self.layers[0]["norm1"], eps, dtype=dt) if self.layers else None
         for li, L in enumerate(self.layers):
             y = (self._mix_delta if L["type"] == "delta" else self._mix_parallel)(li, L, h, pos, meta)
-            if L["mlp"] is not None:
-                y = self._ff(L, ops.residual_add_rmsnorm_(x, y, L["norm2"], eps, dt))
             nxt = self.layers[li + 1]["norm1"] if li + 1 < len(self.layers) else None
-            if S:
-                z = self._lin(ops.residual_add_cast_(x, y, dt), L["sg"])
-                y = self._lin(ops.gelu_gate_rows(z, ids, self.side_embed, li * S), L["sp"])
+            f = L["mlp"]
+            if f is not None:
+                h2 = ops.residual_add_rmsnorm_(x, y, L["norm2"], eps, dt)
+                eid, ew = ops.moe_router(h2, L["router"], f.top, f.scale, ws=self.moe_ws)
+                h = ops.residual_plain_experts_(x, h2, eid, ew, L["w1"], L["wd"], nxt, eps, dt, copy=S > 0, ws=self.moe_ws)
+            elif S:
+                h = ops.residual_add_cast_(x, y, dt)
+            else:
+                h = ops.residual_add_rmsnorm_(x, y, nxt, eps, dt)
+            if S:      # h is a copy of the stream
+                y = self._lin(ops.gelu_gate_rows(self._lin(h, L["sg"]), ids, self.side_embed, li * S), L["sp"])
                 if nxt is not None:
                     h = ops.rmsnorm_residual_next_(x, y, L["sn"], eps, nxt, dt)
                 else:
                     ops.rmsnorm_residual_(x, y, L["sn"], eps)
-            else:
-                h = ops.residual_add_rmsnorm_(x, y, nxt, eps, dt)
             if layer_tap is not None:
                 layer_tap.append(x.clone())
         return ops.rmsnorm_f32(x, self.final_norm, eps, rows=sample_idx, dtype=dt)

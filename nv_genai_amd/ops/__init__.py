@@ -657,7 +657,7 @@ def residual_add_rmsnorm_(x: torch.Tensor, y: torch.Tensor, w: Optional[torch.Te
     if not _gpu(x):
         ref.residual_add_rmsnorm_(x, y, w, eps, out)
         return out
-    kernels().residual_add_rmsnorm(x, y, w, float(eps), out)
+    kernels().residual_add_rmsnorm(x, y, w, float(eps), out, None, 0)
     return out
 
 
@@ -904,7 +904,7 @@ def residual_add_cast_(x: torch.Tensor, y: torch.Tensor, dtype: torch.dtype) -> 
     out = torch.empty(x.shape, dtype=dtype, device=x.device)
     if not _gpu(x):
         return ref.residual_add_cast_(x, y, out)
-    kernels().residual_add_rmsnorm(x, y, None, 0.0, out)
+    kernels().residual_add_rmsnorm(x, y, None, 0.0, out, None, 0)
     return out
 
 
@@ -1404,22 +1404,34 @@ def moe_plain_mfma_ok(x: torch.Tensor, F: int) -> bool:
     return _gpu(x) and x.dtype == torch.bfloat16 and x.shape[1] % 256 == 0 and F % 64 == 0
 
 
-def moe_plain_experts(x: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor,
-                      ws: Optional["MoEWorkspace"] = None) -> torch.Tensor:
-    """Routed experts without a gate on rows x [T, H] -> [T, H]: the sum over a row's experts (``ids`` / ``wts``
-    [T, k]) of ``weight * down_e(gelu(up_e x))`` (erf gelu). ``w1`` [E, F, H], ``w2`` [E, H, F]. GPU: the
-    order of :func:`moe_glu_experts` (align, gathered up GEMM with the activation in its epilogue, down
-    GEMM times the weight, combine), on MFMA tiles where the sizes fit (:func:`moe_plain_mfma_ok`),
-    else on fp32-accumulating VALU tiles."""
-    if not _gpu(x):
-        return ref.moe_plain_experts(x, ids, wts, w1, w2)
+ROUTER_ROWS = 512     # rows up to which the router runs as one launch (beyond, the library GEMM wins)
+
+
+def moe_router(x: torch.Tensor, router: torch.Tensor, k: int, scale: float = 1.0,
+               ws: Optional["MoEWorkspace"] = None) -> Tuple[torch.Tensor, torch.Tensor]:
+    """Softmax router on rows x [T, H]: logits ``x . router^T`` in fp32 (router fp32 [E, H]), scores = softmax over
+    all E, the ``k`` largest (ties: the lower index) with weights ``score / (sum of the chosen + 1e-20) * scale``.
+    ids int32 [T, k], weights fp32 [T, k]. GPU: up to ``ROUTER_ROWS`` rows one launch, beyond a library GEMM on
+    the fp32 copy of the rows and :func:`moe_route_grouped`."""
+    T, H = x.shape
+    E = router.shape[0]
+    if not _gpu(x) or T > ROUTER_ROWS or H > 8192 or E > 512 or k > 64:
+        return moe_route_grouped(linear(x if x.dtype == torch.float32 else x.float(), router), None, k, 1, 1, scale, ws=ws)
+    if ws is not None and ws.rows * ws.k >= T * k:
+        ids, w = ws.ids[:T * k].view(T, k), ws.w[:T * k].view(T, k)
+    else:
+        ids = torch.empty(T, k, dtype=torch.int32, device=x.device)
+        w = torch.empty(T, k, dtype=torch.float32, device=x.device)
+    kernels().moe_router_rows(x, router, int(k), float(scale), ids, w)
+    return ids, w
+
+
+def _plain_expert_rows(x, ids, wts, w1, w2, ws):
+    """(weighted expert rows [T * k, H] sorted by expert, their row numbers per token)."""
     C = kernels()
     T, H = x.shape
     E, F, _ = w1.shape
     k = ids.shape[1]
-    out = torch.empty(T, H, dtype=x.dtype, device=x.device)
-    if T == 0:
-        return out
     M = T * k
     if ws is None:
         ws = MoEWorkspace.get(T, k, E, x.device)
@@ -1438,7 +1450,38 @@ def moe_plain_experts(x: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w1:
     else:
         C.moe_gemm_rows(x, w1, ws.sorted_tok, ws.sorted_w, ws.tiles, mt, h, 2, 0.0, 0.0, False, 0.0)
         C.moe_gemm_rows(h, w2, ws.sorted_tok, ws.sorted_w, ws.tiles, mt, y, 1, 0.0, 0.0, True, 0.0)
-    C.moe_combine_rows(y, ws.inv, T, int(k), None, out, None, None, None, E)
+    return y, ws.inv
+
+
+def moe_plain_experts(x: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor,
+                      ws: Optional["MoEWorkspace"] = None) -> torch.Tensor:
+    """Routed experts without a gate on rows x [T, H] -> [T, H]: the sum over a row's experts (``ids`` / ``wts``
+    [T, k]) of ``weight * down_e(gelu(up_e x))`` (erf gelu). ``w1`` [E, F, H], ``w2`` [E, H, F]. GPU: the
+    order of :func:`moe_glu_experts` (align, gathered up GEMM with the activation in its epilogue, down
+    GEMM times the weight, combine), on MFMA tiles where the sizes fit (:func:`moe_plain_mfma_ok`),
+    else on fp32-accumulating VALU tiles."""
+    if not _gpu(x):
+        return ref.moe_plain_experts(x, ids, wts, w1, w2)
+    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    if x.shape[0]:
+        y, inv = _plain_expert_rows(x, ids, wts, w1, w2, ws)
+        kernels().moe_combine_rows(y, inv, x.shape[0], int(ids.shape[1]), None, out, None, None, None, w1.shape[0])
+    return out
+
+
+def residual_plain_experts_(x: torch.Tensor, h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w1: torch.Tensor,
+                            w2: torch.Tensor, norm_w: Optional[torch.Tensor], eps: float, dtype: torch.dtype,
+                            copy: bool = False, ws: Optional["MoEWorkspace"] = None) -> Optional[torch.Tensor]:
+    """``x += moe_plain_experts(h)`` on an fp32 stream in place, a token's expert rows summed straight into it
+    (fp32) by the launch that also returns ``rmsnorm(x) * norm_w`` in ``dtype``, or, with ``copy``, a copy of the
+    sum; neither: None."""
+    if not _gpu(x):
+        y = ref.moe_plain_experts(h, ids, wts, w1, w2)
+        return residual_add_cast_(x, y, dtype) if copy else residual_add_rmsnorm_(x, y, norm_w, eps, dtype)
+    out = torch.empty(x.shape, dtype=dtype, device=x.device) if copy or norm_w is not None else None
+    if x.shape[0]:
+        y, inv = _plain_expert_rows(h, ids, wts, w1, w2, ws)
+        kernels().residual_add_rmsnorm(x, y, None if copy else norm_w, float(eps), out, inv, int(ids.shape[1]))
     return out
 
 

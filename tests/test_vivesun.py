@@ -555,6 +555,25 @@ def test_routing_without_correction(device):
 
 
 @pytest.mark.parametrize("device,dtype", DTYPES)
+def test_router_of_few_and_many_rows(device, dtype):
+    """The router product with the choice behind it: few rows (one launch) and more than that form takes,
+    widths that are no multiple of 4, tied experts (equal router rows: the lower index), all chosen."""
+    tdt = tdtype(dtype)
+    g = torch.Generator().manual_seed(8)
+    for (T, H, E, k, scale) in ((7, 40, 5, 3, 1.7), (64, 1024, 32, 4, 2.0), (3, 33, 70, 9, 1.0), (5, 16, 1, 1, 3.0), (700, 64, 8, 2, 1.0),
+                                (9, 24, 6, 6, 0.5), (4, 256, 512, 8, 1.0)):
+        x = torch.randn(T, H, generator=g).to(tdt)
+        r = torch.randn(E, H, generator=g) * (3.0 / H ** 0.5)
+        if E == 5:
+            r[3], r[4] = r[1], r[1]
+        want = O.route(x.double() @ r.double().T, {"top": k, "scale": scale})
+        ids, wts = ops.moe_router(x.to(device), r.to(device), k, scale)
+        for t in range(T):
+            assert ids[t].tolist() == [e for e, _ in want[t]], f"{T} x {H}, {E} experts, row {t}"
+            close(wts[t], torch.tensor([w for _, w in want[t]]), "float32", "weights")
+
+
+@pytest.mark.parametrize("device,dtype", DTYPES)
 def test_gelu_experts(device, dtype):
     """Small experts on the tiled form; sizes the MFMA form takes (a partial last block of features,
     more than one block, more rows than one tile)."""
@@ -571,6 +590,17 @@ def test_gelu_experts(device, dtype):
             for e, s in zip(ids[t].tolist(), wts[t].tolist()):
                 want[t] += s * (O.gelu_erf(x[t].double() @ w1[e].double().T) @ w2[e].double().T)
         close(got, want, dtype, f"experts {E}, top {k}, ff {F}")
+        x0, nw = torch.randn(T, H, generator=g), 1 + 0.1 * torch.randn(H, generator=g)
+        args = (x.to(device), ids, wts, w1.to(device), w2.to(device))
+        for mode in ("norm", "copy", "sum"):       # summed straight into the stream
+            xs = x0.clone().to(device)
+            out = ops.residual_plain_experts_(xs, *args, nw.to(device) if mode == "norm" else None, 1e-5, tdt, copy=mode == "copy")
+            xw = x0.double() + want
+            close(xs, xw, dtype, "stream")
+            if mode == "sum":
+                assert out is None
+            else:
+                close(out, xw if mode == "copy" else O.unit_rms(xw, 1e-5) * nw.double(), dtype, mode)
 
 
 # ---------------------------------------------------------------------------- the model on the engine
