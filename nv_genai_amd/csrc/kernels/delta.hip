@@ -215,8 +215,8 @@ __global__ void __launch_bounds__(256) delta_rows_kernel(const DeltaParams P) {
 // Block operands (see the head of the file). Workgroup = (block of a segment, head, segment).
 constexpr int ML = 20;    // row stride of the 16 x 16 matrices in LDS
 
-template <typename T, int MODE>
-__global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, float* __restrict__ ws, int DT) {
+template <typename T, int MODE, int DT>
+__global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, float* __restrict__ ws) {
   using F = GateFn<T>;
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ __attribute__((aligned(16))) float LA[16 * ML], LK[16 * ML], GA[16 * ML], GK[16 * ML], Tm[16 * ML];
@@ -227,7 +227,8 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, fl
   const int tc = t0 + blk * 16;
   if (tc >= t1) return;
   const int nrow = min(16, t1 - tc);
-  const int d = P.d, D = 16 * DT, DS = D + 4;
+  constexpr int D = 16 * DT, DS = D + 4;
+  const int d = P.d;
   // mode 0: rows K, Q; mode 1: rows C, R, alpha, kappa, running log decays, then P_16
   float* X0 = lds;
   float* X1 = lds + 16 * DS;
@@ -239,17 +240,28 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, fl
   const int t = tid >> 4, sub = tid & 15;
   const int64_t row = tc + t;
   const bool live = t < nrow;
+  // rows past the segment read its last row, channels past d the first one (no branch around a load, so
+  // that all of a thread's loads are in flight together), and count as zeros
+  const int64_t lrow = live ? row : t1 - 1;
   if (MODE == 0) {
     const int g = h / (P.H / P.G);
-    float sk = 0.f, sq = 0.f;
-    for (int i = sub; i < D; i += 16) {
-      const bool ok = live && i < d;
-      const float kv = ok ? ldf((const T*)P.k + row * P.ks + g * d + i) : 0.f;
-      const float qv = ok ? ldf((const T*)P.q + row * P.qs + g * d + i) : 0.f;
-      X0[t * DS + i] = kv;
-      X1[t * DS + i] = qv;
-      sk += kv * kv;
-      sq += qv * qv;
+    const T* kp = (const T*)P.k + lrow * P.ks + g * d;
+    const T* qp = (const T*)P.q + lrow * P.qs + g * d;
+    T kr[DT], qr[DT];
+#pragma unroll
+    for (int m = 0; m < DT; ++m) {
+      const int i = sub + 16 * m, ii = i < d ? i : 0;
+      kr[m] = kp[ii];
+      qr[m] = qp[ii];
+    }
+    float kf[DT], qf[DT], sk = 0.f, sq = 0.f;
+#pragma unroll
+    for (int m = 0; m < DT; ++m) {
+      const bool ok = live && sub + 16 * m < d;
+      kf[m] = ok ? ldf(&kr[m]) : 0.f;
+      qf[m] = ok ? ldf(&qr[m]) : 0.f;
+      sk += kf[m] * kf[m];
+      sq += qf[m] * qf[m];
     }
 #pragma unroll
     for (int o = 8; o > 0; o >>= 1) {
@@ -257,9 +269,10 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, fl
       sq += __shfl_xor(sq, o, 64);
     }
     const float ik = 1.0f / sqrtf(sk + 1e-6f), iq = 1.0f / sqrtf(sq + 1e-6f) / sqrtf((float)d);
-    for (int i = sub; i < D; i += 16) {   // the elements this thread wrote
-      X0[t * DS + i] *= ik;
-      X1[t * DS + i] *= iq;
+#pragma unroll
+    for (int m = 0; m < DT; ++m) {
+      X0[t * DS + sub + 16 * m] = kf[m] * ik;
+      X1[t * DS + sub + 16 * m] = qf[m] * iq;
     }
     if (tid < 16) {      // running log decay and step size of the block's rows, one row per lane
       const int64_t r2 = tc + tid;
@@ -278,15 +291,32 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, fl
     }
     __syncthreads();
   } else {
-    float sk = 0.f;
-    for (int i = sub; i < D; i += 16) {
+    const T* kp = (const T*)P.k + lrow * P.ks + h * d;
+    const T* qp = (const T*)P.q + lrow * P.qs + h * d;
+    const T* bp = (const T*)P.b + lrow * P.bs + h * d;
+    const T* wq = (const T*)P.w + lrow * P.ws + h * d;
+    T kr[DT], qr[DT], br[DT], wr[DT];
+    float bb[DT], wb[DT];
+#pragma unroll
+    for (int m = 0; m < DT; ++m) {
+      const int i = sub + 16 * m, ii = i < d ? i : 0;
+      kr[m] = kp[ii];
+      qr[m] = qp[ii];
+      br[m] = bp[ii];
+      wr[m] = wq[ii];
+      bb[m] = P.b_vec[h * d + ii];
+      wb[m] = P.w_vec[h * d + ii];
+    }
+    float kf[DT], sk = 0.f;
+#pragma unroll
+    for (int m = 0; m < DT; ++m) {
+      const int i = sub + 16 * m;
       const bool ok = live && i < d;
-      const float kv = ok ? ldf((const T*)P.k + row * P.ks + h * d + i) : 0.f;
-      X3[t * DS + i] = kv;
-      X1[t * DS + i] = ok ? ldf((const T*)P.q + row * P.qs + h * d + i) : 0.f;
-      X2[t * DS + i] = ok ? F::sigmoid(ldf((const T*)P.b + row * P.bs + h * d + i) + P.b_vec[h * d + i]) : 0.f;
-      X4[t * DS + i] = ok ? -P.decay * F::sigmoid(ldf((const T*)P.w + row * P.ws + h * d + i) + P.w_vec[h * d + i]) : 0.f;
-      sk += kv * kv;
+      kf[m] = ok ? ldf(&kr[m]) : 0.f;
+      sk += kf[m] * kf[m];
+      X1[t * DS + i] = ok ? ldf(&qr[m]) : 0.f;
+      X2[t * DS + i] = ok ? F::sigmoid(ldf(&br[m]) + bb[m]) : 0.f;
+      X4[t * DS + i] = ok ? -P.decay * F::sigmoid(ldf(&wr[m]) + wb[m]) : 0.f;
     }
 #pragma unroll
     for (int o = 8; o > 0; o >>= 1) sk += __shfl_xor(sk, o, 64);
@@ -304,9 +334,11 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, fl
       pc[tid] = F::exp(l[15]);
     }
     __syncthreads();
-    for (int i = sub; i < D; i += 16) {
+#pragma unroll
+    for (int m = 0; m < DT; ++m) {
+      const int i = sub + 16 * m;
       const float c1 = X4[t * DS + i], c0 = t > 0 ? X4[(t - 1) * DS + i] : 0.f;
-      const float kv = X3[t * DS + i], u = kv * ik, down = F::exp(-c1);
+      const float kv = kf[m], u = kv * ik, down = F::exp(-c1);
       X0[t * DS + i] = u * F::exp(c0);
       X1[t * DS + i] *= F::exp(c1);
       X2[t * DS + i] *= -u * down;
@@ -320,6 +352,7 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaParams P, fl
     const float* Ar = MODE == 0 ? (wv == 0 ? X0 : X1) : (wv < 2 ? X0 : X1);
     const float* Br = MODE == 0 ? X0 : ((wv & 1) ? X3 : X2);
     f32x4 acc0 = (f32x4)(0.f), acc1 = (f32x4)(0.f);
+#pragma unroll
     for (int i = 0; i < DT; ++i) {
       const f32x4 av = *reinterpret_cast<const f32x4*>(Ar + l15 * DS + 16 * i + 4 * hh);
       const f32x4 bv = *reinterpret_cast<const f32x4*>(Br + l15 * DS + 16 * i + 4 * hh);
@@ -501,6 +534,15 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1)))
     for (int r = 0; r < 4; ++r)
 #pragma unroll
       for (int i = 0; i < DT; ++i) S[i] = mfma32(B.a[i][r], y[r], S[i]);
+    if constexpr (DT <= 8) {
+      // the next block's loads (issued in front of this step in program order) between the MFMAs: a
+      // wave issues in order, and loads in a row would leave the matrix pipe idle
+#pragma unroll
+      for (int g = 0; g < 5 * DT + 5; ++g) {
+        __builtin_amdgcn_sched_group_barrier(0x008, 2, 0);   // MFMA
+        __builtin_amdgcn_sched_group_barrier(0x020, 1, 0);   // VMEM read
+      }
+    }
     float* op = P.out + (int64_t)(t0 + blk * 16) * P.H * dv + h * dv + col;
     if (blk * 16 + 16 <= t1 - t0) {
       if (colok) {
@@ -521,7 +563,7 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1)))
     for (; blk + 1 < nblk; blk += 2) {
       load(B, blk + 1);
       step(A, blk);
-      if (blk + 2 < nblk) load(A, blk + 2);
+      load(A, min(blk + 2, nblk - 1));
       step(B, blk + 1);
     }
     if (blk < nblk) step(A, blk);
@@ -580,18 +622,28 @@ bool launch_walk_t(const DeltaParams& P, const float* ws, int dt, int n_seg, hip
   }
 }
 
-template <typename T, int MODE>
-void launch_prep_t(const DeltaParams& P, float* ws, int dt, int n_seg, int max_q, hipStream_t stream) {
-  const int D = 16 * dt;
-  const size_t smem = (size_t)((MODE == 0 ? 32 : 80) * (D + 4) + (MODE == 0 ? 0 : D)) * sizeof(float);
+template <typename T, int MODE, int DT>
+void launch_prep_dt(const DeltaParams& P, float* ws, dim3 grid, hipStream_t stream) {
+  constexpr int D = 16 * DT;
+  constexpr size_t smem = (size_t)((MODE == 0 ? 32 : 80) * (D + 4) + (MODE == 0 ? 0 : D)) * sizeof(float);
   static bool attr_set = false;
-  if (smem > 49152 && !attr_set) {     // (with the static part above the default limit: the attribute once, for the largest size)
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_prep_kernel<T, MODE>),
-                              hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 260 * 4 + 256 * 4);
+  if (smem > 49152 && !attr_set) {     // (with the static part above the default limit: the attribute once)
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_prep_kernel<T, MODE, DT>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
     attr_set = true;
   }
+  delta_prep_kernel<T, MODE, DT><<<grid, 256, smem, stream>>>(P, ws);
+}
+
+template <typename T, int MODE>
+void launch_prep_t(const DeltaParams& P, float* ws, int dt, int n_seg, int max_q, hipStream_t stream) {
   const dim3 grid((unsigned)((max_q + 15) / 16), (unsigned)P.H, (unsigned)n_seg);
-  delta_prep_kernel<T, MODE><<<grid, 256, smem, stream>>>(P, ws, dt);
+  switch (dt) {
+#define NGA_PREP(N) case N: launch_prep_dt<T, MODE, N>(P, ws, grid, stream); return;
+    NGA_PREP(1) NGA_PREP(2) NGA_PREP(3) NGA_PREP(4) NGA_PREP(6) NGA_PREP(8) NGA_PREP(12) NGA_PREP(16)
+#undef NGA_PREP
+    default: return;      // (the walk's launch reports a size that is not compiled)
+  }
 }
 
 }  // namespace
