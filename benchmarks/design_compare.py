@@ -42,7 +42,7 @@ LIZEZEN_MLSTM = dict(dim=64, vdim=128)
 # the window of the other designs, a rotation on half the head) beside 64-wide channel-decay delta
 # heads over the whole width, expert sizes of LUMEPEL, a bigram table and a token input
 VIVESUN_PATTERN = ("delta", "parallel")
-VIVESUN = dict(dim=128, vdim=128, conv=4, rdim=64, rank=64, rot=64, side=256, bigram=(65521, 31, 17))
+VIVESUN = dict(dim=128, vdim=128, conv=4, rdim=64, rank=64, rot=64, side=256, bigram=(65521, 40503, 9973))
 BASELINE_OF = {"bidasun": "mistral", "biruvik": "mistral", "lumepel": "mixtral", "lizezen": "mixtral", "vivesun": "mixtral"}
 
 
@@ -58,7 +58,7 @@ def _engine(kind: str, z: dict, max_len: int, pages: int, seqs: int):
                               delta_heads=z["heads"], delta_kv_heads=z["heads"] // 2, delta_dim=v["dim"],
                               delta_vdim=v["vdim"], conv=v["conv"], right_heads=z["hidden"] // v["rdim"],
                               right_dim=v["rdim"], decay_rank=v["rank"], experts=u["experts"], top=u["top"],
-                              expert_ff=u["eff"], route_scale=2.0, rot_base=5e5, rot_dims=v["rot"],
+                              expert_ff=u["eff"], route_scale=2.0, rot_base=1e6, rot_dims=v["rot"],
                               bands=(8.0, 1.0, 4.0, 8192), bigram=v["bigram"], side_dim=v["side"], vocab_size=VOCAB)
     elif kind == "lizezen":
         u = z["lumepel"]
@@ -665,7 +665,7 @@ def vivesun_kernel_times(z: dict, iters: int = 20) -> dict:
     # ---- row kernels (prompt rows): bytes that must move over the time, against 8 TB/s
     qkv = torch.randn(T, (H + 2 * G) * D, device=dev).to(bf)
     slots = torch.arange(T, dtype=torch.int32, device=dev)
-    freq, mag = ops.rotary_frequencies(v["rot"], 5e5, bands=(8.0, 1.0, 4.0, 8192))
+    freq, mag = ops.rotary_frequencies(v["rot"], 1e6, bands=(8.0, 1.0, 4.0, 8192))
     freq = freq.to(dev)
     t_rh = _timed_gpu(lambda: ops.rope_headnorm_cache_(qkv, posr, slots, kr, vr, H, G, D, D, freq, mag, v["rot"], 1e-5,
                                                    v_off=(H + G) * D), iters)
@@ -694,7 +694,7 @@ def vivesun_kernel_times(z: dict, iters: int = 20) -> dict:
         # name: (call, bytes)
         "rope_partial_cache": (t_rh, by_rh), "rope_cache": (t_rk, by_rk),
         "short_conv": (t_cp, T * C * 4.0),
-        "bigram_embed": (lambda: ops.bigram_embed(ids, emb, bg, src, prev, 31, 17), T * Hd * 8.0),   # two bf16 in, fp32 out
+        "bigram_embed": (lambda: ops.bigram_embed(ids, emb, bg, src, prev, *v["bigram"][1:]), T * Hd * 8.0),   # two bf16 in, fp32 out
         "embed_rows": (lambda: ops.embed_rows(ids, emb), T * Hd * 6.0),
         "residual_add_rmsnorm": (lambda: ops.residual_add_rmsnorm_(xs, y1, wn, 1e-5, bf), T * Hd * 12.0),
         "residual_add_cast": (lambda: ops.residual_add_cast_(xs, y1, bf), T * Hd * 12.0),

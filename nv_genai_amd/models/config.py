@@ -1274,7 +1274,7 @@ def vivesun_layers(pattern: Sequence[str], hidden: int, heads: int, kv_heads: in
                    delta_heads: int = 0, delta_kv_heads: int = 0, delta_dim: int = 0, delta_vdim: int = 0, conv: int = 4,
                    right_heads: int = 0, right_dim: int = 0, decay_rank: int = 64, left_scale: float = 1.0,
                    right_scale: float = 1.0, experts: int = 0, top: int = 2, expert_ff: int = 0, route_scale: float = 1.0,
-                   rot_base: float = 500000.0, rot_dims: int = 0, bands: Optional[tuple] = None,
+                   rot_base: float = 10000.0, rot_dims: int = 0, bands: Optional[tuple] = None,
                    bigram: Optional[tuple] = None, side_dim: int = 0, vocab_size: int = 32768, eps: float = 1e-6,
                    name: str = "vivesun") -> VivesunConfig:
     """A Vivesun config from a pattern of mixer types with the same sizes in every layer of a kind

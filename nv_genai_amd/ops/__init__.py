@@ -539,8 +539,9 @@ def headnorm_cache_(proj, slots, kc, vc, nq: int, nk: int, dk: int, nv: int, dv:
     return proj
 
 
-def _out_factor(unit_eps: Optional[float], out_scale: float, factor: float) -> float:
-    return float(factor) * (1.0 if unit_eps is None else float(out_scale))
+def _unit_args(unit_eps: Optional[float], out_scale: float, factor: float) -> Tuple[float, float]:
+    """(eps of the unit RMS or -1, factor on the outputs) as the attention kernels take them."""
+    return (-1.0, float(factor)) if unit_eps is None else (float(unit_eps), float(factor) * float(out_scale))
 
 
 def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk: int, dv: int, scale: float,
@@ -554,7 +555,8 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk:
     ``(h // (H / G)) * maps + m``, both maps read v head ``h // (H / G)``; two maps combine as
     ``a_0 - lam * a_1`` (differential attention). ``unit_eps``: divide every head's output by its
     root mean square (eps inside the root) and multiply by ``out_scale``. ``gate`` [T, H]: the
-    head outputs are multiplied by ``sigmoid(gate)``. ``factor``: the outputs are multiplied by it. ``tok_seq[t]`` is the block-table row of
+    head outputs are multiplied by ``sigmoid(gate)``. ``factor``: the outputs are multiplied by it.
+    ``tok_seq[t]`` is the block-table row of
     token t, ``pos[t]`` its position (negative: padding row, zeros out). Scores, softmax and
     accumulation are fp32. ``v_in_k`` (one map, dv <= dk): the values are the first dv elements of
     the key rows (``vc`` is not read) - keys with extra key-only columns behind a shared latent.
@@ -572,7 +574,7 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk:
         out = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
     kernels().softmax_attention(out, q, gate, kc, kc if v_in_k else vc, block_tables, tok_seq, pos, H, G, dk, dv,
                                 float(scale), int(window), int(maps), float(lam),
-                                -1.0 if unit_eps is None else float(unit_eps), _out_factor(unit_eps, out_scale, factor), bool(v_in_k),
+                                *_unit_args(unit_eps, out_scale, factor), bool(v_in_k),
                                 float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 
@@ -613,7 +615,7 @@ def softmax_attention_prefill(q, kc, vc, block_tables, cu_q, ctx_lens, max_q_len
         out = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
     kernels().softmax_attention_prefill(out, q, gate, kc, kc if v_in_k else vc, block_tables, cu_q, ctx_lens,
                                         int(max_q_len), H, G, dk, dv, float(scale), int(window), int(maps), float(lam),
-                                        -1.0 if unit_eps is None else float(unit_eps), _out_factor(unit_eps, out_scale, factor), bool(v_in_k),
+                                        *_unit_args(unit_eps, out_scale, factor), bool(v_in_k),
                                         float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 
@@ -642,7 +644,7 @@ def softmax_attention_rows(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int
         out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
     C.softmax_attention_decode(out, ws, parts, q, gate, kc, kc if v_in_k else vc, block_tables, tok_seq, pos, H, G, dk,
                                dv, float(scale), int(window), int(maps), float(lam),
-                               -1.0 if unit_eps is None else float(unit_eps), _out_factor(unit_eps, out_scale, factor), bool(v_in_k),
+                               *_unit_args(unit_eps, out_scale, factor), bool(v_in_k),
                                float(softcap), int(chunk), -math.inf if sink is None else float(sink))
     return out
 
