@@ -564,13 +564,15 @@ class RotarySpec:
     frequencies of slow pairs are divided by ``factor`` along a linear ramp over the pair index,
     and cos / sin are multiplied by ``0.1 ln(factor) + 1``. ``bands`` = (factor, low, high, original)
     or None: the frequencies are divided by ``factor`` along a ramp over the wavelength, from
-    ``original / high`` to ``original / low`` (:func:`ops.rotary_frequencies`)."""
+    ``original / high`` to ``original / low`` (:func:`ops.rotary_frequencies`). ``linear``: every
+    frequency is divided by it."""
 
     dims: int
     base: float
     interleaved: bool = False
     yarn: Optional[tuple] = None
     bands: Optional[tuple] = None
+    linear: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -1294,3 +1296,262 @@ def vivesun_layers(pattern: Sequence[str], hidden: int, heads: int, kv_heads: in
         blocks.append(VivesunLayer(t, m, PlainMoeSpec(experts, top, expert_ff, route_scale) if experts else None))
     return VivesunConfig(name=name, vocab_size=vocab_size, hidden=hidden, eps=eps, blocks=tuple(blocks),
                          bigram=None if not bigram else BigramSpec(*bigram), side_dim=side_dim)
+
+
+# ---------------------------------------------------------------------------------------------
+# Kevelorn: pre-norm layers with scaled sub-layer outputs and a repeated span of layers; linear
+# recurrences with a diagonal decay, one of them side by side with windowed attention.
+@dataclass(frozen=True)
+class WindowAttentionSpec:
+    """Softmax attention with GQA over the last ``window`` positions (the query's own included; 0: all
+    earlier ones): rotary positions, then unit RMS of every q and k head, ``scale`` on the scores, a
+    sigmoid gate per output element."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot: RotarySpec
+    window: int = 0
+
+
+@dataclass(frozen=True)
+class LightningSpec:
+    """Mixer ``lightning``: a matrix memory per head with one constant decay, ``S <- decay S + k v^T``,
+    ``o = S^T q``, silu on q, k and v; one RMS norm over all heads together, a sigmoid gate."""
+
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+
+
+@dataclass(frozen=True)
+class GlaSpec:
+    """Mixer ``gla``: a matrix memory per head with a decay per key channel and token,
+    ``S <- diag(sigmoid(z)^(1 / tau)) S + k v^T``, ``o = S^T q``, ``q`` scaled by ``dim^(-1/2)``, z from a low-
+    rank projection (``rank`` 0: as the checkpoint's tensors have it); RMS norm per head, a silu gate."""
+
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    rank: int = 0
+
+
+@dataclass(frozen=True)
+class NormedHalvesSpec:
+    """Mixer ``parallel``: half the sum of two mixers' outputs on one input, each brought to unit RMS
+    over the model width and weighted."""
+
+    left: WindowAttentionSpec
+    right: LightningSpec
+
+
+@dataclass(frozen=True)
+class SharedMoeSpec:
+    """``experts`` SwiGLU experts of ``ff`` features of which a token uses the ``top`` with the largest router
+    logit, weighted by the softmax over those; ``shared`` (features, 0: none): an expert every token
+    uses, times ``sigmoid(sg . x)``."""
+
+    experts: int
+    top: int
+    ff: int
+    shared: int = 0
+    kind: str = "moe"
+
+
+@dataclass(frozen=True)
+class KevelornLayer:
+    type: str                 # "parallel" | "lightning" | "gla"
+    mixer: object
+    mlp: object = None        # DenseMlpSpec | SharedMoeSpec | None
+
+
+_KEVELORN_MIXERS = ("parallel", "lightning", "gla")
+
+
+@dataclass(frozen=True)
+class KevelornConfig:
+    """Kevelorn: ``x += m mixer(norm1(x))``, ``x += m ff(norm2(x))`` on an fp32 stream (RMS norms with
+    weights stored around zero, ``m`` = ``residual_mult``); a span of layers runs ``loop.times`` times with
+    the same weights and caches of its own per pass, ``x += x0`` (x0 = the embedding rows; not in front of
+    the first pass) and ``x += step_t`` in front of pass t. Every size and every constant that can differ
+    between models comes from config.json (:meth:`from_dict`)."""
+
+    name: str = "kevelorn"
+    vocab_size: int = 512
+    hidden: int = 128
+    eps: float = 1e-6
+    residual_mult: float = 1.0
+    blocks: tuple = ()
+    loop: Optional[LoopSpec] = None
+    max_position: int = 1 << 20     # no position table: only the engine's bookkeeping is bounded
+    arch: str = "kevelorn"
+    bos_id: int = 0
+    eos_ids: tuple = ()
+    chat_format: str = "plain"
+
+    @property
+    def layers(self) -> int:
+        return len(self.blocks)
+
+    @property
+    def runs(self) -> tuple:
+        """The order the layers run in: ((layer index, t), ...), t = the number of the pass that begins
+        with this run, else None."""
+        n, lp = len(self.blocks), self.loop
+        if lp is None:
+            return tuple((i, None) for i in range(n))
+        out = [(i, None) for i in range(lp.start)]
+        for t in range(lp.times):
+            out += [(i, t if i == lp.start else None) for i in range(lp.start, lp.stop)]
+        return tuple(out + [(i, None) for i in range(lp.stop, n)])
+
+    @property
+    def is_moe(self) -> bool:
+        return any(isinstance(b.mlp, SharedMoeSpec) for b in self.blocks)
+
+    @property
+    def experts_per_tok(self) -> int:
+        """Largest top-k of any layer (sizes the engine's routing workspace)."""
+        return max([b.mlp.top for b in self.blocks if isinstance(b.mlp, SharedMoeSpec)] or [1])
+
+    @property
+    def num_experts(self) -> int:
+        return max([b.mlp.experts for b in self.blocks if isinstance(b.mlp, SharedMoeSpec)] or [0])
+
+    @staticmethod
+    def _attention(m: dict, what: str) -> WindowAttentionSpec:
+        dim, r = int(m["dim"]), m["rot"]
+        rot = RotarySpec(dims=int(r["dims"]), base=float(r["base"]), interleaved=True,
+                         linear=float((r.get("scaling") or {}).get("factor", 1.0)))
+        if rot.dims % 2 or not 0 < rot.dims <= dim or not rot.linear > 0:
+            raise ValueError(f"{what}: rot.dims must be even and at most dim, the scaling factor positive")
+        a = WindowAttentionSpec(heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=dim,
+                                vdim=int(m.get("vdim", dim)), scale=float(m["scale"]), rot=rot,
+                                window=int((m.get("mask") or {}).get("size") or 0))
+        if min(a.heads, a.kv_heads, a.dim, a.vdim) < 1 or a.heads % a.kv_heads or a.window < 0:
+            raise ValueError(f"{what}: heads must be a multiple of kv_heads and sizes positive")
+        return a
+
+    @staticmethod
+    def _lightning(m: dict, what: str) -> LightningSpec:
+        s = LightningSpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])),
+                          decay=tuple(float(v) for v in m["decay"]))
+        if min(s.heads, s.dim, s.vdim) < 1 or len(s.decay) != s.heads or not all(0.0 <= v <= 1.0 for v in s.decay):
+            raise ValueError(f"{what}: sizes must be positive, one decay in [0, 1] per head")
+        return s
+
+    @classmethod
+    def from_dict(cls, d: dict, name: str = "kevelorn") -> "KevelornConfig":
+        blocks = []
+        for i, b in enumerate(d["layers"]):
+            t, m, what = b["type"], b["mixer"], f"layer {i}"
+            if t == "parallel":
+                mixer = NormedHalvesSpec(cls._attention(m["left"], what), cls._lightning(m["right"], what))
+            elif t == "lightning":
+                mixer = cls._lightning(m, what)
+            elif t == "gla":
+                mixer = GlaSpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])),
+                                tau=float(m["tau"]), rank=int(m.get("rank") or 0))
+                if min(mixer.heads, mixer.dim, mixer.vdim) < 1 or not mixer.tau > 0:
+                    raise ValueError(f"{what}: sizes and tau must be positive")
+            else:
+                raise ValueError(f"{what}: unknown mixer type {t!r} (known: {_KEVELORN_MIXERS})")
+            mlp = b.get("mlp")
+            if mlp is not None:
+                kind = mlp.get("kind", "dense")
+                if kind == "dense":
+                    mlp = DenseMlpSpec(ff=int(mlp["ff"]))
+                elif kind == "moe":
+                    sh = mlp.get("shared")
+                    mlp = SharedMoeSpec(experts=int(mlp["router"]["experts"]), top=int(mlp["router"]["top"]),
+                                        ff=int(mlp["expert"]["ff"]), shared=int(sh["ff"]) if sh else 0)
+                    if not 1 <= mlp.top <= mlp.experts:
+                        raise ValueError(f"{what}: top {mlp.top} of {mlp.experts} experts")
+                else:
+                    raise ValueError(f"{what}: unknown feed-forward kind {kind!r}")
+                if mlp.ff < 1:
+                    raise ValueError(f"{what}: ff must be positive")
+            blocks.append(KevelornLayer(type=t, mixer=mixer, mlp=mlp))
+        lp, loop = d.get("loop"), None
+        if lp:
+            loop = LoopSpec(start=int(lp["start"]), stop=int(lp["stop"]), times=int(lp["times"]))
+            if not (0 <= loop.start < loop.stop <= len(blocks)) or loop.times < 1:
+                raise ValueError(f"loop {lp} does not fit {len(blocks)} layers")
+        return cls(name=name, vocab_size=int(d["vocab"]), hidden=int(d["width"]), eps=float(d["norm"]["eps"]),
+                   residual_mult=float(d.get("residual_mult", 1.0)), blocks=tuple(blocks), loop=loop)
+
+    def to_json_dict(self) -> dict:
+        """The config.json form (inverse of :meth:`from_dict`)."""
+
+        def lightning(s):
+            return {"heads": s.heads, "dim": s.dim, "vdim": s.vdim, "decay": list(s.decay)}
+
+        layers = []
+        for b in self.blocks:
+            m, f = b.mixer, b.mlp
+            if b.type == "parallel":
+                a = m.left
+                rot = {"base": a.rot.base, "dims": a.rot.dims}
+                if a.rot.linear != 1.0:
+                    rot["scaling"] = {"factor": a.rot.linear}
+                left = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim, "scale": a.scale, "rot": rot}
+                if a.window:
+                    left["mask"] = {"size": a.window}
+                mx = {"left": left, "right": lightning(m.right)}
+            elif b.type == "lightning":
+                mx = lightning(m)
+            else:
+                mx = {"heads": m.heads, "dim": m.dim, "vdim": m.vdim, "tau": m.tau}
+                if m.rank:
+                    mx["rank"] = m.rank
+            if isinstance(f, SharedMoeSpec):
+                ff = {"kind": "moe", "router": {"experts": f.experts, "top": f.top}, "expert": {"ff": f.ff}}
+                if f.shared:
+                    ff["shared"] = {"ff": f.shared}
+            else:
+                ff = None if f is None else {"kind": "dense", "ff": f.ff}
+            layers.append({"type": b.type, "mixer": mx, "mlp": ff})
+        out = {"architecture": "Kevelorn", "vocab": self.vocab_size, "width": self.hidden, "norm": {"eps": self.eps},
+               "residual_mult": self.residual_mult, "layers": layers}
+        if self.loop is not None:
+            out["loop"] = {"start": self.loop.start, "stop": self.loop.stop, "times": self.loop.times}
+        return out
+
+    def to_dict(self):
+        return asdict(self)
+
+
+def kevelorn_layers(pattern: Sequence[str], hidden: int, heads: int, kv_heads: int, dim: int, vdim: int, ff: int = 0,
+                    window: int = 0, rec_heads: int = 0, rec_dim: int = 0, rec_vdim: int = 0, tau: float = 16.0,
+                    rank: int = 0, experts: int = 0, top: int = 2, expert_ff: int = 0, shared_ff: int = 0,
+                    rot_base: float = 10000.0, rot_dims: int = 0, rot_factor: float = 1.0, residual_mult: float = 1.0,
+                    loop: Optional[tuple] = None, vocab_size: int = 32768, eps: float = 1e-6,
+                    name: str = "kevelorn") -> KevelornConfig:
+    """A Kevelorn config from a pattern of mixer types with the same sizes in every layer of a kind
+    (benchmarks, tests). ``experts`` > 0: mixtures in all layers but the ``parallel`` ones, which have dense
+    feed-forwards of ``ff`` (``ff`` 0: mixtures there too, or none). ``loop`` = (start, stop, times)."""
+    rh, rd, rv = rec_heads or heads, rec_dim or dim, rec_vdim or vdim
+    decay = tuple(1.0 - 2.0 ** (-1.0 - 7.0 * h / max(1, rh - 1)) for h in range(rh))
+    blocks = []
+    for t in pattern:
+        light = LightningSpec(rh, rd, rv, decay)
+        if t == "parallel":
+            rot = RotarySpec(rot_dims or dim, rot_base, interleaved=True, linear=rot_factor)
+            m = NormedHalvesSpec(WindowAttentionSpec(heads, kv_heads, dim, vdim, dim ** -0.5, rot, window), light)
+        elif t == "lightning":
+            m = light
+        elif t == "gla":
+            m = GlaSpec(rh, rd, rv, tau, rank)
+        else:
+            raise ValueError(f"unknown mixer type {t!r}")
+        if experts and (t != "parallel" or not ff):
+            mlp = SharedMoeSpec(experts, top, expert_ff, shared_ff)
+        else:
+            mlp = DenseMlpSpec(ff) if ff else None
+        blocks.append(KevelornLayer(t, m, mlp))
+    return KevelornConfig(name=name, vocab_size=vocab_size, hidden=hidden, eps=eps, residual_mult=residual_mult,
+                          blocks=tuple(blocks), loop=None if not loop else LoopSpec(*loop))

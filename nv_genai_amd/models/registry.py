@@ -14,7 +14,8 @@ from typing import Callable, Dict, Optional, Tuple
 
 import torch
 
-from .config import LLAMA_PRESETS, BidasunConfig, BiruvikConfig, LizezenConfig, LlamaConfig, LumepelConfig, VivesunConfig
+from .config import (LLAMA_PRESETS, BidasunConfig, BiruvikConfig, KevelornConfig, LizezenConfig, LlamaConfig, LumepelConfig,
+                     VivesunConfig)
 
 # design name (lower case) -> (config builder from the config.json dict, model class loader)
 _REGISTRY: Dict[str, Tuple[Callable[[dict], object], Callable[[], type]]] = {}
@@ -52,6 +53,12 @@ def _vivesun_class():
     from .vivesun import VivesunModel
 
     return VivesunModel
+
+
+def _kevelorn_class():
+    from .kevelorn import KevelornModel
+
+    return KevelornModel
 
 
 def _llama_class():
@@ -94,6 +101,7 @@ register("biruvik", BiruvikConfig.from_dict, _biruvik_class)
 register("lumepel", LumepelConfig.from_dict, _lumepel_class)
 register("lizezen", LizezenConfig.from_dict, _lizezen_class)
 register("vivesun", VivesunConfig.from_dict, _vivesun_class)
+register("kevelorn", KevelornConfig.from_dict, _kevelorn_class)
 for _t in _HF_ARCH:
     register(_t, _hf_decoder_config, _llama_class)
 
@@ -110,6 +118,8 @@ def model_class_for(cfg) -> type:
         return _lizezen_class()
     if isinstance(cfg, VivesunConfig):
         return _vivesun_class()
+    if isinstance(cfg, KevelornConfig):
+        return _kevelorn_class()
     if isinstance(cfg, LlamaConfig):
         return _llama_class()
     raise ValueError(f"no model class for {type(cfg).__name__}")

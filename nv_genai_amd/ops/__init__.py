@@ -554,8 +554,9 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H: int, G: int, dk:
     head: q head (h, m) is column block ``h * maps + m``, its keys are k head
     ``(h // (H / G)) * maps + m``, both maps read v head ``h // (H / G)``; two maps combine as
     ``a_0 - lam * a_1`` (differential attention). ``unit_eps``: divide every head's output by its
-    root mean square (eps inside the root) and multiply by ``out_scale``. ``gate`` [T, H]: the
-    head outputs are multiplied by ``sigmoid(gate)``. ``factor``: the outputs are multiplied by it.
+    root mean square (eps inside the root) and multiply by ``out_scale``. ``gate`` [T, H] or
+    [T, H * dv]: the head outputs are multiplied by ``sigmoid(gate)``, one gate per head or one per
+    element. ``factor``: the outputs are multiplied by it.
     ``tok_seq[t]`` is the block-table row of
     token t, ``pos[t]`` its position (negative: padding row, zeros out). Scores, softmax and
     accumulation are fp32. ``v_in_k`` (one map, dv <= dk): the values are the first dv elements of
@@ -663,9 +664,9 @@ def residual_add_rmsnorm_(x: torch.Tensor, y: torch.Tensor, w: Optional[torch.Te
     return out
 
 
-def rotary_frequencies(dims: int, base: float, yarn=None, bands=None) -> Tuple[torch.Tensor, float]:
+def rotary_frequencies(dims: int, base: float, yarn=None, bands=None, linear: float = 1.0) -> Tuple[torch.Tensor, float]:
     """(float64 frequencies [dims / 2], factor on cos and sin) of rotary positions on ``dims``
-    elements: ``f_i = base^(-2i / dims)``. ``yarn`` = (factor, original, fast, slow): with
+    elements: ``f_i = base^(-2i / dims) / linear``. ``yarn`` = (factor, original, fast, slow): with
     ``pair(t) = dims ln(original / (2 pi t)) / (2 ln base)`` the index of the pair that turns t
     times in ``original`` positions, ``lo = max(floor(pair(fast)), 0)``,
     ``hi = min(ceil(pair(slow)), dims - 1)`` and ``ramp_i = clamp((i - lo) / max(hi - lo, 0.001),
@@ -675,7 +676,7 @@ def rotary_frequencies(dims: int, base: float, yarn=None, bands=None) -> Tuple[t
     (``l > original / low``) or is ``(1 - s) f / factor + s f`` with
     ``s = (original / l - low) / (high - low)`` in between."""
     i = torch.arange(dims // 2, dtype=torch.float64)
-    f = torch.tensor([float(base) ** (-2.0 * k / dims) for k in range(dims // 2)], dtype=torch.float64)
+    f = torch.tensor([float(base) ** (-2.0 * k / dims) / linear for k in range(dims // 2)], dtype=torch.float64)
     if bands:
         factor, low, high, orig = (float(v) for v in bands)
         turns = orig * f / (2.0 * math.pi)                       # original / wavelength
@@ -797,11 +798,14 @@ def bias_gelu_tanh_(x: torch.Tensor, bias: Optional[torch.Tensor]) -> torch.Tens
 
 
 def rope_headnorm_cache_(proj, pos, slots, kc, vc, H: int, G: int, dk: int, dv: int, freq, mag: float, rot_dims: int,
-                         eps: float, q_w=None, k_w=None, v_off: Optional[int] = None):
+                         eps: float, q_w=None, k_w=None, v_off: Optional[int] = None, interleaved: bool = False,
+                         unit: bool = False):
     """Projection rows ``[q: H heads of dk | k: G heads of dk | ...]`` in place, one launch:
     RMS-normalise every q head with ``q_w`` [dk] and every k head with ``k_w`` [dk] (None: left
-    as it is), then rotary positions on the first ``rot_dims`` elements of every q and k head
-    (pair i = elements (i, i + rot_dims / 2) at angle ``pos * freq[i]`` - float64 product reduced
+    as it is, or, with ``unit``, normalised without a weight - a rotation keeps the mean square, so
+    with ``mag`` 1 that is also the norm of the rotated head), then rotary positions on the first
+    ``rot_dims`` elements of every q and k head (pair i = elements (i, i + rot_dims / 2), or
+    (2i, 2i + 1) when ``interleaved``, at angle ``pos * freq[i]`` - float64 product reduced
     to one turn before the fp32 cos / sin -, cos and sin times ``mag``), q and k written back, k
     into the token's page slot of K [blocks, G, 64, dk]. The values go into V [blocks, G, 64, dv]:
     columns ``v_off .. v_off + G * dv`` of the row, or, with ``v_off`` None (dv = dk), the k heads
@@ -811,9 +815,11 @@ def rope_headnorm_cache_(proj, pos, slots, kc, vc, H: int, G: int, dk: int, dv: 
     if v_off is None and dv != dk:
         raise ValueError("values taken from the keys need dv = dk")
     if not _gpu(proj):
-        return ref.rope_headnorm_cache_(proj, pos, slots, kc, vc, H, G, dk, dv, freq, mag, rot_dims, eps, q_w, k_w, v_off)
+        return ref.rope_headnorm_cache_(proj, pos, slots, kc, vc, H, G, dk, dv, freq, mag, rot_dims, eps, q_w, k_w, v_off,
+                                        interleaved, unit)
     kernels().rope_headnorm_cache(proj, pos, slots, kc, vc, int(H), int(G), int(dk), int(dv), freq, float(mag),
-                                  int(rot_dims), float(eps), q_w, k_w, -1 if v_off is None else int(v_off))
+                                  int(rot_dims), float(eps), q_w, k_w, -1 if v_off is None else int(v_off),
+                                  bool(interleaved), bool(unit))
     return proj
 
 
@@ -998,6 +1004,65 @@ def _delta(out, q, k, v, w, b, w_vec, b_vec, state, mode, H, G, d, dv, decay, cu
             raise ValueError("delta scans of portions need max_q, the rows of the longest one")
         ws = _delta_workspace(T, n - ns, H, d, out.device)
         C.delta_blocks(out, ws, q, k, v, w, b, *args, cu[ns:], slots[ns:], pos, int(max_q))
+
+
+# ------------------------------------------------------------------------- diagonal linear recurrences, scaled steps
+LINEAR_CHUNK = 16       # rows per block of the matrix form
+
+
+def linear_scan(q, k, v, state, H: int, d: int, dv: int, cu, slots, pos, z=None, z_bias=None, tau: float = 1.0,
+                log_decay=None, q_scale: float = 1.0, silu: bool = False, n_single: int = 0, max_q: int = 0) -> torch.Tensor:
+    """Linear attention with a diagonal decay over a step's rows: q, k rows [T, H*d], v rows [T, H*dv] (any row
+    strides). Per head ``S <- diag(w) S + k v^T``, ``o = S^T q`` with, in fp32, ``w = sigmoid(z + z_bias)^(1 / tau)``
+    per key channel and row (``z`` rows [T, H*d], ``z_bias`` fp32 [H*d]), or one constant
+    ``w = exp(log_decay)`` per head (``log_decay`` fp32 [H], at most 0); ``silu``: q, k and v pass silu first; q
+    is multiplied by ``q_scale``. Segment b is rows ``cu[b] .. cu[b + 1]`` (``cu`` None: row b alone) of one
+    sequence; its state [H, d, dv] (fp32) comes from ``state[slots[b]]``, or zeros when the segment
+    starts at position 0 - a reused slot needs no clearing - and goes back there. ``slots[b]`` < 0:
+    nothing is read or kept. Returns the fp32 outputs [T, H*dv].
+
+    GPU: single rows (``cu`` None, or the first ``n_single`` segments) take the row kernel; portions (at
+    most ``max_q`` rows each) the matrix form (csrc/kernels/linear_scan.hip)."""
+    if (z is None) == (log_decay is None) or (z is not None and z_bias is None):
+        raise ValueError("linear_scan: a decay per channel (z, z_bias) or a constant one per head (log_decay)")
+    if not tau > 0:
+        raise ValueError("linear_scan: tau must be positive")
+    if not _gpu(q):
+        return ref.linear_scan(q, k, v, state, H, d, dv, cu, slots, pos, z, z_bias, tau, log_decay, q_scale, silu)
+    C = kernels()
+    T, n = q.shape[0], slots.numel()
+    out = torch.empty(T, H * dv, dtype=torch.float32, device=q.device)
+    vec = log_decay if z is None else z_bias
+    args = (vec, state, int(H), int(d), int(dv), 1.0 / float(tau), float(q_scale), bool(silu))
+    ns = n if cu is None else int(n_single)
+    if ns:   # single rows: the first ns segments are the first ns rows
+        C.linear_rows(out[:ns], q[:ns], k[:ns], v[:ns], None if z is None else z[:ns], *args, slots[:ns], pos[:ns])
+    if ns < n:
+        if max_q < 1:
+            raise ValueError("linear_scan of portions needs max_q, the rows of the longest one")
+        D = 16 * int(C.delta_key_tiles(d))
+        ws = torch.empty((T // LINEAR_CHUNK + n - ns) * H * (33 * D + 256), dtype=torch.float32, device=q.device)
+        C.linear_blocks(out, ws, q, k, v, z, *args, cu[ns:], slots[ns:], pos, int(max_q))
+    return out
+
+
+def residual_step_(x: torch.Tensor, y: Optional[torch.Tensor], norm_w: Optional[torch.Tensor], eps: float,
+                   dtype: torch.dtype, mult: float = 1.0, y2: Optional[torch.Tensor] = None, pair: Optional[tuple] = None,
+                   x0: Optional[torch.Tensor] = None, row: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """Step on an fp32 stream in one launch: ``x += mult * a`` in place with ``a = y`` (+ ``y2``), or, with ``pair`` =
+    (w1, w2), ``a = rmsnorm(y) * w1 + rmsnorm(y2) * w2``; then ``x += x0`` (fp32 rows) and ``x += row`` (one fp32
+    row) where given. Returns ``rmsnorm(x) * norm_w`` in ``dtype`` (``norm_w`` None: None). ``y`` None: the
+    additions only."""
+    if pair is not None and y2 is None:
+        raise ValueError("residual_step_: a pair of norms needs both outputs")
+    out = None if norm_w is None else torch.empty(x.shape, dtype=dtype, device=x.device)
+    if not _gpu(x):
+        ref.residual_step_(x, y, norm_w, eps, out, mult, y2, pair, x0, row)
+        return out
+    w1, w2 = pair if pair is not None else (None, None)
+    kernels().residual_step(x, y, y2, w1, w2, float(mult), x0, row, norm_w, float(eps), out, None, 0,
+                            dtype == torch.float32)
+    return out
 
 
 class DecodeWorkspace:
@@ -1360,16 +1425,27 @@ def moe_glu_experts(x: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w13: 
     weight and the activation in its epilogue -> grouped down GEMM -> combine (fp32 sum per token).
     bf16 rows with MFMA-sized experts run the grouped MFMA GEMMs, everything else (fp32, other
     sizes) a tiled fp32-accumulating kernel of the same structure."""
-    swiglu = math.isinf(limit) and alpha == 1.0 and shift == 0.0 and not weight_input
     if not _gpu(x):
         return ref.moe_glu_experts(x, ids, wts, w13, w2, limit, alpha, weight_input, add, shift, identity)
+    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    if x.shape[0] == 0:
+        return out
+    y, inv = _glu_expert_rows(x, ids, wts, w13, w2, limit, alpha, weight_input, shift, ws)
+    k, E = int(ids.shape[1]), w13.shape[0]
+    if identity:
+        kernels().moe_combine_rows(y, inv, x.shape[0], k, add, out, x, ids.reshape(-1), wts.reshape(-1), E)
+    else:
+        kernels().moe_combine_rows(y, inv, x.shape[0], k, add, out, None, None, None, E)
+    return out
+
+
+def _glu_expert_rows(x, ids, wts, w13, w2, limit, alpha, weight_input, shift, ws):
+    """(expert rows [T * k, H] sorted by expert, their row numbers per token)."""
+    swiglu = math.isinf(limit) and alpha == 1.0 and shift == 0.0 and not weight_input
     C = kernels()
     T, H = x.shape
     E, F2, K = w13.shape
     F, k = F2 // 2, ids.shape[1]
-    out = torch.empty(T, H, dtype=x.dtype, device=x.device)
-    if T == 0:
-        return out
     M = T * k
     if ws is None:
         ws = MoEWorkspace.get(T, k, E, x.device)
@@ -1394,10 +1470,24 @@ def moe_glu_experts(x: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w13: 
         C.moe_gemm_rows(x, w13, ws.sorted_tok, ws.sorted_w, ws.tiles, mt, h, 0, lim, float(alpha),
                         bool(weight_input), float(shift))
         C.moe_gemm_rows(h, w2, ws.sorted_tok, ws.sorted_w, ws.tiles, mt, y, 1, 0.0, 0.0, not weight_input, 0.0)
-    if identity:
-        C.moe_combine_rows(y, ws.inv, T, int(k), add, out, x, ids.reshape(-1), wts.reshape(-1), E)
-    else:
-        C.moe_combine_rows(y, ws.inv, T, int(k), add, out, None, None, None, E)
+    return y, ws.inv
+
+
+def residual_glu_experts_(x: torch.Tensor, h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w13: torch.Tensor,
+                          w2: torch.Tensor, norm_w: Optional[torch.Tensor], eps: float, dtype: torch.dtype,
+                          mult: float = 1.0, add: Optional[torch.Tensor] = None, x0: Optional[torch.Tensor] = None,
+                          row: Optional[torch.Tensor] = None, ws: Optional["MoEWorkspace"] = None) -> Optional[torch.Tensor]:
+    """``x += mult * (sum of the token's SwiGLU expert outputs + add)`` on an fp32 stream in place, the expert rows
+    summed straight into it (fp32) by the launch that also does the rest of :func:`residual_step_` (``x0``,
+    ``row``, the next norm). ``add`` [T, H]: a shared expert's output."""
+    if not _gpu(x):
+        y = ref.moe_glu_experts(h, ids, wts, w13, w2, math.inf, 1.0, False, None, 0.0, False)
+        return residual_step_(x, y, norm_w, eps, dtype, mult, add, None, x0, row)
+    out = None if norm_w is None else torch.empty(x.shape, dtype=dtype, device=x.device)
+    if x.shape[0]:
+        y, inv = _glu_expert_rows(h, ids, wts, w13, w2, math.inf, 1.0, False, 0.0, ws)
+        kernels().residual_step(x, y, add, None, None, float(mult), x0, row, norm_w, float(eps), out, inv,
+                                int(ids.shape[1]), dtype == torch.float32)
     return out
 
 

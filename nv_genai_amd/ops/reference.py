@@ -583,7 +583,7 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale
     """Softmax attention of token rows over row-major pages, one row at a time. ``maps`` score
     maps per head (q head (h, m) at column (h * maps + m) * dk, k head (h // (H / G)) * maps + m,
     v head h // (H / G)), combined as a_0 - lam * a_1; optional unit RMS per head (times
-    ``out_scale``) and a per-head sigmoid gate. ``v_in_k``: the values are the first dv elements
+    ``out_scale``) and a sigmoid gate per head or per output element. ``v_in_k``: the values are the first dv elements
     of the key rows. ``softcap`` > 0: scores become softcap * tanh(score / softcap). ``chunk`` > 0:
     only keys of the query's own chunk; ``sink``: score of a key without a value;
     ``factor``: multiplies the outputs."""
@@ -617,7 +617,7 @@ def softmax_attention(q, kc, vc, block_tables, tok_seq, pos, H, G, dk, dv, scale
         out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + unit_eps) * out_scale
     out = out * factor
     if gate is not None:
-        out = out * torch.sigmoid(gate.float())[:, :, None]
+        out = out * torch.sigmoid(gate.float()).view(T, H, -1)
     return out.reshape(T, H * dv).to(q.dtype)
 
 
@@ -812,19 +812,19 @@ def bias_gelu_tanh_(x, bias):
 
 
 def rope_headnorm_cache_(proj, pos, slots, kc, vc, H, G, dk, dv, freq, mag, rot_dims, eps, q_w=None, k_w=None,
-                         v_off=None):
+                         v_off=None, interleaved=False, unit=False):
     """See :func:`nv_genai_amd.ops.rope_headnorm_cache_`."""
     T = proj.shape[0]
     n0, n1 = H * dk, (H + G) * dk
     q = proj[:, :n0].float().view(T, H, dk)
     k = proj[:, n0:n1].float().view(T, G, dk)
     v = k.clone() if v_off is None else proj[:, v_off:v_off + G * dv].float().view(T, G, dv)
-    if q_w is not None:
-        q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * q_w
-    if k_w is not None:
-        k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * k_w
+    if q_w is not None or unit:
+        q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * (1.0 if q_w is None else q_w)
+    if k_w is not None or unit:
+        k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * (1.0 if k_w is None else k_w)
     cos, sin = rotary_cos_sin(pos.clamp(min=0), freq, mag)
-    q, k = _rotate(q, cos, sin, rot_dims, False), _rotate(k, cos, sin, rot_dims, False)
+    q, k = _rotate(q, cos, sin, rot_dims, interleaved), _rotate(k, cos, sin, rot_dims, interleaved)
     proj[:, :n0] = q.reshape(T, n0).to(proj.dtype)
     proj[:, n0:n1] = k.reshape(T, n1 - n0).to(proj.dtype)
     sl = slots.long()
@@ -1015,3 +1015,47 @@ def moe_plain_experts(x, ids, wts, w1, w2):
             h = torch.nn.functional.gelu(x[tok].float() @ w1[e].float().t()).to(x.dtype)
             out.index_add_(0, tok, (h.float() @ w2[e].float().t()) * wts[tok, slot].unsqueeze(1))
     return out.to(x.dtype)
+
+
+# ------------------------------------------------------------------------- diagonal linear recurrences, scaled steps
+def linear_scan(q, k, v, state, H, d, dv, cu, slots, pos, z=None, z_bias=None, tau=1.0, log_decay=None, q_scale=1.0,
+                silu=False):
+    """See :func:`nv_genai_amd.ops.linear_scan`."""
+    T = q.shape[0]
+    qf, kf, vf = q.float(), k.float(), v.float()
+    if silu:
+        qf, kf, vf = (torch.nn.functional.silu(t) for t in (qf, kf, vf))
+    qf, kf, vf = (qf * q_scale).reshape(T, H, d), kf.reshape(T, H, d), vf.reshape(T, H, dv)
+    if z is None:
+        w = torch.exp(log_decay)[None, :, None].expand(T, H, d)
+    else:
+        w = torch.exp(torch.nn.functional.logsigmoid(z.float() + z_bias) / tau).reshape(T, H, d)
+    out = torch.zeros(T, H, dv, dtype=torch.float32, device=q.device)
+    for t0, t1, sl, S in _delta_segments(state, cu, slots, pos):
+        for t in range(t0, t1):
+            S = w[t][:, :, None] * S + kf[t][:, :, None] * vf[t][:, None, :]
+            out[t] = torch.einsum("hdv,hd->hv", S, qf[t])
+        if sl >= 0:
+            state[sl] = S
+    return out.reshape(T, H * dv)
+
+
+def residual_step_(x, y, norm_w, eps, out, mult, y2, pair, x0, row):
+    """See :func:`nv_genai_amd.ops.residual_step_`."""
+    def unit(t):
+        t = t.float()
+        return t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps)
+
+    if y is not None:
+        if pair is not None:
+            a = unit(y) * pair[0] + unit(y2) * pair[1]
+        else:
+            a = y.float() if y2 is None else y.float() + y2.float()
+        x.add_(a * mult)
+    if x0 is not None:
+        x.add_(x0)
+    if row is not None:
+        x.add_(row)
+    if norm_w is not None:
+        out.copy_(unit(x) * norm_w)
+    return x
