@@ -1326,6 +1326,59 @@ void residual_add_rmsnorm(Tensor x, Tensor y, c10::optional<Tensor> w, double ep
                                    (float)eps, x.size(0), (int)H, op, ip, (int)k, f32, cur_stream(x));
 }
 
+void residual_step(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> y2, c10::optional<Tensor> w1,
+                   c10::optional<Tensor> w2, double mult, c10::optional<Tensor> x0, c10::optional<Tensor> row,
+                   c10::optional<Tensor> w, double eps, c10::optional<Tensor> out, c10::optional<Tensor> inv, int64_t k,
+                   bool f32) {
+  CHECK_F32(x); CHECK_CONTIG(x);
+  const int64_t T = x.size(0), H = x.size(1);
+  const auto st = f32 ? at::kFloat : at::kBFloat16;
+  nga::ResidualStepParams p{};
+  p.x = x.data_ptr<float>();
+  if (inv.has_value()) {   // rows of y gathered by number (numbers < y rows: moe_align writes them below T * k)
+    CHECK_I32(*inv);
+    TORCH_CHECK(k >= 1 && y.has_value() && inv->numel() >= T * k && y->size(0) >= T * k && !w1.has_value());
+    p.inv = inv->data_ptr<int32_t>();
+    p.k = (int)k;
+  }
+  auto rows = [&](const Tensor& t, bool gathered, const char* what) {
+    TORCH_CHECK(t.is_cuda() && t.scalar_type() == st && t.dim() == 2 && (gathered || t.size(0) == T) && t.size(1) == H &&
+                t.stride(1) == 1, "residual_step: ", what, " rows");
+  };
+  if (y.has_value()) {
+    rows(*y, p.inv != nullptr, "y");
+    p.y = y->data_ptr();
+    p.ys = y->stride(0);
+  }
+  if (y2.has_value()) {
+    TORCH_CHECK(y.has_value());
+    rows(*y2, false, "y2");
+    p.y2 = y2->data_ptr();
+    p.y2s = y2->stride(0);
+  }
+  TORCH_CHECK(w1.has_value() == w2.has_value() && (!w1.has_value() || y2.has_value()),
+              "residual_step: a pair of norms needs both weights and both outputs");
+  p.w1 = opt_f32(w1, H, "norm weight");
+  p.w2 = opt_f32(w2, H, "norm weight");
+  p.mult = (float)mult;
+  if (x0.has_value()) {
+    CHECK_F32(*x0); CHECK_CONTIG(*x0);
+    TORCH_CHECK(x0->sizes() == x.sizes());
+    p.x0 = x0->data_ptr<float>();
+  }
+  p.row = opt_f32(row, H, "row");
+  p.w = opt_f32(w, H, "norm weight");
+  p.eps = (float)eps;
+  TORCH_CHECK(w.has_value() == out.has_value(), "residual_step: a norm weight and its output come together");
+  if (out.has_value()) {
+    CHECK_CONTIG(*out);
+    TORCH_CHECK(out->is_cuda() && out->scalar_type() == st && out->sizes() == x.sizes());
+    p.out = out->data_ptr();
+  }
+  p.H = (int)H;
+  nga::launch_residual_step(p, T, f32, cur_stream(x));
+}
+
 void clamped_glu(Tensor out, Tensor x, int64_t F, double limit, double alpha, int64_t gate_col, double shift) {
   const bool f32 = act_f32(x);
   CHECK_CONTIG(out);
@@ -1480,7 +1533,7 @@ void bias_gelu_tanh(Tensor x, c10::optional<Tensor> bias) {
 
 void rope_headnorm_cache(Tensor proj, Tensor pos, Tensor slots, Tensor kc, Tensor vc, int64_t H, int64_t G, int64_t dk,
                          int64_t dv, Tensor freq, double mag, int64_t rot_dims, double eps, c10::optional<Tensor> q_w,
-                         c10::optional<Tensor> k_w, int64_t v_off) {
+                         c10::optional<Tensor> k_w, int64_t v_off, bool interleaved, bool unit) {
   const bool f32 = act_f32(proj);
   CHECK_I32(pos); CHECK_I32(slots);
   const int64_t T = proj.size(0), W = proj.size(1);
@@ -1511,6 +1564,8 @@ void rope_headnorm_cache(Tensor proj, Tensor pos, Tensor slots, Tensor kc, Tenso
   p.q_w = opt_f32(q_w, dk, "q head norm weight");
   p.k_w = opt_f32(k_w, dk, "k head norm weight");
   p.v_off = (int)v_off;
+  p.interleaved = interleaved ? 1 : 0;
+  p.unit = unit ? 1 : 0;
   nga::launch_rope_headnorm_cache(p, T, f32, cur_stream(proj));
 }
 
@@ -1592,6 +1647,7 @@ void headnorm_cache(Tensor proj, Tensor slots, Tensor kc, c10::optional<Tensor> 
 struct SoftmaxArgs {
   const void* gp = nullptr;
   int64_t gs = 0;
+  int gd = 1;      // gates per head
 };
 
 SoftmaxArgs check_softmax_args(const Tensor& out, const Tensor& q, const c10::optional<Tensor>& gate, const Tensor& kc,
@@ -1615,9 +1671,10 @@ SoftmaxArgs check_softmax_args(const Tensor& out, const Tensor& q, const c10::op
   SoftmaxArgs a;
   if (gate.has_value()) {
     TORCH_CHECK(gate->is_cuda() && gate->scalar_type() == q.scalar_type() && gate->dim() == 2 && gate->size(0) == T &&
-                gate->size(1) == H && gate->stride(1) == 1, "gate must be [T, H] rows");
+                (gate->size(1) == H || gate->size(1) == H * dv) && gate->stride(1) == 1, "gate must be [T, H] or [T, H * dv] rows");
     a.gp = gate->data_ptr();
     a.gs = gate->stride(0);
+    a.gd = gate->size(1) == H ? 1 : (int)dv;
   }
   return a;
 }
@@ -1632,7 +1689,7 @@ void softmax_attention(Tensor out, Tensor q, c10::optional<Tensor> gate, Tensor 
   const SoftmaxArgs a = check_softmax_args(out, q, gate, kc, vc, H, G, dk, dv, window, maps, v_in_k);
   const int64_t T = q.size(0);
   TORCH_CHECK(tok_seq.numel() == T && pos.numel() == T && block_tables.dim() == 2);
-  nga::launch_softmax_attention(out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), a.gp, a.gs, kc.data_ptr(), vc.data_ptr(),
+  nga::launch_softmax_attention(out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), a.gp, a.gs, a.gd, kc.data_ptr(), vc.data_ptr(),
                                 block_tables.data_ptr<int32_t>(), (int)block_tables.size(1),
                                 tok_seq.data_ptr<int32_t>(), pos.data_ptr<int32_t>(), T, (int)H, (int)G, (int)dk,
                                 (int)dv, (float)scale, (int)window, (int)maps, (float)lam, (float)unit_eps,
@@ -1653,9 +1710,10 @@ void softmax_attention_prefill(Tensor out, Tensor q, c10::optional<Tensor> gate,
   TORCH_CHECK(nga::softmax_attention_mfma_supported((int)dk, (int)dv, (int)(H / G), (int)maps),
               "softmax_attention_prefill: head sizes the MFMA kernel does not take");
   TORCH_CHECK(q.stride(0) % 8 == 0 && (uintptr_t)q.data_ptr() % 16 == 0, "q rows must be 16-B aligned");
+  TORCH_CHECK(a.gd == 1 || (a.gs % 4 == 0 && (uintptr_t)a.gp % 8 == 0), "gates per element must be 8-B aligned rows");
   const int64_t B = ctx_lens.numel();
   TORCH_CHECK(cu_q.numel() == B + 1 && block_tables.dim() == 2 && block_tables.size(0) >= B && max_q_len >= 0);
-  nga::launch_softmax_attention_mfma(bfp(out), out.stride(0), bfp(q), q.stride(0), (const uint16_t*)a.gp, a.gs, bfp(kc), bfp(vc),
+  nga::launch_softmax_attention_mfma(bfp(out), out.stride(0), bfp(q), q.stride(0), (const uint16_t*)a.gp, a.gs, a.gd, bfp(kc), bfp(vc),
                                      block_tables.data_ptr<int32_t>(), (int)block_tables.size(1),
                                      cu_q.data_ptr<int32_t>(), ctx_lens.data_ptr<int32_t>(), (int)B, (int)max_q_len,
                                      (int)H, (int)G, (int)dk, (int)dv, (float)scale, (int)window, (int)maps, (float)lam,
@@ -1680,7 +1738,7 @@ void softmax_attention_decode(Tensor out, Tensor ws, int64_t parts, Tensor q, c1
               (uintptr_t)ws.data_ptr() % 16 == 0);
   TORCH_CHECK(tok_seq.numel() == T && pos.numel() == T && block_tables.dim() == 2);
   nga::launch_softmax_decode_mfma(bfp(out), out.stride(0), ws.data_ptr<float>(), (int)parts, bfp(q), q.stride(0),
-                                  (const uint16_t*)a.gp, a.gs, bfp(kc), bfp(vc), block_tables.data_ptr<int32_t>(),
+                                  (const uint16_t*)a.gp, a.gs, a.gd, bfp(kc), bfp(vc), block_tables.data_ptr<int32_t>(),
                                   (int)block_tables.size(1), tok_seq.data_ptr<int32_t>(), pos.data_ptr<int32_t>(), T,
                                   (int)H, (int)G, (int)dk, (int)dv, (float)scale, (int)window, (int)maps, (float)lam,
                                   (float)unit_eps, (float)out_scale, v_in_k, (float)softcap, (int)chunk, (float)sink, cur_stream(q));
@@ -1818,6 +1876,65 @@ void delta_blocks(Tensor out, Tensor ws, Tensor q, Tensor k, Tensor v, Tensor w,
   nga::launch_delta_blocks(p, ws.data_ptr<float>(), (int)n, (int)max_q, f32, cur_stream(q));
 }
 
+nga::LinearParams linear_params(const Tensor& out, const Tensor& q, const Tensor& k, const Tensor& v,
+                                const c10::optional<Tensor>& z, const Tensor& vec, const Tensor& state, int64_t H, int64_t d,
+                                int64_t dv, double inv_tau, double q_scale, bool silu, const Tensor& slots, const Tensor& pos) {
+  CHECK_F32(out); CHECK_CONTIG(out); CHECK_F32(vec); CHECK_CONTIG(vec); CHECK_F32(state); CHECK_CONTIG(state);
+  CHECK_I32(slots); CHECK_I32(pos);
+  const int64_t T = q.size(0);
+  TORCH_CHECK(H >= 1 && d >= 1 && d <= 256 && dv >= 1, "linear_scan: heads, key size (at most 256) or value size");
+  auto rows = [&](const Tensor& t, int64_t cols, const char* what) {
+    TORCH_CHECK(t.is_cuda() && t.scalar_type() == q.scalar_type() && t.dim() == 2 && t.size(0) == T && t.size(1) == cols &&
+                t.stride(1) == 1, "linear_scan: ", what, " rows");
+  };
+  rows(q, H * d, "q"); rows(k, H * d, "k"); rows(v, H * dv, "v");
+  if (z.has_value()) rows(*z, H * d, "decay");
+  TORCH_CHECK(vec.numel() == (z.has_value() ? H * d : H));
+  TORCH_CHECK(out.dim() == 2 && out.size(0) == T && out.size(1) == H * dv && pos.numel() == T);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == d && state.size(3) == dv,
+              "linear_scan: state [slots, H, d, dv]");
+  nga::LinearParams p{};
+  p.out = out.data_ptr<float>();
+  p.q = q.data_ptr(); p.k = k.data_ptr(); p.v = v.data_ptr();
+  p.qs = q.stride(0); p.ks = k.stride(0); p.vs = v.stride(0);
+  if (z.has_value()) {
+    p.z = z->data_ptr();
+    p.zs = z->stride(0);
+  }
+  p.vec = vec.data_ptr<float>();
+  p.state = state.data_ptr<float>();
+  p.H = (int)H; p.d = (int)d; p.dv = (int)dv; p.silu = silu ? 1 : 0;
+  p.inv_tau = (float)inv_tau;
+  p.q_scale = (float)q_scale;
+  p.slots = slots.data_ptr<int32_t>();
+  p.pos = pos.data_ptr<int32_t>();
+  return p;
+}
+
+// single rows: row i is segment i
+void linear_rows(Tensor out, Tensor q, Tensor k, Tensor v, c10::optional<Tensor> z, Tensor vec, Tensor state, int64_t H,
+                 int64_t d, int64_t dv, double inv_tau, double q_scale, bool silu, Tensor slots, Tensor pos) {
+  const bool f32 = act_f32(q);
+  TORCH_CHECK(slots.numel() == q.size(0), "linear_rows: every row is a segment");
+  nga::launch_linear_rows(linear_params(out, q, k, v, z, vec, state, H, d, dv, inv_tau, q_scale, silu, slots, pos),
+                          (int)q.size(0), f32, cur_stream(q));
+}
+
+// portions: segment i is rows cu[i] .. cu[i + 1] of the launch's rows, at most max_q of them; ws: block operands
+void linear_blocks(Tensor out, Tensor ws, Tensor q, Tensor k, Tensor v, c10::optional<Tensor> z, Tensor vec, Tensor state,
+                   int64_t H, int64_t d, int64_t dv, double inv_tau, double q_scale, bool silu, Tensor cu, Tensor slots,
+                   Tensor pos, int64_t max_q) {
+  const bool f32 = act_f32(q);
+  CHECK_F32(ws); CHECK_CONTIG(ws); CHECK_I32(cu);
+  nga::LinearParams p = linear_params(out, q, k, v, z, vec, state, H, d, dv, inv_tau, q_scale, silu, slots, pos);
+  const int64_t n = slots.numel(), T = q.size(0), dt = nga::delta_key_tiles((int)d);
+  TORCH_CHECK(cu.numel() == n + 1 && max_q >= 1 && max_q <= T);
+  TORCH_CHECK(ws.numel() >= (T / 16 + n) * H * (33 * 16 * dt + 256) && (uintptr_t)ws.data_ptr() % 16 == 0,
+              "linear_blocks: workspace too small");
+  p.cu = cu.data_ptr<int32_t>();
+  nga::launch_linear_blocks(p, ws.data_ptr<float>(), (int)n, (int)max_q, f32, cur_stream(q));
+}
+
 void hgrn2_scan(Tensor out, Tensor proj, Tensor f_bias, Tensor lower, Tensor state, int64_t H, int64_t d, int64_t dv,
                 c10::optional<Tensor> cu, Tensor slots, Tensor pos) {
   const bool f32 = act_f32(proj);
@@ -1913,6 +2030,9 @@ PYBIND11_MODULE(_C, m) {
   m.def("gelu_gate_rows", checked("gelu_gate_rows", &gelu_gate_rows));
   m.def("tanh_rows", checked("tanh_rows", &tanh_rows));
   m.def("short_conv", checked("short_conv", &short_conv));
+  m.def("residual_step", checked("residual_step", &residual_step));
+  m.def("linear_rows", checked("linear_rows", &linear_rows));
+  m.def("linear_blocks", checked("linear_blocks", &linear_blocks));
   m.def("delta_rows", checked("delta_rows", &delta_rows));
   m.def("delta_blocks", checked("delta_blocks", &delta_blocks));
   m.def("delta_key_tiles", [](int64_t d) { return (int64_t)nga::delta_key_tiles((int)d); });

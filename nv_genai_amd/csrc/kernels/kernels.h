@@ -302,6 +302,23 @@ void launch_softcap(float* z, int64_t n, float cap, float scale, hipStream_t str
 // inv != nullptr: row t adds the sum of the k rows inv[t k ..] of y (< 0: none)
 void launch_residual_add_rmsnorm(float* x, const void* y, int64_t y_stride, const float* w, float eps, int64_t T, int H,
                                  void* out, const int32_t* inv, int k, bool f32, hipStream_t stream);
+// x += mult * a, a = y (+ y2) or rmsnorm(y) w1 + rmsnorm(y2) w2 (w1 != nullptr), or, with inv, the sum of y's rows
+// inv[t k ..] (+ y2); then x += x0 (rows) and += row; out = rmsnorm(x) * w. Everything but x may be nullptr.
+struct ResidualStepParams {
+  float* x;                  // [T, H]
+  const void *y, *y2;        // activation type
+  int64_t ys, y2s;           // row strides
+  const float *w1, *w2;
+  float mult;
+  const float* x0;           // [T, H]
+  const float* row;          // [H]
+  const float* w;
+  float eps;
+  void* out;                 // [T, H] activation type (with w)
+  const int32_t* inv;
+  int k, H;
+};
+void launch_residual_step(const ResidualStepParams& p, int64_t T, bool f32, hipStream_t stream);
 void launch_clamped_glu(void* out, const void* in, int64_t in_stride, int64_t T, int F, float limit, float alpha,
                         int gate_col, float shift, bool f32, hipStream_t stream);
 void launch_dyt_norm(void* out, const float* x, float alpha, const float* w, const float* b, const int64_t* rows,
@@ -332,7 +349,8 @@ struct LatentRopeParams {
   const float* n_w;
 };
 void launch_latent_rope_cache(const LatentRopeParams& p, int64_t T, bool f32, hipStream_t stream);
-// rope_headnorm_cache: rows [q: H heads of dk | k: G heads of dk | ...], head norms, rotary pairs (i, i + rot_dims / 2)
+// rope_headnorm_cache: rows [q: H heads of dk | k: G heads of dk | ...], head norms, rotary pairs (i, i + rot_dims / 2) or,
+// interleaved, (2i, 2i + 1)
 struct RopeHeadnormParams {
   void* proj;                // [T, stride] projection rows (activation type)
   int64_t stride;
@@ -346,6 +364,8 @@ struct RopeHeadnormParams {
   const float* q_w;          // [dk] or nullptr: no norm of the q heads
   const float* k_w;          // [dk] or nullptr
   int v_off;                 // value columns [v_off, v_off + G * dv), or < 0: the k heads before norm and rotation
+  int interleaved;
+  int unit;                  // heads without a weight are normalised too
 };
 void launch_rope_headnorm_cache(const RopeHeadnormParams& p, int64_t T, bool f32, hipStream_t stream);
 // w: gs weights shared by the groups, or groups * gs (w_full); gate [T, groups * gs] rows of the output type or nullptr
@@ -368,24 +388,24 @@ void launch_tanh_rows(void* out, const void* x, int64_t x_stride, int64_t T, int
 void launch_headnorm_cache(void* proj, int64_t stride, const int32_t* slots, void* kc, void* vc, int64_t T, int nq,
                            int nk, int dk, int nv, int dv, float eps, const float* qw, const float* kw,
                            const float* bias, const int32_t* pos, float coef, int every, bool f32, hipStream_t stream);
-// chunk > 0: keys of the query's own chunk only; sink: score of a key without a value (-inf: none); o_stride: elements
+// gate: g_dim pre-sigmoid values per head (1 or dv) in rows of stride g_stride; chunk > 0: keys of the query's own chunk only; sink: score of a key without a value (-inf: none); o_stride: elements
 // between output rows
 void launch_softmax_attention(void* out, int64_t o_stride, const void* q, int64_t q_stride, const void* gate, int64_t g_stride,
-                              const void* kc, const void* vc, const int32_t* block_tables, int max_blocks,
+                              int g_dim, const void* kc, const void* vc, const int32_t* block_tables, int max_blocks,
                               const int32_t* tok_seq, const int32_t* pos, int64_t T, int H, int G, int dk, int dv,
                               float scale, int window, int maps, float lam, float unit_eps, float out_scale, bool v_in_k,
                               float softcap, int chunk, float sink, bool f32, hipStream_t stream);
 
 bool softmax_attention_mfma_supported(int dk, int dv, int group, int maps);
 void launch_softmax_attention_mfma(uint16_t* out, int64_t o_stride, const uint16_t* q, int64_t q_stride, const uint16_t* gate,
-                                   int64_t g_stride, const uint16_t* kc, const uint16_t* vc,
+                                   int64_t g_stride, int g_dim, const uint16_t* kc, const uint16_t* vc,
                                    const int32_t* block_tables, int max_blocks, const int32_t* cu_q,
                                    const int32_t* ctx_lens, int B, int max_q_len, int H, int G, int dk, int dv,
                                    float scale, int window, int maps, float lam, float unit_eps, float out_scale,
                                    bool v_in_k, float softcap, int chunk, float sink, hipStream_t stream);
 int softmax_decode_parts(int rows, int G, int max_ctx, int window);
 void launch_softmax_decode_mfma(uint16_t* out, int64_t o_stride, float* ws, int parts, const uint16_t* q, int64_t q_stride,
-                                const uint16_t* gate, int64_t g_stride, const uint16_t* kc, const uint16_t* vc,
+                                const uint16_t* gate, int64_t g_stride, int g_dim, const uint16_t* kc, const uint16_t* vc,
                                 const int32_t* block_tables, int max_blocks, const int32_t* tok_seq,
                                 const int32_t* pos, int64_t T, int H, int G, int dk, int dv, float scale, int window,
                                 int maps, float lam, float unit_eps, float out_scale, bool v_in_k, float softcap,
@@ -420,6 +440,23 @@ struct DeltaParams {
   const int32_t* slots;      // [n_seg]
   const int32_t* pos;        // [T]
 };
+// linear_scan.hip: rows q, k [H * d], v [H * dv]; z != nullptr: decay pre-activations [H * d] with bias vec [H * d]
+// (sigmoid(z + vec)^inv_tau); else vec = log decay per head [H]
+struct LinearParams {
+  float* out;                // [T, H * dv]
+  const void *q, *k, *v, *z;
+  int64_t qs, ks, vs, zs;    // row strides
+  const float* vec;
+  float* state;              // [slots, H, d, dv]
+  int H, d, dv, silu;        // silu: on q, k and v
+  float inv_tau, q_scale;
+  const int32_t* cu;         // portions: [n_seg + 1] row offsets
+  const int32_t* slots;      // [n_seg]
+  const int32_t* pos;        // [T]
+};
+void launch_linear_rows(const LinearParams& p, int n, bool f32, hipStream_t stream);
+void launch_linear_blocks(const LinearParams& p, float* ws, int n_seg, int max_q, bool f32, hipStream_t stream);
+
 int delta_key_tiles(int d);
 void launch_delta_rows(const DeltaParams& p, int n, bool f32, hipStream_t stream);
 void launch_delta_blocks(const DeltaParams& p, float* ws, int n_seg, int max_q, bool f32, hipStream_t stream);

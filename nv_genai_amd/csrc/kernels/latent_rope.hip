@@ -141,7 +141,7 @@ constexpr int MAX_HEAD = 512;   // widest q / k head of rope_headnorm_cache
 
 // One wave per (token, chunk of head units); units are the H q heads, the G k heads and, when the
 // values have columns of their own, G value heads that are only copied into the V page. A lane owns
-// the rotary pairs p = lane, lane + 64, ... (elements p and p + rot_dims / 2 of the head) and the
+// the rotary pairs p = lane, lane + 64, ... (elements p and p + rot_dims / 2 of the head, or 2 p and 2 p + 1) and the
 // unrotated tail elements rot_dims + lane, ...: both elements of a pair live in one lane, so the
 // rotation needs no exchange between lanes and no LDS, and the statistics of the head norm are one
 // wave reduction. cos / sin of the lane's pairs are computed once per wave and kept in registers.
@@ -158,6 +158,7 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_kernel(const RopeHead
   T* pr = (T*)P.proj + row * P.stride;
   const int p = P.pos[row] < 0 ? 0 : P.pos[row];
   const int half = P.rot_dims >> 1, dk = P.dk, tail = dk - P.rot_dims;
+  const int pm = P.interleaved ? 2 : 1, po = P.interleaved ? 1 : half;   // pair i = elements pm i and pm i + po
   float cs[MP], sn[MP];
 #pragma unroll
   for (int j = 0; j < MP; ++j) {
@@ -194,8 +195,8 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_kernel(const RopeHead
 #pragma unroll
     for (int j = 0; j < MP; ++j) {
       const int i = lane + 64 * j;
-      xa[j] = i < half ? ldf(src + i) : 0.f;
-      xb[j] = i < half ? ldf(src + half + i) : 0.f;
+      xa[j] = i < half ? ldf(src + pm * i) : 0.f;
+      xb[j] = i < half ? ldf(src + pm * i + po) : 0.f;
       ss += xa[j] * xa[j] + xb[j] * xb[j];
     }
 #pragma unroll
@@ -210,8 +211,8 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_kernel(const RopeHead
       for (int j = 0; j < MP; ++j) {
         const int i = lane + 64 * j;
         if (i < half) {
-          stf(vd + i, xa[j]);
-          stf(vd + half + i, xb[j]);
+          stf(vd + pm * i, xa[j]);
+          stf(vd + pm * i + po, xb[j]);
         }
       }
 #pragma unroll
@@ -221,7 +222,8 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_kernel(const RopeHead
       }
     }
     float r = 1.f;
-    if (w != nullptr) {
+    const bool normed = w != nullptr || P.unit;
+    if (normed) {
       ss = wave_sum(ss);
       r = 1.0f / sqrtf(ss / (float)dk + P.eps);
     }
@@ -230,18 +232,18 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_kernel(const RopeHead
     for (int j = 0; j < MP; ++j) {
       const int i = lane + 64 * j;
       if (i < half) {
-        float u = xa[j], v = xb[j];
+        float u = xa[j] * r, v = xb[j] * r;
         if (w != nullptr) {
-          u = u * r * w[i];
-          v = v * r * w[half + i];
+          u *= w[pm * i];
+          v *= w[pm * i + po];
         }
         // (u, v) -> (u cos - v sin, v cos + u sin)
         const float ru = u * cs[j] - v * sn[j], rv = v * cs[j] + u * sn[j];
-        stf(src + i, ru);
-        stf(src + half + i, rv);
+        stf(src + pm * i, ru);
+        stf(src + pm * i + po, rv);
         if (kdst) {
-          stf(kdst + i, ru);
-          stf(kdst + half + i, rv);
+          stf(kdst + pm * i, ru);
+          stf(kdst + pm * i + po, rv);
         }
       }
     }
@@ -249,8 +251,8 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_kernel(const RopeHead
     for (int j = 0; j < MT; ++j) {
       const int i = lane + 64 * j;
       if (i < tail) {
-        const float v = w != nullptr ? xt[j] * r * w[P.rot_dims + i] : xt[j];
-        if (w != nullptr) stf(src + P.rot_dims + i, v);
+        const float v = w != nullptr ? xt[j] * r * w[P.rot_dims + i] : xt[j] * r;
+        if (normed) stf(src + P.rot_dims + i, v);
         if (kdst) stf(kdst + P.rot_dims + i, v);
       }
     }
@@ -261,7 +263,8 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_kernel(const RopeHead
 // columns and pages: a lane owns two runs of 8 elements, so every access is 16 bytes, a head takes
 // CPH = dk / 16 lanes and a wave works on 64 / CPH heads at a time. The first rot_dims / 16 lanes of a
 // head own 8 neighbouring pairs (elements 8c .. 8c + 7 and those rot_dims / 2 further), the others 16
-// unrotated elements (cos 1, sin 0). cos / sin of the token go through the wave's LDS row (one sincos
+// unrotated elements (cos 1, sin 0). Interleaved pairs: a lane's two runs are 16 neighbouring elements, the same
+// pairs 8c .. 8c + 7, both elements of a pair in one run. cos / sin of the token go through the wave's LDS row (one sincos
 // per lane). A wave takes the head rounds r = blockIdx.y, + gridDim.y, ...; the last y also copies
 // value columns of their own into the V page.
 __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const RopeHeadnormParams P, int64_t T_rows) {
@@ -290,7 +293,9 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const R
   const int hpr = 64 / CPH;                // heads per round
   const int c8 = (lane & (CPH - 1)) * 8, hsub = lane / CPH;
   const bool rot = c8 < rhalf;                       // (a lane's pairs are all rotated or none is)
-  const int ea = rot ? c8 : 2 * c8, eb = rot ? rhalf + c8 : 2 * c8 + 8;   // the lane's two runs of the head
+  // the lane's two runs of the head
+  const bool halves = rot && !P.interleaved;
+  const int ea = halves ? c8 : 2 * c8, eb = halves ? rhalf + c8 : 2 * c8 + 8;
   const int heads = P.H + P.G;
   float cc[8], sv[8];
 #pragma unroll
@@ -323,25 +328,37 @@ __global__ void __launch_bounds__(256) rope_headnorm_cache_bf16x8_kernel(const R
       ss += xa[j] * xa[j] + xb[j] * xb[j];
     }
     const float* w = is_k ? P.k_w : P.q_w;
-    if (P.q_w != nullptr || P.k_w != nullptr) {   // (wave-uniform: the shuffles run in every lane)
+    const bool normed = w != nullptr || P.unit;
+    if (P.q_w != nullptr || P.k_w != nullptr || P.unit) {   // (wave-uniform: the shuffles run in every lane)
       for (int o = CPH >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
-      if (live && w != nullptr) {
+      if (live && normed) {
         const float r = 1.0f / sqrtf(ss / (float)dk + P.eps);
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          xa[j] *= r * w[ea + j];
-          xb[j] *= r * w[eb + j];
+          xa[j] *= w != nullptr ? r * w[ea + j] : r;
+          xb[j] *= w != nullptr ? r * w[eb + j] : r;
         }
       }
     }
     if (!live) continue;
     u16x8 oa, ob;
+    if (P.interleaved) {
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {   // (u, v) -> (u cos - v sin, v cos + u sin)
-      oa[j] = f2bf(xa[j] * cc[j] - xb[j] * sv[j]);
-      ob[j] = f2bf(xb[j] * cc[j] + xa[j] * sv[j]);
+      for (int j = 0; j < 4; ++j) {   // pairs j and j + 4 of the lane
+        const float ua = xa[2 * j], va = xa[2 * j + 1], ub = xb[2 * j], vb = xb[2 * j + 1];
+        oa[2 * j] = f2bf(ua * cc[j] - va * sv[j]);
+        oa[2 * j + 1] = f2bf(va * cc[j] + ua * sv[j]);
+        ob[2 * j] = f2bf(ub * cc[j + 4] - vb * sv[j + 4]);
+        ob[2 * j + 1] = f2bf(vb * cc[j + 4] + ub * sv[j + 4]);
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {   // (u, v) -> (u cos - v sin, v cos + u sin)
+        oa[j] = f2bf(xa[j] * cc[j] - xb[j] * sv[j]);
+        ob[j] = f2bf(xb[j] * cc[j] + xa[j] * sv[j]);
+      }
     }
-    if (rot || w != nullptr) {
+    if (rot || normed) {
       store8(src + ea, oa);
       store8(src + eb, ob);
     }

@@ -15,6 +15,8 @@
 //   residual_add_rmsnorm   x[t] += y[t], out[t] = rmsnorm(x[t]) * w: the residual sum of one
 //                     pre-norm sub-layer and the norm in front of the next in one pass; y[t] may be
 //                     the sum of a token's expert rows (inv: their k row numbers, < 0: none)
+//   residual_step     x += m * (y + y2), or m * (rmsnorm(y) w1 + rmsnorm(y2) w2), or m times the sum of gathered
+//                     rows of y (+ y2); then fp32 rows and one row added; then the next norm
 //   clamped_glu       [gate F | up F | ...] -> g sigmoid(alpha g) (u + shift), g = min(gate, limit),
 //                     u = clamp(up, +-limit), optionally times sigmoid of one gate column of the row
 //   group_rmsnorm     RMS norm of each of G equal column groups of fp32 rows (heads), weight per
@@ -345,6 +347,194 @@ bool launch_residual_step_vec(float* x, const uint16_t* y, int64_t y_stride, con
   }
 #undef NGA_STEP
   return true;
+}
+
+// The general step (see ResidualStepParams), any width. Each thread re-reads only the columns it wrote itself.
+template <typename T>
+__global__ void __launch_bounds__(256) residual_step_kernel(const ResidualStepParams P) {
+  __shared__ float red[4];
+  const int64_t row = blockIdx.x;
+  const int H = P.H;
+  float* xr = P.x + row * H;
+  const T* y = (const T*)P.y + (P.inv ? 0 : row * P.ys);
+  const T* y2 = (const T*)P.y2 + row * P.y2s;
+  float r1 = 0.f, r2 = 0.f;
+  if (P.w1) {
+    float s1 = 0.f, s2 = 0.f;
+    for (int c = threadIdx.x; c < H; c += blockDim.x) {
+      const float a = ldf(y + c), b = ldf(y2 + c);
+      s1 += a * a;
+      s2 += b * b;
+    }
+    r1 = 1.0f / sqrtf(block_sum(s1, red) / (float)H + P.eps);
+    __syncthreads();
+    r2 = 1.0f / sqrtf(block_sum(s2, red) / (float)H + P.eps);
+    __syncthreads();
+  }
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < H; c += blockDim.x) {
+    float a = 0.f;
+    if (P.inv) {
+      for (int j = 0; j < P.k; ++j) {
+        const int p = P.inv[row * P.k + j];
+        if (p >= 0) a += ldf(y + (int64_t)p * P.ys + c);
+      }
+    } else if (P.w1) {
+      a = ldf(y + c) * r1 * P.w1[c] + ldf(y2 + c) * r2 * P.w2[c];
+    } else if (P.y) {
+      a = ldf(y + c);
+    }
+    if (P.y2 && !P.w1) a += ldf(y2 + c);
+    float v = xr[c] + P.mult * a;
+    if (P.x0) v += P.x0[row * H + c];
+    if (P.row) v += P.row[c];
+    xr[c] = v;
+    ss += v * v;
+  }
+  if (!P.w) return;
+  const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)H + P.eps);
+  for (int c = threadIdx.x; c < H; c += blockDim.x) stf((T*)P.out + row * H + c, xr[c] * r * P.w[c]);
+}
+
+// The same for bf16 rows with H % 4 == 0 and aligned rows, the row in registers: TPR threads per row (a wave, or the
+// workgroup when the rows are few), NV runs of four elements per thread, one read and one write of the stream.
+template <int TPR, int NV, bool PAIR>
+__global__ void __launch_bounds__(256) residual_step_general_bf16x4_kernel(const ResidualStepParams P, int64_t T_rows) {
+  __shared__ float red[2][4];
+  const int64_t row = TPR == 64 ? (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6) : (int64_t)blockIdx.x;
+  if (row >= T_rows) return;                 // (whole waves / workgroups)
+  const int l = TPR == 64 ? threadIdx.x & 63 : threadIdx.x;
+  const int H = P.H;
+  float* xr = P.x + row * H;
+  const uint16_t* y = (const uint16_t*)P.y;
+  const uint16_t* y2 = P.y2 ? (const uint16_t*)P.y2 + row * P.y2s : nullptr;
+  auto get = [](const uint16_t* p) {
+    const u16x4 a = *reinterpret_cast<const u16x4*>(p);
+    return make_float4(bf2f(a[0]), bf2f(a[1]), bf2f(a[2]), bf2f(a[3]));
+  };
+  float4 xv[NV], a[NV], b[PAIR ? NV : 1];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * (l + TPR * i);
+    xv[i] = a[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if constexpr (PAIR) b[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (c < H) {
+      xv[i] = *reinterpret_cast<const float4*>(xr + c);
+      if (y && !P.inv) a[i] = get(y + row * P.ys + c);
+      if constexpr (PAIR) {
+        b[i] = get(y2 + c);
+      } else if (y2) {
+        const float4 t = get(y2 + c);
+        a[i].x += t.x, a[i].y += t.y, a[i].z += t.z, a[i].w += t.w;
+      }
+    }
+  }
+  if (!PAIR && P.inv) {
+    for (int j = 0; j < P.k; ++j) {
+      const int p = P.inv[row * P.k + j];
+      if (p < 0) continue;
+      const uint16_t* pr = y + (int64_t)p * P.ys;
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = 4 * (l + TPR * i);
+        if (c < H) {
+          const float4 t = get(pr + c);
+          a[i].x += t.x, a[i].y += t.y, a[i].z += t.z, a[i].w += t.w;
+        }
+      }
+    }
+  }
+  auto sq = [](const float4& v) { return v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w; };
+  if constexpr (PAIR) {
+    float s1 = 0.f, s2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      s1 += sq(a[i]);
+      s2 += sq(b[i]);
+    }
+    s1 = wave_sum(s1);
+    s2 = wave_sum(s2);
+    if constexpr (TPR != 64) {
+      if ((threadIdx.x & 63) == 0) {
+        red[0][threadIdx.x >> 6] = s1;
+        red[1][threadIdx.x >> 6] = s2;
+      }
+      __syncthreads();
+      s1 = red[0][0] + red[0][1] + red[0][2] + red[0][3];
+      s2 = red[1][0] + red[1][1] + red[1][2] + red[1][3];
+      __syncthreads();
+    }
+    const float r1 = 1.0f / sqrtf(s1 / (float)H + P.eps), r2 = 1.0f / sqrtf(s2 / (float)H + P.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = 4 * (l + TPR * i);
+      if (c < H) {
+        const float4 u = *reinterpret_cast<const float4*>(P.w1 + c), v = *reinterpret_cast<const float4*>(P.w2 + c);
+        a[i] = make_float4(a[i].x * r1 * u.x + b[i].x * r2 * v.x, a[i].y * r1 * u.y + b[i].y * r2 * v.y,
+                           a[i].z * r1 * u.z + b[i].z * r2 * v.z, a[i].w * r1 * u.w + b[i].w * r2 * v.w);
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * (l + TPR * i);
+    if (c >= H) continue;
+    float4 v = make_float4(xv[i].x + P.mult * a[i].x, xv[i].y + P.mult * a[i].y, xv[i].z + P.mult * a[i].z,
+                           xv[i].w + P.mult * a[i].w);
+    if (P.x0) {
+      const float4 t = *reinterpret_cast<const float4*>(P.x0 + row * H + c);
+      v.x += t.x, v.y += t.y, v.z += t.z, v.w += t.w;
+    }
+    if (P.row) {
+      const float4 t = *reinterpret_cast<const float4*>(P.row + c);
+      v.x += t.x, v.y += t.y, v.z += t.z, v.w += t.w;
+    }
+    *reinterpret_cast<float4*>(xr + c) = v;
+    xv[i] = v;
+    ss += sq(v);
+  }
+  if (!P.w) return;
+  ss = wave_sum(ss);
+  if constexpr (TPR != 64) {
+    if ((threadIdx.x & 63) == 0) red[0][threadIdx.x >> 6] = ss;
+    __syncthreads();
+    ss = red[0][0] + red[0][1] + red[0][2] + red[0][3];
+  }
+  const float r = 1.0f / sqrtf(ss / (float)H + P.eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * (l + TPR * i);
+    if (c < H) {
+      const float4 u = *reinterpret_cast<const float4*>(P.w + c);
+      u16x4 o;
+      o[0] = f2bf(xv[i].x * r * u.x);
+      o[1] = f2bf(xv[i].y * r * u.y);
+      o[2] = f2bf(xv[i].z * r * u.z);
+      o[3] = f2bf(xv[i].w * r * u.w);
+      *reinterpret_cast<u16x4*>((uint16_t*)P.out + row * H + c) = o;
+    }
+  }
+}
+
+template <bool PAIR>
+void launch_residual_step_general(const ResidualStepParams& p, int64_t T, hipStream_t stream) {
+#define NGA_STEP(TPR, NV)                                                                                       \
+  residual_step_general_bf16x4_kernel<TPR, NV, PAIR>                                                            \
+      <<<dim3((unsigned)(TPR == 64 ? (T + 3) / 4 : T)), 256, 0, stream>>>(p, T)
+  if (T >= 4096 && p.H <= 4096) {      // rows enough to fill the chip with one wave each
+    if (p.H <= 256) NGA_STEP(64, 1);
+    else if (p.H <= 512) NGA_STEP(64, 2);
+    else if (p.H <= 1024) NGA_STEP(64, 4);
+    else if (p.H <= 2048) NGA_STEP(64, 8);
+    else NGA_STEP(64, 16);
+  } else {
+    if (p.H <= 1024) NGA_STEP(256, 1);
+    else if (p.H <= 2048) NGA_STEP(256, 2);
+    else if (p.H <= 4096) NGA_STEP(256, 4);
+    else NGA_STEP(256, 8);
+  }
+#undef NGA_STEP
 }
 
 template <typename T>
@@ -817,6 +1007,19 @@ void launch_residual_add_rmsnorm(float* x, const void* y, int64_t y_stride, cons
   else
     residual_add_rmsnorm_kernel<uint16_t><<<dim3((unsigned)T), 256, 0, stream>>>(x, (const uint16_t*)y, y_stride, w, eps,
                                                                                 H, (uint16_t*)out, inv, k);
+}
+
+void launch_residual_step(const ResidualStepParams& p, int64_t T, bool f32, hipStream_t stream) {
+  if (T == 0) return;
+  auto al = [](const void* q, int a) { return ((uintptr_t)q % a) == 0; };
+  if (f32) {
+    residual_step_kernel<float><<<dim3((unsigned)T), 256, 0, stream>>>(p);
+  } else if (p.H % 4 == 0 && p.H <= 8192 && p.ys % 4 == 0 && p.y2s % 4 == 0 && al(p.x, 16) && al(p.y, 8) && al(p.y2, 8) &&
+             al(p.w1, 16) && al(p.w2, 16) && al(p.x0, 16) && al(p.row, 16) && al(p.w, 16) && al(p.out, 8)) {
+    p.w1 ? launch_residual_step_general<true>(p, T, stream) : launch_residual_step_general<false>(p, T, stream);
+  } else {
+    residual_step_kernel<uint16_t><<<dim3((unsigned)T), 256, 0, stream>>>(p);
+  }
 }
 
 void launch_clamped_glu(void* out, const void* in, int64_t in_stride, int64_t T, int F, float limit, float alpha,

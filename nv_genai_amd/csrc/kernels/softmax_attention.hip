@@ -18,7 +18,7 @@
 // `maps` score maps (1 or 2) that share its values: q head (h, m) is column block h * maps + m,
 // its keys are k head (h / (H / G)) * maps + m. Two maps combine as a_0 - lam * a_1
 // (differential attention). Optional: unit RMS of the head output (eps inside the root) times
-// out_scale, and a per-head sigmoid gate; a sink: one more key of a given score without a value. Visible
+// out_scale, and a sigmoid gate per head or per output element (g_dim = 1 or dv gates per head); a sink: one more key of a given score without a value. Visible
 // keys of the query at position i: j <= i, i - j < window when window > 0, and, when chunk > 0, keys of
 // the query's own chunk only (j >= floor(i / chunk) chunk). v_row: elements between two value rows of a page; v_row = dk with
 // vc = kc reads the values out of the first dv elements of the key rows (one map: a latent that is
@@ -49,6 +49,10 @@ template <> __device__ __forceinline__ void stf<uint16_t>(uint16_t* p, float v) 
 template <> __device__ __forceinline__ void stf<float>(float* p, float v) { *p = v; }
 
 __device__ __forceinline__ float sigmoidf_(float z) { return 1.0f / (1.0f + expf(-z)); }
+// on the hardware exp2 and reciprocal, for results that are rounded to bf16
+__device__ __forceinline__ float fast_sigmoid(float z) {
+  return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
 
 // q . k over dk elements, q in LDS (fp32), k a page row; 16-byte loads when vec
 __device__ __forceinline__ float dot_row(const float* qs, const uint16_t* kr, int dk, bool vec) {
@@ -128,10 +132,10 @@ __global__ void __launch_bounds__(256) headnorm_cache_kernel(
 }
 
 // One wave per (token row, head). q: row stride q_stride, head (h, m) at (h * maps + m) * dk.
-// gate: row stride g_stride, one pre-sigmoid value per head (nullptr: no gate). out [T, H * dv].
+// gate: row stride g_stride, g_dim pre-sigmoid values per head (1 or dv; nullptr: no gate). out [T, H * dv].
 template <typename T>
 __global__ void __launch_bounds__(64) softmax_attention_kernel(
-    T* __restrict__ out, const T* __restrict__ q, int64_t q_stride, const T* __restrict__ gate, int64_t g_stride,
+    T* __restrict__ out, const T* __restrict__ q, int64_t q_stride, const T* __restrict__ gate, int64_t g_stride, int g_dim,
     const T* __restrict__ kc, const T* __restrict__ vc, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ pos, int H, int G, int dk, int dv, float scale,
     int window, int maps, float lam, float unit_eps, float out_scale, int v_row, float softcap, int chunk, float sink,
@@ -208,11 +212,12 @@ __global__ void __launch_bounds__(64) softmax_attention_kernel(
     ss = wave_sum(ss);
     r = out_scale / sqrtf(ss / (float)dv + unit_eps);
   }
-  if (gate) r *= sigmoidf_(ldf(gate + row * g_stride + h));
+  const T* gr = gate ? gate + row * g_stride + (int64_t)h * g_dim : nullptr;
+  if (gr && g_dim == 1) r *= sigmoidf_(ldf(gr));
 #pragma unroll
   for (int u = 0; u < MAXV; ++u) {
     const int d = lane + u * 64;
-    if (d < dv) stf(orow + d, res[u] * r);
+    if (d < dv) stf(orow + d, gr && g_dim > 1 ? res[u] * r * sigmoidf_(ldf(gr + d)) : res[u] * r);
   }
 }
 
@@ -240,7 +245,7 @@ __device__ __forceinline__ int sm_row_swz(int row) { return (row & 3) | (((row >
 struct SmMfmaParams {
   uint16_t* out;             // [T, H * DV], row stride o_stride
   const uint16_t* q;         // row stride q_stride, head (h, m) at (h * MAPS + m) * DK
-  const uint16_t* gate;      // row stride g_stride, one value per head (nullptr: none)
+  const uint16_t* gate;      // row stride g_stride, g_dim values per head (nullptr: none)
   const uint16_t* kc;
   const uint16_t* vc;
   const int32_t* block_tables;
@@ -254,7 +259,33 @@ struct SmMfmaParams {
   int chunk;                 // > 0: keys of the query's own chunk only
   float sink_log2;           // score of a key without a value times log2 e (-inf: none)
   int64_t o_stride;
+  int g_dim;                 // gates per head: 1 or DV
 };
+
+// A query's output columns 16 dt + 4 h .. + 3 of one head, times rs and its gate(s), in bf16.
+template <int DT>
+__device__ __forceinline__ void sm_store_gated(const SmMfmaParams& P, int64_t row, int head, int h, const f32x4* o, float rs) {
+  const uint16_t* gp = P.gate ? P.gate + row * P.g_stride + (int64_t)head * P.g_dim : nullptr;
+  const bool each = gp && P.g_dim > 1;
+  if (gp && !each) rs *= sigmoidf_(bf2f(*gp));
+  uint16_t* op = P.out + row * P.o_stride + (int64_t)head * (16 * DT);
+  u16x4 gv[DT];
+  if (each) {
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) gv[dt] = *reinterpret_cast<const u16x4*>(gp + 16 * dt + 4 * h);
+  }
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt) {
+    u16x4 ov;
+#pragma unroll
+    for (int rr = 0; rr < 4; ++rr) {
+      float v = o[dt][rr] * rs;
+      if (each) v *= fast_sigmoid(bf2f(gv[dt][rr]));
+      ov[rr] = f2bf(v);
+    }
+    *reinterpret_cast<u16x4*>(op + 16 * dt + 4 * h) = ov;
+  }
+}
 
 // WPE: waves per SIMD the register allocation aims at. Large tiles (maps x DK + DV >= 192) are
 // compiled for two: with the whole register file the scheduler keeps a tile's LDS reads in flight
@@ -506,15 +537,7 @@ softmax_attention_mfma_kernel(const SmMfmaParams P) {
       }
       if (row_ok) {
         const int head = 2 * hq + m;
-        if (P.gate) rs *= sigmoidf_(bf2f(P.gate[(int64_t)(q0 + r) * P.g_stride + head]));
-        uint16_t* op = P.out + (int64_t)(q0 + r) * P.o_stride + (int64_t)head * DV;
-#pragma unroll
-        for (int dt = 0; dt < DT; ++dt) {
-          u16x4 ov;
-#pragma unroll
-          for (int rr = 0; rr < 4; ++rr) ov[rr] = f2bf(o[m][dt][rr] * rs);
-          *reinterpret_cast<u16x4*>(op + 16 * dt + 4 * h) = ov;
-        }
+        sm_store_gated<DT>(P, (int64_t)(q0 + r), head, h, o[m], rs);
       }
     }
     return;
@@ -536,15 +559,7 @@ softmax_attention_mfma_kernel(const SmMfmaParams P) {
     rs = P.out_scale / sqrtf(ss / (float)DV + P.unit_eps);
   }
   if (!row_ok) return;
-  if (P.gate) rs *= sigmoidf_(bf2f(P.gate[(int64_t)(q0 + r) * P.g_stride + hq]));
-  uint16_t* op = P.out + (int64_t)(q0 + r) * P.o_stride + (int64_t)hq * DV;
-#pragma unroll
-  for (int dt = 0; dt < DT; ++dt) {
-    u16x4 ov;
-#pragma unroll
-    for (int rr = 0; rr < 4; ++rr) ov[rr] = f2bf(o[0][dt][rr] * rs);
-    *reinterpret_cast<u16x4*>(op + 16 * dt + 4 * h) = ov;
-  }
+  sm_store_gated<DT>(P, (int64_t)(q0 + r), hq, h, o[0], rs);
 }
 
 template <int DK, int DV, int MAPS>
@@ -867,7 +882,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
 // one wave per (token row, head): merge the partials of each map, a_0 - lam * a_1, unit RMS, gate
 __global__ void __launch_bounds__(64) softmax_decode_reduce_kernel(
     uint16_t* __restrict__ out, const float* __restrict__ ws, int slots, const uint16_t* __restrict__ gate,
-    int64_t g_stride, int H, int dv, int maps, float lam, float unit_eps, float out_scale, float sink_log2,
+    int64_t g_stride, int g_dim, int H, int dv, int maps, float lam, float unit_eps, float out_scale, float sink_log2,
     int64_t o_stride) {
   const int64_t row = blockIdx.x;
   const int head = blockIdx.y, lane = threadIdx.x;
@@ -903,10 +918,14 @@ __global__ void __launch_bounds__(64) softmax_decode_reduce_kernel(
     ss = wave_sum(ss);
     r = out_scale / sqrtf(ss / (float)dv + unit_eps);
   }
-  if (gate) r *= sigmoidf_(bf2f(gate[row * g_stride + head]));
+  const uint16_t* gr = gate ? gate + row * g_stride + (int64_t)head * g_dim : nullptr;
+  if (gr && g_dim == 1) r *= sigmoidf_(bf2f(*gr));
 #pragma unroll
   for (int u = 0; u < MAXV; ++u)
-    if (lane + 64 * u < dv) out[row * o_stride + (int64_t)head * dv + lane + 64 * u] = f2bf(res[u] * r);
+    if (lane + 64 * u < dv) {
+      const float f = gr && g_dim > 1 ? r * fast_sigmoid(bf2f(gr[lane + 64 * u])) : r;
+      out[row * o_stride + (int64_t)head * dv + lane + 64 * u] = f2bf(res[u] * f);
+    }
 }
 
 template <int DK, int DV, int MAPS>
@@ -995,7 +1014,7 @@ int softmax_decode_parts(int rows, int G, int max_ctx, int window) {
 
 // ws: fp32 [T, H, maps, parts, dv + 4]
 void launch_softmax_decode_mfma(uint16_t* out, int64_t o_stride, float* ws, int parts, const uint16_t* q, int64_t q_stride,
-                                const uint16_t* gate, int64_t g_stride, const uint16_t* kc, const uint16_t* vc,
+                                const uint16_t* gate, int64_t g_stride, int g_dim, const uint16_t* kc, const uint16_t* vc,
                                 const int32_t* block_tables, int max_blocks, const int32_t* tok_seq,
                                 const int32_t* pos, int64_t T, int H, int G, int dk, int dv, float scale, int window,
                                 int maps, float lam, float unit_eps, float out_scale, bool v_in_k, float softcap,
@@ -1010,7 +1029,7 @@ void launch_softmax_decode_mfma(uint16_t* out, int64_t o_stride, float* ws, int 
                             : launch_sm_decode_dk<1>(ws, q, q_stride, kc, vc, block_tables, max_blocks, tok_seq, pos, H, G,
                                                      scale_log2, cap_log2, window, v_row, chunk, dk, dv, grid, stream);
   if (!ok) abort();   // the caller checks softmax_attention_mfma_supported
-  softmax_decode_reduce_kernel<<<dim3((unsigned)T, (unsigned)H), 64, 0, stream>>>(out, ws, parts, gate, g_stride, H,
+  softmax_decode_reduce_kernel<<<dim3((unsigned)T, (unsigned)H), 64, 0, stream>>>(out, ws, parts, gate, g_stride, g_dim, H,
                                                                                    dv, maps, lam, unit_eps, out_scale,
                                                                                    sink * 1.4426950408889634f, o_stride);
 }
@@ -1027,7 +1046,7 @@ bool softmax_attention_mfma_supported(int dk, int dv, int group, int maps) {
 // prompt portions: sequence b owns rows [cu_q[b], cu_q[b + 1]) of q / gate / out, the last ones of
 // its ctx_lens[b] keys. q rows must be 16-byte aligned (checked by the caller).
 void launch_softmax_attention_mfma(uint16_t* out, int64_t o_stride, const uint16_t* q, int64_t q_stride, const uint16_t* gate,
-                                   int64_t g_stride, const uint16_t* kc, const uint16_t* vc,
+                                   int64_t g_stride, int g_dim, const uint16_t* kc, const uint16_t* vc,
                                    const int32_t* block_tables, int max_blocks, const int32_t* cu_q,
                                    const int32_t* ctx_lens, int B, int max_q_len, int H, int G, int dk, int dv,
                                    float scale, int window, int maps, float lam, float unit_eps, float out_scale,
@@ -1036,7 +1055,7 @@ void launch_softmax_attention_mfma(uint16_t* out, int64_t o_stride, const uint16
   SmMfmaParams P{out, q, gate, kc, vc, block_tables, cu_q, ctx_lens, q_stride, g_stride, max_blocks, H, G, window,
                  scale * 1.4426950408889634f, lam, unit_eps, out_scale,
                  softcap > 0.f ? softcap * 1.4426950408889634f : 0.f, v_in_k ? dk : dv, chunk,
-                 sink * 1.4426950408889634f, o_stride};
+                 sink * 1.4426950408889634f, o_stride, g_dim};
   const dim3 grid((unsigned)H, (unsigned)B, (unsigned)((max_q_len + 63) / 64));   // (head, sequence, row block)
   const bool ok = maps == 2 ? launch_sm_mfma_dk<2>(P, dk, dv, grid, stream) : launch_sm_mfma_dk<1>(P, dk, dv, grid, stream);
   if (!ok) abort();   // the caller checks softmax_attention_mfma_supported
@@ -1057,7 +1076,7 @@ void launch_headnorm_cache(void* proj, int64_t stride, const int32_t* slots, voi
 }
 
 void launch_softmax_attention(void* out, int64_t o_stride, const void* q, int64_t q_stride, const void* gate, int64_t g_stride,
-                              const void* kc, const void* vc, const int32_t* block_tables, int max_blocks,
+                              int g_dim, const void* kc, const void* vc, const int32_t* block_tables, int max_blocks,
                               const int32_t* tok_seq, const int32_t* pos, int64_t T, int H, int G, int dk, int dv,
                               float scale, int window, int maps, float lam, float unit_eps, float out_scale, bool v_in_k,
                               float softcap, int chunk, float sink, bool f32, hipStream_t stream) {
@@ -1067,12 +1086,12 @@ void launch_softmax_attention(void* out, int64_t o_stride, const void* q, int64_
   const size_t smem = (size_t)(maps * dk + 64) * sizeof(float);
   if (f32)
     softmax_attention_kernel<float><<<grid, 64, smem, stream>>>(
-        (float*)out, (const float*)q, q_stride, (const float*)gate, g_stride, (const float*)kc, (const float*)vc,
+        (float*)out, (const float*)q, q_stride, (const float*)gate, g_stride, g_dim, (const float*)kc, (const float*)vc,
         block_tables, max_blocks, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam, unit_eps, out_scale, v_row,
         softcap, chunk, sink, o_stride);
   else
     softmax_attention_kernel<uint16_t><<<grid, 64, smem, stream>>>(
-        (uint16_t*)out, (const uint16_t*)q, q_stride, (const uint16_t*)gate, g_stride, (const uint16_t*)kc,
+        (uint16_t*)out, (const uint16_t*)q, q_stride, (const uint16_t*)gate, g_stride, g_dim, (const uint16_t*)kc,
         (const uint16_t*)vc, block_tables, max_blocks, tok_seq, pos, H, G, dk, dv, scale, window, maps, lam, unit_eps,
         out_scale, v_row, softcap, chunk, sink, o_stride);
 }
