@@ -1,10 +1,10 @@
-"""The layer-list designs (Bidasun, Biruvik, Lumepel, Lizezen, Vivesun) beside the closest Llama-layout model
-at equal sizes (Mistral with a sliding window; Mixtral for Lumepel, Lizezen and Vivesun, whose
-feed-forwards are routed experts):
+"""The layer-list designs (Bidasun, Biruvik, Lumepel, Lizezen, Vivesun, Kevelorn) beside the closest Llama-layout
+model at equal sizes (Mistral with a sliding window; Mixtral for Lumepel, Lizezen, Vivesun and Kevelorn, whose
+feed-forwards are routed experts; Kevelorn also beside Vivesun):
 prefill and decode throughput through the serving engine, and the design's kernels alone with
 their distance from the roofline. Random weights, synthetic token ids.
 
-    python bench.py --workload designs [--design-sizes s,m,l] [--design-models bidasun,biruvik,lumepel,lizezen,vivesun]
+    python bench.py --workload designs [--design-sizes s,m,l] [--design-models bidasun,biruvik,lumepel,lizezen,vivesun,kevelorn]
 
 Prints one JSON line (``metric: design_compare``); bench.py's default workload is untouched.
 """
@@ -43,15 +43,28 @@ LIZEZEN_MLSTM = dict(dim=64, vdim=128)
 # heads over the whole width, expert sizes of LUMEPEL, a bigram table and a token input
 VIVESUN_PATTERN = ("delta", "parallel")
 VIVESUN = dict(dim=128, vdim=128, conv=4, rdim=64, rank=64, rot=64, side=256, bigram=(65521, 40503, 9973))
-BASELINE_OF = {"bidasun": "mistral", "biruvik": "mistral", "lumepel": "mixtral", "lizezen": "mixtral", "vivesun": "mixtral"}
+# Kevelorn: windowed attention (the window of the other designs, interleaved rotation on the whole head) beside
+# a lightning recurrence, GLA and lightning layers with states of 128 x 128 per head, expert sizes of LUMEPEL
+# with a shared expert in every layer, no repeated span (layer counts stay equal)
+KEVELORN_PATTERN = ("parallel", "gla", "lightning", "gla")
+KEVELORN = dict(dim=128, vdim=128, rank=64, tau=16.0, mult=0.3)
+BASELINE_OF = {"bidasun": ("mistral",), "biruvik": ("mistral",), "lumepel": ("mixtral",), "lizezen": ("mixtral",),
+               "vivesun": ("mixtral",), "kevelorn": ("vivesun", "mixtral")}
 
 
 def _engine(kind: str, z: dict, max_len: int, pages: int, seqs: int):
     from nv_genai_amd.engine.llm_engine import EngineConfig, LLMEngine
     from nv_genai_amd.models.config import LlamaConfig, bidasun_uniform, biruvik_layers, lizezen_layers, lumepel_layers
-    from nv_genai_amd.models.config import vivesun_layers
+    from nv_genai_amd.models.config import kevelorn_layers, vivesun_layers
 
-    if kind == "vivesun":
+    if kind == "kevelorn":
+        u, v = z["lumepel"], KEVELORN
+        pat = [KEVELORN_PATTERN[i % len(KEVELORN_PATTERN)] for i in range(z["layers"])]
+        mcfg = kevelorn_layers(pat, z["hidden"], z["heads"], z["kv"], z["d"], z["d"], window=z["window"],
+                               rec_heads=z["heads"], rec_dim=v["dim"], rec_vdim=v["vdim"], tau=v["tau"], rank=v["rank"],
+                               experts=u["experts"], top=u["top"], expert_ff=u["eff"], shared_ff=u["eff"], rot_base=1e6,
+                               rot_factor=4.0, residual_mult=v["mult"], vocab_size=VOCAB)
+    elif kind == "vivesun":
         u, v = z["lumepel"], VIVESUN
         pat = [VIVESUN_PATTERN[i % len(VIVESUN_PATTERN)] for i in range(z["layers"])]
         mcfg = vivesun_layers(pat, z["hidden"], z["heads"], z["kv"], z["d"], z["d"], chunk=z["window"],
@@ -713,6 +726,156 @@ def vivesun_kernel_times(z: dict, iters: int = 20) -> dict:
     return out
 
 
+def kevelorn_kernel_times(z: dict, iters: int = 20) -> dict:
+    """The Kevelorn kernels alone on one layer's shapes beside the like kernels of the other models: the
+    diagonal linear scans against the delta-rule scans of Vivesun (a constant decay beside the gated rule,
+    channel decays beside the channel-wise rule; equal state sizes; fp32 flops per state element and row: 5, 7
+    and 9), windowed attention with a gate per element against the windowed Llama-layout kernels, SwiGLU
+    experts against the Mixtral experts, and the row kernels against theirs, priced by the flops or bytes
+    they must move."""
+    from nv_genai_amd import ops
+    from nv_genai_amd.ops import reference as ref
+
+    dev, bf = "cuda", torch.bfloat16
+    u, v = z["lumepel"], KEVELORN
+    H, G, D, W, Hd = z["heads"], z["kv"], z["d"], z["window"], z["hidden"]
+    nb, L = z["pf"]
+    nd, ctx = z["dec"]
+    T = nb * L
+    cu = torch.arange(0, T + 1, L, dtype=torch.int32, device=dev)
+    posr = torch.arange(L, dtype=torch.int32, device=dev).repeat(nb)
+    sl_p = torch.arange(nb, dtype=torch.int32, device=dev)
+    sl_d = torch.arange(nd, dtype=torch.int32, device=dev)
+    posd = torch.full((nd,), ctx - 1, dtype=torch.int32, device=dev)
+    out = {"scan": {}}
+    # ---- scans: prompts (nb segments of L rows) and single rows (nd segments)
+    d, dv = v["dim"], v["vdim"]
+    nq, nv = H * d, H * dv
+    proj = torch.randn(T, 4 * nq + nv + 2 * H, device=dev).to(bf)
+    c = [proj[:, i * nq:(i + 1) * nq] for i in range(4)]
+    vv, ba = proj[:, 4 * nq:4 * nq + nv], proj[:, 4 * nq + nv:]
+    xq = torch.randn(T, nq + nv, device=dev).to(bf)                        # q / k heads shared by two value heads
+    st = torch.zeros(max(nb, nd), H, d, dv, device=dev)
+    zb, ld = torch.ones(nq, device=dev), torch.linspace(-0.7, -0.004, H, device=dev)
+    hz, hb = torch.zeros(H, device=dev), torch.full((H,), -2.0, device=dev)
+    nz, nb3 = torch.zeros(nq, device=dev), torch.full((nq,), -3.0, device=dev)
+
+    def both(fn):
+        return (_timed_gpu(lambda: fn(slice(None), dict(cu=cu, slots=sl_p, pos=posr, max_q=L)), iters),
+                _timed_gpu(lambda: fn(slice(nd), dict(cu=None, slots=sl_d, pos=posd)), iters))
+
+    runs = {
+        "gla": (5.0, lambda r, s: ops.linear_scan(c[0][r], c[1][r], vv[r], st, H, d, dv, z=c[2][r], z_bias=zb, tau=v["tau"],
+                                                  q_scale=d ** -0.5, **s)),
+        "channel_delta": (9.0, lambda r, s: ops.channel_delta_scan(c[0][r], c[1][r], vv[r], c[2][r], c[3][r], nz, nb3, st, H,
+                                                                   d, dv, 0.6065306597126334, **s)),
+        "lightning": (5.0, lambda r, s: ops.linear_scan(c[0][r], c[1][r], vv[r], st, H, d, dv, log_decay=ld, silu=True, **s)),
+        "gated_delta": (7.0, lambda r, s: ops.gated_delta_scan(xq[r], ba[r], hz, hb, st, H, H // 2, d, dv, **s))}
+    for name, (flops, fn) in runs.items():
+        t_p, t_d = both(fn)
+        out["scan"][name] = {"prefill_ms": round(t_p * 1e3, 3), "fp32_frac": round(flops * T * H * d * dv / t_p / PEAK_VALU, 4),
+                             "decode_ms": round(t_d * 1e3, 4),
+                             "state_hbm_frac": round(nd * H * d * dv * 8.0 / t_d / PEAK_HBM, 4)}
+    del proj, c, vv, ba, xq, st
+    # ---- attention: window and a gate per element on row-major pages against the windowed Llama-layout kernels
+    pages_seq = -(-max(L, ctx) // 64)
+    nseq = max(nb, nd)
+    npg = nseq * pages_seq
+    bt = torch.arange(npg, dtype=torch.int32, device=dev).view(nseq, pages_seq)
+    kr = (torch.randn(npg, G, 64, D, device=dev) * 0.5).to(bf)
+    vr = (torch.randn(npg, G, 64, D, device=dev) * 0.5).to(bf)
+    vt = (torch.randn(npg, G, D, 64, device=dev) * 0.5).to(bf)
+    cx = torch.full((nb,), L, dtype=torch.int32, device=dev)
+    q1 = torch.randn(T, H * D, device=dev).to(bf)
+    gt = torch.randn(T, H * D, device=dev).to(bf)
+    pairs = nb * sum(min(i + 1, W) for i in range(L)) * H
+    sc = D ** -0.5
+    out["mfma_attention"] = bool(ops.softmax_attention_mfma_ok(q1, D, D, H // G, 1))
+    kw = dict(scale=sc, window=W)
+    cxd = torch.full((nd,), ctx, dtype=torch.int32, device=dev)
+    ws = ops.DecodeWorkspace(nd, H, G, ctx, dev, None, D=D)
+    kvb = nd * G * 2 * D * 2.0 * min(ctx, W)
+    att = {
+        "gated_window": (lambda: ops.softmax_attention_prefill(q1, kr, vr, bt, cu, cx, L, H, G, D, D, gate=gt, **kw),
+                         lambda: ops.softmax_attention_rows(q1[:nd], kr, vr, bt, sl_d, posd, H, G, D, D, max_ctx=ctx,
+                                                            gate=gt[:nd], **kw)),
+        "window_ungated": (lambda: ops.softmax_attention_prefill(q1, kr, vr, bt, cu, cx, L, H, G, D, D, **kw),
+                           lambda: ops.softmax_attention_rows(q1[:nd], kr, vr, bt, sl_d, posd, H, G, D, D, max_ctx=ctx, **kw)),
+        "vivesun_chunked": (lambda: ops.softmax_attention_prefill(q1, kr, vr, bt, cu, cx, L, H, G, D, D, scale=sc, chunk=W, sink=0.0),
+                            lambda: ops.softmax_attention_rows(q1[:nd], kr, vr, bt, sl_d, posd, H, G, D, D, max_ctx=ctx,
+                                                               scale=sc, chunk=W, sink=0.0)),
+        "windowed_llama_layout": (lambda: ops.prefill_attention_paged(q1, kr, vt, bt, cu, cx, H, G, D, L, sc, window=W, impl=4),
+                                  lambda: ops.decode_attention(q1[:nd], kr, vt, bt, cxd, H, G, ctx, sc, ws=ws, window=W))}
+    out["attention"] = {}
+    for name, (fp, fd) in att.items():
+        t_p, t_d = _timed_gpu(fp, iters), _timed_gpu(fd, iters)
+        pr = nb * sum(i % W + 1 for i in range(L)) * H if name == "vivesun_chunked" else pairs
+        kb = nd * G * 2 * D * 2.0 * ((ctx - 1) % W + 1) if name == "vivesun_chunked" else kvb
+        out["attention"][name] = {"prefill_ms": round(t_p * 1e3, 3), "mfma_frac": round(4.0 * pr * D / t_p / PEAK_BF16, 4),
+                                  "decode_ms": round(t_d * 1e3, 4), "hbm_frac": round(kb / t_d / PEAK_HBM, 4)}
+    # ---- experts: T rows (prompts) and nd rows (single tokens), expert sum and residual step included on both sides
+    E, k, F = u["experts"], u["top"], u["eff"]
+    x = torch.randn(T, Hd, device=dev).to(bf)
+    router = torch.randn(E, Hd, device=dev) * Hd ** -0.5
+    w13 = (torch.randn(E, 2 * F, Hd, device=dev) * Hd ** -0.5).to(bf)
+    w2 = (torch.randn(E, Hd, F, device=dev) * F ** -0.5).to(bf)
+    rb = router.to(bf)
+    xs = torch.randn(T, Hd, device=dev)
+    xb, y1 = xs.to(bf), torch.randn(T, Hd, device=dev).to(bf)
+    wn = torch.ones(Hd, device=dev)
+    wbf = wn.to(bf)
+
+    def kev(n):
+        ids, wts = ops.moe_router(x[:n], router, k)
+        return ops.residual_glu_experts_(xs[:n], x[:n], ids, wts, w13, w2, wn, 1e-6, bf, 0.3)
+
+    out["experts"] = {}
+    for name, rows in (("prefill", T), ("decode", nd)):
+        fl, by = 6.0 * rows * k * Hd * F, min(E, rows * k) * Hd * F * 6.0
+        t_k = _timed_gpu(lambda: kev(rows), iters)
+        t_m = _timed_gpu(lambda: ops.add_rmsnorm(xb[:rows], ops.moe_ffn(x[:rows], rb, w13, w2, k), wbf, 1e-5), iters)
+        out["experts"][name] = {"kevelorn_ms": round(t_k * 1e3, 3), "mixtral_ms": round(t_m * 1e3, 3),
+                                "kevelorn_mfma_frac": round(fl / t_k / PEAK_BF16, 4), "mixtral_mfma_frac": round(fl / t_m / PEAK_BF16, 4),
+                                "kevelorn_weight_hbm_frac": round(by / t_k / PEAK_HBM, 4),
+                                "mixtral_weight_hbm_frac": round(by / t_m / PEAK_HBM, 4)}
+    del w13, w2
+    # ---- row kernels (prompt rows): bytes that must move over the time, against 8 TB/s
+    qkv = torch.randn(T, (H + 2 * G) * D, device=dev).to(bf)
+    slots = torch.arange(T, dtype=torch.int32, device=dev)
+    freq = ops.rotary_frequencies(D, 1e6, linear=4.0)[0].to(dev)
+    cs = ref.rope_cos_sin(L, D, 1e6).to(dev)
+    by_r = T * (2 * (H + G) * D + 2 * G * D) * 2.0       # q, k read + written, k and v pages written, v read
+    o = torch.randn(T, nv, device=dev)
+    gg = torch.randn(T, nv, device=dev).to(bf)
+    wd, wv = torch.ones(dv, device=dev), torch.ones(nv, device=dev)
+    y2, x0 = torch.randn(T, Hd, device=dev).to(bf), torch.randn(T, Hd, device=dev)
+    Fd = z["ffn"] // 8 * 8
+    gu = torch.randn(T, 2 * Fd, device=dev).to(bf)
+    row_kernels = {
+        # name: (call, bytes)
+        "rope_unit_interleaved_cache": (lambda: ops.rope_headnorm_cache_(qkv, posr, slots, kr, vr, H, G, D, D, freq, 1.0, D, 1e-6,
+                                                                         v_off=(H + G) * D, interleaved=True, unit=True), by_r),
+        "rope_cache": (lambda: ops.rope_cache_(qkv, posr, cs, slots, kr, vt, H, G, D), by_r),
+        "residual_step": (lambda: ops.residual_step_(xs, y1, wn, 1e-6, bf, 0.3), T * Hd * 12.0),
+        "residual_step_shared": (lambda: ops.residual_step_(xs, y1, wn, 1e-6, bf, 0.3, y2), T * Hd * 14.0),
+        "residual_step_pair": (lambda: ops.residual_step_(xs, y1, wn, 1e-6, bf, 0.15, y2, (wn, wn)), T * Hd * 14.0),
+        "residual_step_pass": (lambda: ops.residual_step_(xs, y1, wn, 1e-6, bf, 0.3, x0=x0, row=wn), T * Hd * 16.0),
+        "residual_add_rmsnorm": (lambda: ops.residual_add_rmsnorm_(xs, y1, wn, 1e-6, bf), T * Hd * 12.0),
+        "add_rmsnorm": (lambda: ops.add_rmsnorm(xb, y1, wbf, 1e-5), T * Hd * 8.0),
+        "whole_row_norm_sigmoid": (lambda: ops.group_rmsnorm(o, wv, 1, 1e-6, bf, gate=gg), T * nv * 8.0),
+        "head_norm_silu": (lambda: ops.group_rmsnorm(o, wd, H, 1e-6, bf, gate=gg, gate_act="silu"), T * nv * 8.0),
+        "whole_row_norm_sigmoid_64": (lambda: ops.group_rmsnorm(o[:nd], wv, 1, 1e-6, bf, gate=gg[:nd]), nd * nv * 8.0),
+        "head_norm_silu_64": (lambda: ops.group_rmsnorm(o[:nd], wd, H, 1e-6, bf, gate=gg[:nd], gate_act="silu"), nd * nv * 8.0),
+        "add_rmsnorm_64": (lambda: ops.add_rmsnorm(xb[:nd], y1[:nd], wbf, 1e-5), nd * Hd * 8.0),
+        "glu_gelu_tanh": (lambda: ops.glu_gelu_tanh(gu), T * Fd * 6.0),
+        "silu_mul": (lambda: ops.silu_mul(gu), T * Fd * 6.0)}
+    out["rows"] = {}
+    for name, (fn, by) in row_kernels.items():
+        t = _timed_gpu(fn, iters)
+        out["rows"][name] = {"ms": round(t * 1e3, 4), "hbm_frac": round(by / t / PEAK_HBM, 4)}
+    return out
+
+
 def run(args) -> None:
     names = [s for s in (args.design_sizes or "s,m,l").split(",") if s]
     models = [m for m in (getattr(args, "design_models", None) or "bidasun").split(",") if m]
@@ -722,7 +885,7 @@ def run(args) -> None:
     for n in names:
         z = dict(SIZES[n], lumepel=LUMEPEL[n])
         res[n] = {"shape": {k: v for k, v in z.items()}}
-        for kind in models + sorted({BASELINE_OF[m] for m in models}):
+        for kind in models + sorted({b for m in models for b in BASELINE_OF[m]} - set(models)):
             res[n][kind] = engine_rates(kind, z, max(1, args.steps), max(1, args.warmup))
             torch.cuda.empty_cache()
         if "bidasun" in models:
@@ -739,6 +902,9 @@ def run(args) -> None:
             torch.cuda.empty_cache()
         if "vivesun" in models:
             res[n]["vivesun_kernels"] = vivesun_kernel_times(z)
+            torch.cuda.empty_cache()
+        if "kevelorn" in models:
+            res[n]["kevelorn_kernels"] = kevelorn_kernel_times(z)
             torch.cuda.empty_cache()
         print(f"[designs] {n}: {json.dumps(res[n])}", flush=True)
     line = {"metric": "design_compare", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,

@@ -333,12 +333,10 @@ bool launch_residual_step_vec(float* x, const uint16_t* y, int64_t y_stride, con
 #define NGA_STEP(TPR, NV)                                                                                              \
   residual_step_bf16x4_kernel<TPR, NV, POST><<<dim3((unsigned)(TPR == 64 ? (T + 3) / 4 : T)), 256, 0, stream>>>(        \
       x, y, y_stride, w, nw, eps, H, T, out, inv, k)
-  if (T >= 4096 && H <= 4096) {      // rows enough to fill the chip with one wave each
+  if (T >= 4096 && H <= 1024) {      // rows enough to fill the chip with one wave each
     if (H <= 256) NGA_STEP(64, 1);
     else if (H <= 512) NGA_STEP(64, 2);
-    else if (H <= 1024) NGA_STEP(64, 4);
-    else if (H <= 2048) NGA_STEP(64, 8);
-    else NGA_STEP(64, 16);
+    else NGA_STEP(64, 4);
   } else {
     if (H <= 1024) NGA_STEP(256, 1);
     else if (H <= 2048) NGA_STEP(256, 2);
@@ -367,9 +365,7 @@ __global__ void __launch_bounds__(256) residual_step_kernel(const ResidualStepPa
       s2 += b * b;
     }
     r1 = 1.0f / sqrtf(block_sum(s1, red) / (float)H + P.eps);
-    __syncthreads();
     r2 = 1.0f / sqrtf(block_sum(s2, red) / (float)H + P.eps);
-    __syncthreads();
   }
   float ss = 0.f;
   for (int c = threadIdx.x; c < H; c += blockDim.x) {
@@ -522,12 +518,10 @@ void launch_residual_step_general(const ResidualStepParams& p, int64_t T, hipStr
 #define NGA_STEP(TPR, NV)                                                                                       \
   residual_step_general_bf16x4_kernel<TPR, NV, PAIR>                                                            \
       <<<dim3((unsigned)(TPR == 64 ? (T + 3) / 4 : T)), 256, 0, stream>>>(p, T)
-  if (T >= 4096 && p.H <= 4096) {      // rows enough to fill the chip with one wave each
+  if (T >= 4096 && p.H <= 1024) {      // rows enough to fill the chip with one wave each
     if (p.H <= 256) NGA_STEP(64, 1);
     else if (p.H <= 512) NGA_STEP(64, 2);
-    else if (p.H <= 1024) NGA_STEP(64, 4);
-    else if (p.H <= 2048) NGA_STEP(64, 8);
-    else NGA_STEP(64, 16);
+    else NGA_STEP(64, 4);
   } else {
     if (p.H <= 1024) NGA_STEP(256, 1);
     else if (p.H <= 2048) NGA_STEP(256, 2);
@@ -674,6 +668,54 @@ __global__ void __launch_bounds__(256) group_rmsnorm_bf16x4_kernel(uint16_t* __r
 #pragma unroll
     for (int q = 0; q < 4; ++q) o4[q] = f2bf(y[q]);
     *reinterpret_cast<u16x4*>(out + row * o_stride + (int64_t)hg * gs + c) = o4;
+  }
+}
+
+// the same for groups of more than 512 columns: a workgroup per (row, group), the group in registers (NV runs of
+// four elements per thread, up to 1024 NV columns), one read of x
+template <int NV>
+__global__ void __launch_bounds__(256) group_rmsnorm_wide_bf16x4_kernel(uint16_t* __restrict__ out, const float* __restrict__ x,
+                                                                        const float* __restrict__ w, int gs, float eps,
+                                                                        int groups, int w_full, const uint16_t* __restrict__ gate,
+                                                                        int64_t g_stride, int silu, int64_t o_stride) {
+  __shared__ float red[4];
+  const int64_t g = blockIdx.x;
+  const float* xr = x + g * gs;
+  const int64_t row = g / groups;
+  const int hg = (int)(g - row * groups);
+  const float* wr = w_full ? w + (int64_t)hg * gs : w;
+  const uint16_t* gr = gate ? gate + row * g_stride + (int64_t)hg * gs : nullptr;
+  uint16_t* orow = out + row * o_stride + (int64_t)hg * gs;
+  float4 v[NV];
+  u16x4 g4[NV];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * (threadIdx.x + 256 * i);
+    v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (c < gs) {
+      v[i] = *reinterpret_cast<const float4*>(xr + c);
+      if (gr) g4[i] = *reinterpret_cast<const u16x4*>(gr + c);
+    }
+    ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+  }
+  const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)gs + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * (threadIdx.x + 256 * i);
+    if (c >= gs) continue;
+    const float4 ww = *reinterpret_cast<const float4*>(wr + c);
+    float y[4] = {v[i].x * r * ww.x, v[i].y * r * ww.y, v[i].z * r * ww.z, v[i].w * r * ww.w};
+    u16x4 o4;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      if (gr) {
+        const float z = bf2f(g4[i][q]);
+        y[q] *= (silu ? z : 1.0f) * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+      }
+      o4[q] = f2bf(y[q]);
+    }
+    *reinterpret_cast<u16x4*>(orow + c) = o4;
   }
 }
 
@@ -1049,6 +1091,17 @@ void launch_group_rmsnorm(void* out, int64_t o_stride, const float* x, const flo
   if (ng == 0) return;
   if (!f32 && gs % 4 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0 && ((uintptr_t)out % 8) == 0 &&
       o_stride % 4 == 0 && (gate == nullptr || (g_stride % 4 == 0 && ((uintptr_t)gate % 8) == 0))) {
+    if (gs > 512 && gs <= 8192) {
+#define NGA_WIDE(NV)                                                                                              \
+  group_rmsnorm_wide_bf16x4_kernel<NV><<<dim3((unsigned)ng), 256, 0, stream>>>(                                   \
+      (uint16_t*)out, x, w, gs, eps, groups, w_full ? 1 : 0, (const uint16_t*)gate, g_stride, gate_silu ? 1 : 0, o_stride)
+      if (gs <= 1024) NGA_WIDE(1);
+      else if (gs <= 2048) NGA_WIDE(2);
+      else if (gs <= 4096) NGA_WIDE(4);
+      else NGA_WIDE(8);
+#undef NGA_WIDE
+      return;
+    }
     group_rmsnorm_bf16x4_kernel<<<dim3((unsigned)((ng + 7) / 8)), 256, 0, stream>>>(
         (uint16_t*)out, x, w, ng, gs, eps, groups, w_full ? 1 : 0, (const uint16_t*)gate, g_stride, gate_silu ? 1 : 0,
         o_stride);
