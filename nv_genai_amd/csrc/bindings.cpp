@@ -1927,12 +1927,12 @@ void linear_blocks(Tensor out, Tensor ws, Tensor q, Tensor k, Tensor v, c10::opt
   const bool f32 = act_f32(q);
   CHECK_F32(ws); CHECK_CONTIG(ws); CHECK_I32(cu);
   nga::LinearParams p = linear_params(out, q, k, v, z, vec, state, H, d, dv, inv_tau, q_scale, silu, slots, pos);
-  const int64_t n = slots.numel(), T = q.size(0), dt = nga::delta_key_tiles((int)d);
+  const int64_t n = slots.numel(), T = q.size(0);
   TORCH_CHECK(cu.numel() == n + 1 && max_q >= 1 && max_q <= T);
-  TORCH_CHECK(ws.numel() >= (T / 16 + n) * H * (33 * 16 * dt + 256) && (uintptr_t)ws.data_ptr() % 16 == 0,
-              "linear_blocks: workspace too small");
+  TORCH_CHECK(ws.numel() >= nga::linear_workspace(T, (int)n, (int)H, (int)d, (int)dv, (int)max_q) &&
+              (uintptr_t)ws.data_ptr() % 16 == 0, "linear_blocks: workspace too small");
   p.cu = cu.data_ptr<int32_t>();
-  nga::launch_linear_blocks(p, ws.data_ptr<float>(), (int)n, (int)max_q, f32, cur_stream(q));
+  nga::launch_linear_blocks(p, ws.data_ptr<float>(), T, (int)n, (int)max_q, f32, cur_stream(q));
 }
 
 void hgrn2_scan(Tensor out, Tensor proj, Tensor f_bias, Tensor lower, Tensor state, int64_t H, int64_t d, int64_t dv,
@@ -2033,6 +2033,9 @@ PYBIND11_MODULE(_C, m) {
   m.def("residual_step", checked("residual_step", &residual_step));
   m.def("linear_rows", checked("linear_rows", &linear_rows));
   m.def("linear_blocks", checked("linear_blocks", &linear_blocks));
+  m.def("linear_workspace", [](int64_t T, int64_t n, int64_t H, int64_t d, int64_t dv, int64_t max_q) {
+    return nga::linear_workspace(T, (int)n, (int)H, (int)d, (int)dv, (int)max_q);
+  });
   m.def("delta_rows", checked("delta_rows", &delta_rows));
   m.def("delta_blocks", checked("delta_blocks", &delta_blocks));
   m.def("delta_key_tiles", [](int64_t d) { return (int64_t)nga::delta_key_tiles((int)d); });

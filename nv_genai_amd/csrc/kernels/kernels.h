@@ -455,7 +455,9 @@ struct LinearParams {
   const int32_t* pos;        // [T]
 };
 void launch_linear_rows(const LinearParams& p, int n, bool f32, hipStream_t stream);
-void launch_linear_blocks(const LinearParams& p, float* ws, int n_seg, int max_q, bool f32, hipStream_t stream);
+// ws: linear_workspace(T, n_seg, ..) floats, 16-byte aligned; T: rows of the tensors
+int64_t linear_workspace(int64_t T, int n_seg, int H, int d, int dv, int max_q);
+void launch_linear_blocks(const LinearParams& p, float* ws, int64_t T, int n_seg, int max_q, bool f32, hipStream_t stream);
 
 int delta_key_tiles(int d);
 void launch_delta_rows(const DeltaParams& p, int n, bool f32, hipStream_t stream);

@@ -16,6 +16,9 @@
 //   R_t = q_t e^(c_t),  K'_s = k_s e^(c_E - c_s),  N_ts = sum_channels q_t k_s e^(c_t - c_s)  (s <= t)
 // so that the walk over the blocks of a segment is
 //   O = R S + N V,  S <- diag(e^(c_E)) S + K'^T V.
+// The state enters linearly, so a launch with too few waves for the chip walks the segments in parts: one pass
+// leaves what every part adds to the state and by how much it decays, a second one starts every part from the
+// sum of what came before it and writes the outputs.
 // No exponent above is positive. N of a constant decay takes its factor behind the product of q and k; N of
 // channel decays is (q e^(c_t)) . (k e^(-c_s)) as long as no channel of the block decays by more than e^-SAFE
 // (the factors stay far inside fp32), else the pairs of rows are summed one by one.
@@ -260,68 +263,108 @@ __global__ void __launch_bounds__(256) linear_prep_kernel(const LinearParams P, 
   wp[32 * D + 4 * ((n_s >> 2) * 16 + n_t) + (n_s & 3)] = n;
 }
 
-// One wave = 16 value columns of one head of one segment, over all its blocks. Up to 8 key tiles the
-// next block's operands are loaded into a second register set while the current one is used.
-template <typename T, int DT>
+// One wave = 16 value columns of one head of one segment (PASS 0), or of one of the n_split parts of its blocks
+// (PASS 1: the state each part adds, PASS 2: the outputs). Up to 8 key tiles the next block's operands are
+// loaded into a second register set while the current one is used.
+template <typename T, int DT, bool OUT>
 struct LinearRegs {
-  f32x4 r[DT], k[DT], p[DT], n;
+  f32x4 k[DT], p[DT], r[OUT ? DT : 1], n;
   T v[4];      // raw values (converted at their use: a conversion behind the load would wait for it)
 };
 
-template <typename T, int DT>
+template <typename T, int DT, int PASS>
 __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1))) linear_walk_kernel(
-    const LinearParams P, const float* __restrict__ ws) {
+    const LinearParams P, const float* __restrict__ ws, float* __restrict__ es, float* __restrict__ ps, int n_split) {
   constexpr int D = 16 * DT;
-  const int h = blockIdx.x % P.H, b = blockIdx.x / P.H, tile = blockIdx.y;
+  constexpr bool OUT = PASS != 1;
+  const int h = blockIdx.x % P.H, b = blockIdx.x / P.H, tile = blockIdx.y, part = PASS ? blockIdx.z : 0;
   const int lane = threadIdx.x, l15 = lane & 15, hh = lane >> 4;
   const int t0 = P.cu[b], t1 = P.cu[b + 1];
   if (t1 <= t0) return;
+  const int nblk = (t1 - t0 + 15) / 16;
+  const int per = PASS ? (nblk + n_split - 1) / n_split : nblk;
+  const int b0 = part * per, b1 = min(nblk, b0 + per);
+  if (b0 >= b1) return;
+  if (PASS == 1 && part > 0 && b1 == nblk) return;       // nothing follows the last part
   const int slot = P.slots[b];
   const bool fresh = slot < 0 || P.pos[t0] == 0;
   const int d = P.d, dv = P.dv, col = tile * 16 + l15;
   const bool colok = col < dv;
   float* sp = slot >= 0 ? P.state + ((int64_t)slot * P.H + h) * (int64_t)d * dv + col : nullptr;
-  f32x4 S[DT];
+  // states of the parts in lane order: entry 0 the segment's first state, entry c > 0 what part c - 1 leaves (part 0
+  // from the first state, the others from zero); ps: the parts' whole decays
+  float* ep = PASS ? es + (((int64_t)b * P.H + h) * gridDim.y + tile) * n_split * (int64_t)(16 * D) + 4 * lane : nullptr;
+  float* pp = PASS ? ps + ((int64_t)b * P.H + h) * n_split * (int64_t)D + 4 * hh : nullptr;
+  f32x4 S[DT], pt[PASS == 1 ? DT : 1];
+  if (PASS == 2) {
+    const float* e = ep + (part ? 16 * D : 0);
 #pragma unroll
-  for (int i = 0; i < DT; ++i)
+    for (int i = 0; i < DT; ++i) S[i] = *reinterpret_cast<const f32x4*>(e + 256 * i);
+    for (int c = 1; c < part; ++c) {
+      e += 16 * D;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int ch = 16 * i + 4 * hh + r;
-      S[i][r] = (!fresh && colok && ch < d) ? sp[(int64_t)ch * dv] : 0.f;
+      for (int i = 0; i < DT; ++i)
+        S[i] = S[i] * *reinterpret_cast<const f32x4*>(pp + (int64_t)c * D + 16 * i) + *reinterpret_cast<const f32x4*>(e + 256 * i);
     }
+  } else {
+    const bool load = !fresh && part == 0 && colok;
+#pragma unroll
+    for (int i = 0; i < DT; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int ch = 16 * i + 4 * hh + r;
+        S[i][r] = (load && ch < d) ? sp[(int64_t)ch * dv] : 0.f;
+      }
+    if (PASS == 1) {
+      if (part == 0) {
+#pragma unroll
+        for (int i = 0; i < DT; ++i) *reinterpret_cast<f32x4*>(ep + 256 * i) = S[i];
+        if (b1 == nblk) return;
+      }
+#pragma unroll
+      for (int i = 0; i < DT; ++i) pt[i] = (f32x4)(1.f);
+    }
+  }
   const int64_t ent = (int64_t)P.H * (33 * D + 256);       // one block of all heads
   const float* wp = ws + ((int64_t)((t0 - P.cu[0]) / 16 + b) * P.H + h) * (int64_t)(33 * D + 256);
   // no branch around a load (each would wait for all loads in flight): rows past the segment read its
   // last row - the block operands are zero there -, columns past dv the first one, and are not stored
   const T* vp = (const T*)P.v + (int64_t)t0 * P.vs + h * dv + (colok ? col : 0);
   const bool act = P.silu;
-  auto load = [&](LinearRegs<T, DT>& B, int blk) {
+  auto load = [&](LinearRegs<T, DT, OUT>& B, int blk) {
     const float* w = wp + blk * ent;
+    if constexpr (OUT) {
 #pragma unroll
-    for (int i = 0; i < DT; ++i) B.r[i] = *reinterpret_cast<const f32x4*>(w + (i * 64 + lane) * 4);
+      for (int i = 0; i < DT; ++i) B.r[i] = *reinterpret_cast<const f32x4*>(w + (i * 64 + lane) * 4);
+      B.n = *reinterpret_cast<const f32x4*>(w + 32 * D + 4 * lane);
+    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = min(blk * 16 + 4 * hh + r, t1 - t0 - 1);
       B.v[r] = vp[(int64_t)t * P.vs];
     }
-    B.n = *reinterpret_cast<const f32x4*>(w + 32 * D + 4 * lane);
 #pragma unroll
     for (int i = 0; i < DT; ++i) {
       B.k[i] = *reinterpret_cast<const f32x4*>(w + 16 * D + (i * 64 + lane) * 4);
       B.p[i] = *reinterpret_cast<const f32x4*>(w + 32 * D + 256 + 16 * i + 4 * hh);
     }
   };
-  auto step = [&](const LinearRegs<T, DT>& B, int blk) {
+  auto step = [&](const LinearRegs<T, DT, OUT>& B, int blk) {
     f32x4 o = (f32x4)(0.f), o2 = (f32x4)(0.f);
+    if constexpr (OUT) {
 #pragma unroll
-    for (int i = 0; i < DT; ++i) {
-      o = mfma32(B.r[i][0], S[i][0], o);
-      o2 = mfma32(B.r[i][1], S[i][1], o2);
-      o = mfma32(B.r[i][2], S[i][2], o);
-      o2 = mfma32(B.r[i][3], S[i][3], o2);
+      for (int i = 0; i < DT; ++i) {
+        o = mfma32(B.r[i][0], S[i][0], o);
+        o2 = mfma32(B.r[i][1], S[i][1], o2);
+        o = mfma32(B.r[i][2], S[i][2], o);
+        o2 = mfma32(B.r[i][3], S[i][3], o2);
+      }
     }
 #pragma unroll
-    for (int i = 0; i < DT; ++i) S[i] *= B.p[i];
+    for (int i = 0; i < DT; ++i) {
+      S[i] *= B.p[i];
+      if constexpr (PASS == 1) pt[i] *= B.p[i];
+    }
     float v[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -330,53 +373,64 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1)))
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      if (r & 1) o2 = mfma32(B.n[r], v[r], o2);
-      else o = mfma32(B.n[r], v[r], o);
+      if constexpr (OUT) {
+        if (r & 1) o2 = mfma32(B.n[r], v[r], o2);
+        else o = mfma32(B.n[r], v[r], o);
+      }
 #pragma unroll
       for (int i = 0; i < DT; ++i) S[i] = mfma32(B.k[i][r], v[r], S[i]);
     }
-    o += o2;
     if constexpr (DT <= 8) {
       // the next block's loads (issued in front of this step in program order) between the MFMAs: a
       // wave issues in order, and loads in a row would leave the matrix pipe idle
 #pragma unroll
-      for (int g = 0; g < 3 * DT + 5; ++g) {
+      for (int g = 0; g < (OUT ? 3 * DT + 5 : 2 * DT + 4); ++g) {
         __builtin_amdgcn_sched_group_barrier(0x008, 2, 0);   // MFMA
         __builtin_amdgcn_sched_group_barrier(0x020, 1, 0);   // VMEM read
       }
     }
-    float* op = P.out + (int64_t)(t0 + blk * 16) * P.H * dv + h * dv + col;
-    if (blk * 16 + 16 <= t1 - t0) {
-      if (colok) {
+    if constexpr (OUT) {
+      o += o2;
+      float* op = P.out + (int64_t)(t0 + blk * 16) * P.H * dv + h * dv + col;
+      if (blk * 16 + 16 <= t1 - t0) {
+        if (colok) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) op[(int64_t)(4 * hh + r) * P.H * dv] = o[r];
+          for (int r = 0; r < 4; ++r) op[(int64_t)(4 * hh + r) * P.H * dv] = o[r];
+        }
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (colok && blk * 16 + 4 * hh + r < t1 - t0) op[(int64_t)(4 * hh + r) * P.H * dv] = o[r];
       }
-    } else {
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        if (colok && blk * 16 + 4 * hh + r < t1 - t0) op[(int64_t)(4 * hh + r) * P.H * dv] = o[r];
     }
   };
-  const int nblk = (t1 - t0 + 15) / 16;
   if constexpr (DT <= 8) {
-    LinearRegs<T, DT> A, B;
-    load(A, 0);
-    int blk = 0;
-    for (; blk + 1 < nblk; blk += 2) {
+    LinearRegs<T, DT, OUT> A, B;
+    load(A, b0);
+    int blk = b0;
+    for (; blk + 1 < b1; blk += 2) {
       load(B, blk + 1);
       step(A, blk);
-      load(A, min(blk + 2, nblk - 1));
+      load(A, min(blk + 2, b1 - 1));
       step(B, blk + 1);
     }
-    if (blk < nblk) step(A, blk);
+    if (blk < b1) step(A, blk);
   } else {
-    LinearRegs<T, DT> A;
-    for (int blk = 0; blk < nblk; ++blk) {
+    LinearRegs<T, DT, OUT> A;
+    for (int blk = b0; blk < b1; ++blk) {
       load(A, blk);
       step(A, blk);
     }
   }
-  if (sp && colok) {
+  if (PASS == 1) {
+#pragma unroll
+    for (int i = 0; i < DT; ++i) {
+      *reinterpret_cast<f32x4*>(ep + (int64_t)(part + 1) * (16 * D) + 256 * i) = S[i];
+      if (tile == 0 && l15 == 0) *reinterpret_cast<f32x4*>(pp + (int64_t)part * D + 16 * i) = pt[i];
+    }
+    return;
+  }
+  if (sp && colok && b1 == nblk) {
 #pragma unroll
     for (int i = 0; i < DT; ++i)
 #pragma unroll
@@ -413,20 +467,39 @@ void launch_rows_t(const LinearParams& P, int n, hipStream_t stream) {
     launch_rows_nr<T, CH, 16, 1>(P, n, stream);
 }
 
+// parts a segment's blocks are walked in: enough waves for every SIMD (256 CUs x 4), at least PART_ROWS rows each
+constexpr int PART_ROWS = 128, SIMDS = 1024;
+int linear_parts(int waves, int max_q) {
+  const int p = SIMDS / (waves > 0 ? waves : 1), q = max_q / PART_ROWS;
+  const int n = p < q ? p : q;
+  return n < 2 ? 1 : (n > 32 ? 32 : n);
+}
+
 template <typename T, int DT>
-void launch_blocks_dt(const LinearParams& P, float* ws, int n_seg, int max_q, hipStream_t stream) {
+void launch_blocks_dt(const LinearParams& P, float* ws, int64_t entries, int n_seg, int max_q, hipStream_t stream) {
   const dim3 grid((unsigned)((max_q + 15) / 16), (unsigned)P.H, (unsigned)n_seg);
   if (P.z)
     linear_prep_kernel<T, true, DT><<<grid, 256, 0, stream>>>(P, ws);
   else
     linear_prep_kernel<T, false, DT><<<grid, 256, 0, stream>>>(P, ws);
-  linear_walk_kernel<T, DT><<<dim3((unsigned)(P.H * n_seg), (unsigned)((P.dv + 15) / 16)), 64, 0, stream>>>(P, ws);
+  const int tiles = (P.dv + 15) / 16, parts = linear_parts(n_seg * P.H * tiles, max_q);
+  dim3 walk((unsigned)(P.H * n_seg), (unsigned)tiles);
+  if (parts == 1) {
+    linear_walk_kernel<T, DT, 0><<<walk, 64, 0, stream>>>(P, ws, nullptr, nullptr, 1);
+    return;
+  }
+  float* es = ws + entries * P.H * (33 * 16 * DT + 256);
+  float* ps = es + (int64_t)n_seg * P.H * tiles * parts * (256 * DT);
+  walk.z = (unsigned)(parts - 1);
+  linear_walk_kernel<T, DT, 1><<<walk, 64, 0, stream>>>(P, ws, es, ps, parts);
+  walk.z = (unsigned)parts;
+  linear_walk_kernel<T, DT, 2><<<walk, 64, 0, stream>>>(P, ws, es, ps, parts);
 }
 
 template <typename T>
-bool launch_blocks_t(const LinearParams& P, float* ws, int n_seg, int max_q, hipStream_t stream) {
+bool launch_blocks_t(const LinearParams& P, float* ws, int64_t entries, int n_seg, int max_q, hipStream_t stream) {
   switch (delta_key_tiles(P.d)) {
-#define NGA_LINEAR(N) case N: launch_blocks_dt<T, N>(P, ws, n_seg, max_q, stream); return true;
+#define NGA_LINEAR(N) case N: launch_blocks_dt<T, N>(P, ws, entries, n_seg, max_q, stream); return true;
     NGA_LINEAR(1) NGA_LINEAR(2) NGA_LINEAR(3) NGA_LINEAR(4) NGA_LINEAR(6) NGA_LINEAR(8) NGA_LINEAR(12) NGA_LINEAR(16)
 #undef NGA_LINEAR
     default: return false;
@@ -443,10 +516,19 @@ void launch_linear_rows(const LinearParams& P, int n, bool f32, hipStream_t stre
     P.z ? launch_rows_t<uint16_t, true>(P, n, stream) : launch_rows_t<uint16_t, false>(P, n, stream);
 }
 
-// ws: (rows / 16 + n_seg) * H * (33 * 16 * delta_key_tiles(d) + 256) floats, 16-byte aligned
-void launch_linear_blocks(const LinearParams& P, float* ws, int n_seg, int max_q, bool f32, hipStream_t stream) {
+// Floats of the workspace of a launch over T rows: block operands, then, when the segments are walked in parts,
+// the parts' states and decays.
+int64_t linear_workspace(int64_t T, int n_seg, int H, int d, int dv, int max_q) {
+  const int64_t D = 16 * delta_key_tiles(d), tiles = (dv + 15) / 16;
+  const int64_t parts = linear_parts((int)(n_seg * H * tiles), max_q);
+  return (T / 16 + n_seg) * H * (33 * D + 256) + (parts > 1 ? n_seg * H * parts * (tiles * 16 * D + D) : 0);
+}
+
+void launch_linear_blocks(const LinearParams& P, float* ws, int64_t T, int n_seg, int max_q, bool f32, hipStream_t stream) {
   if (n_seg == 0 || max_q == 0) return;
-  if (!(f32 ? launch_blocks_t<float>(P, ws, n_seg, max_q, stream) : launch_blocks_t<uint16_t>(P, ws, n_seg, max_q, stream)))
+  const int64_t entries = T / 16 + n_seg;
+  if (!(f32 ? launch_blocks_t<float>(P, ws, entries, n_seg, max_q, stream)
+            : launch_blocks_t<uint16_t>(P, ws, entries, n_seg, max_q, stream)))
     abort();   // the binding checks d
 }
 

@@ -1007,9 +1007,6 @@ def _delta(out, q, k, v, w, b, w_vec, b_vec, state, mode, H, G, d, dv, decay, cu
 
 
 # ------------------------------------------------------------------------- diagonal linear recurrences, scaled steps
-LINEAR_CHUNK = 16       # rows per block of the matrix form
-
-
 def linear_scan(q, k, v, state, H: int, d: int, dv: int, cu, slots, pos, z=None, z_bias=None, tau: float = 1.0,
                 log_decay=None, q_scale: float = 1.0, silu: bool = False, n_single: int = 0, max_q: int = 0) -> torch.Tensor:
     """Linear attention with a diagonal decay over a step's rows: q, k rows [T, H*d], v rows [T, H*dv] (any row
@@ -1022,7 +1019,8 @@ def linear_scan(q, k, v, state, H: int, d: int, dv: int, cu, slots, pos, z=None,
     nothing is read or kept. Returns the fp32 outputs [T, H*dv].
 
     GPU: single rows (``cu`` None, or the first ``n_single`` segments) take the row kernel; portions (at
-    most ``max_q`` rows each) the matrix form (csrc/kernels/linear_scan.hip)."""
+    most ``max_q`` rows each) the matrix form in blocks of 16 rows, long ones in parts side by side when there
+    are few (csrc/kernels/linear_scan.hip)."""
     if (z is None) == (log_decay is None) or (z is not None and z_bias is None):
         raise ValueError("linear_scan: a decay per channel (z, z_bias) or a constant one per head (log_decay)")
     if not tau > 0:
@@ -1040,8 +1038,7 @@ def linear_scan(q, k, v, state, H: int, d: int, dv: int, cu, slots, pos, z=None,
     if ns < n:
         if max_q < 1:
             raise ValueError("linear_scan of portions needs max_q, the rows of the longest one")
-        D = 16 * int(C.delta_key_tiles(d))
-        ws = torch.empty((T // LINEAR_CHUNK + n - ns) * H * (33 * D + 256), dtype=torch.float32, device=q.device)
+        ws = torch.empty(int(C.linear_workspace(T, n - ns, H, d, dv, int(max_q))), dtype=torch.float32, device=q.device)
         C.linear_blocks(out, ws, q, k, v, z, *args, cu[ns:], slots[ns:], pos, int(max_q))
     return out
 
