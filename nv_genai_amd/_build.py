@@ -84,9 +84,11 @@ def _run(cmd):
 # AGPR->VGPR once per key tile (32 v_accvgpr_read per tile). VGPR form removes the copies
 # and lowers the register count (160+44 -> 149, 2 -> 3 waves/SIMD): 735 -> 658 us on 27
 # sequences x 1200 tokens. The same flag made decode attention slower (296 -> 335 us at
-# 256 x 1400, more resident waves contending for HBM), so it is per file.
+# 256 x 1400, more resident waves contending for HBM), so it is per file. The walk of the
+# linear scan scales its state with VALU ops once per block of rows.
 PER_FILE_FLAGS = {
     "attention_prefill": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
+    "linear_scan": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
 }
 
 

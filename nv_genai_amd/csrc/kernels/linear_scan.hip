@@ -272,7 +272,7 @@ struct LinearRegs {
   T v[4];      // raw values (converted at their use: a conversion behind the load would wait for it)
 };
 
-template <typename T, int DT, int PASS>
+template <typename T, int DT, int PASS, bool SILU>
 __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1))) linear_walk_kernel(
     const LinearParams P, const float* __restrict__ ws, float* __restrict__ es, float* __restrict__ ps, int n_split) {
   constexpr int D = 16 * DT;
@@ -330,7 +330,6 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1)))
   // no branch around a load (each would wait for all loads in flight): rows past the segment read its
   // last row - the block operands are zero there -, columns past dv the first one, and are not stored
   const T* vp = (const T*)P.v + (int64_t)t0 * P.vs + h * dv + (colok ? col : 0);
-  const bool act = P.silu;
   auto load = [&](LinearRegs<T, DT, OUT>& B, int blk) {
     const float* w = wp + blk * ent;
     if constexpr (OUT) {
@@ -369,7 +368,7 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 1)))
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       v[r] = ldf(&B.v[r]);
-      if (act) v[r] = silu_<T>(v[r]);
+      if constexpr (SILU) v[r] = silu_<T>(v[r]);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -467,12 +466,29 @@ void launch_rows_t(const LinearParams& P, int n, hipStream_t stream) {
     launch_rows_nr<T, CH, 16, 1>(P, n, stream);
 }
 
-// parts a segment's blocks are walked in: enough waves for every SIMD (256 CUs x 4), at least PART_ROWS rows each
+// parts a segment's blocks are walked in: enough waves for every SIMD (256 CUs x 4), at least PART_ROWS rows each;
+// fewer than four do not pay for the second pass (measured)
 constexpr int PART_ROWS = 128, SIMDS = 1024;
 int linear_parts(int waves, int max_q) {
   const int p = SIMDS / (waves > 0 ? waves : 1), q = max_q / PART_ROWS;
   const int n = p < q ? p : q;
-  return n < 2 ? 1 : (n > 32 ? 32 : n);
+  return n < 4 ? 1 : (n > 32 ? 32 : n);
+}
+
+template <typename T, int DT, bool SILU>
+void launch_walk(const LinearParams& P, float* ws, int64_t entries, int n_seg, int max_q, hipStream_t stream) {
+  const int tiles = (P.dv + 15) / 16, parts = linear_parts(n_seg * P.H * tiles, max_q);
+  dim3 walk((unsigned)(P.H * n_seg), (unsigned)tiles);
+  if (parts == 1) {
+    linear_walk_kernel<T, DT, 0, SILU><<<walk, 64, 0, stream>>>(P, ws, nullptr, nullptr, 1);
+    return;
+  }
+  float* es = ws + entries * P.H * (33 * 16 * DT + 256);
+  float* ps = es + (int64_t)n_seg * P.H * tiles * parts * (256 * DT);
+  walk.z = (unsigned)(parts - 1);
+  linear_walk_kernel<T, DT, 1, SILU><<<walk, 64, 0, stream>>>(P, ws, es, ps, parts);
+  walk.z = (unsigned)parts;
+  linear_walk_kernel<T, DT, 2, SILU><<<walk, 64, 0, stream>>>(P, ws, es, ps, parts);
 }
 
 template <typename T, int DT>
@@ -482,18 +498,8 @@ void launch_blocks_dt(const LinearParams& P, float* ws, int64_t entries, int n_s
     linear_prep_kernel<T, true, DT><<<grid, 256, 0, stream>>>(P, ws);
   else
     linear_prep_kernel<T, false, DT><<<grid, 256, 0, stream>>>(P, ws);
-  const int tiles = (P.dv + 15) / 16, parts = linear_parts(n_seg * P.H * tiles, max_q);
-  dim3 walk((unsigned)(P.H * n_seg), (unsigned)tiles);
-  if (parts == 1) {
-    linear_walk_kernel<T, DT, 0><<<walk, 64, 0, stream>>>(P, ws, nullptr, nullptr, 1);
-    return;
-  }
-  float* es = ws + entries * P.H * (33 * 16 * DT + 256);
-  float* ps = es + (int64_t)n_seg * P.H * tiles * parts * (256 * DT);
-  walk.z = (unsigned)(parts - 1);
-  linear_walk_kernel<T, DT, 1><<<walk, 64, 0, stream>>>(P, ws, es, ps, parts);
-  walk.z = (unsigned)parts;
-  linear_walk_kernel<T, DT, 2><<<walk, 64, 0, stream>>>(P, ws, es, ps, parts);
+  P.silu ? launch_walk<T, DT, true>(P, ws, entries, n_seg, max_q, stream)
+         : launch_walk<T, DT, false>(P, ws, entries, n_seg, max_q, stream);
 }
 
 template <typename T>
